@@ -38,7 +38,8 @@ from .pool import PAGE_TOKENS, CacheFull, CacheMisuse, FreeList, PageTable, page
 # host bookkeeping up to date, without making the host wait for the device); ``on_open(slot)``; ``nbytes()``;
 # ``attach(layer_cache, entry)``, which hangs what the part is to see on the entry's ``LayerCache`` under a field of
 # the need's choosing (the shipped ones use ``kv``, ``rows[name]`` and ``states[name]``).  Storage in pages derives
-# from ``PagedGroup``, which reads one thing of its need: ``window`` (absent or None: every position is kept).
+# from ``PagedGroup``, which reads two things of its need: ``window`` (absent or None: every position is kept) and
+# ``chunked`` (absent: false; the window is a chunk of positions that only queries of the same chunk read).
 
 @dataclass(frozen=True)
 class KVNeed:
@@ -51,6 +52,8 @@ class KVNeed:
     # its own) says so; None: as many value heads as key heads, of the keys' size
     value_heads: int | None = None
     value_dim: int | None = None
+    # a query reads the positions of its own chunk of ``window`` positions (counted from the sequence's start) only
+    chunked: bool = False
 
     def make_group(self, n_entries, n_pages, n_slots, max_pages_per_slot, dtype, device):
         return KVGroup(self, n_entries, n_pages, n_slots, max_pages_per_slot, dtype, device)
@@ -87,7 +90,7 @@ class PagedGroup:
 
     def __init__(self, need, n_entries: int, n_pages: int, n_slots: int, max_pages_per_slot: int, device):
         self.need, self.n_entries, self.n_pages = need, n_entries, n_pages
-        self.table = PageTable(n_pages, n_slots, max_pages_per_slot, getattr(need, "window", None))
+        self.table = PageTable(n_pages, n_slots, max_pages_per_slot, getattr(need, "window", None), getattr(need, "chunked", False))
         self.pad_page = n_pages
         self.table_host = torch.full((n_slots + 1, max_pages_per_slot), self.pad_page, dtype=torch.int32)
         self.table_dev = self.table_host.to(device)

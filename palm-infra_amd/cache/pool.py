@@ -78,11 +78,15 @@ class PageTable:
 
     ``window``: if set, only the last ``window`` positions before a query are ever read, so pages
     that lie wholly below ``length - window`` are given back as the sequence grows (their entries in
-    the slot's list become -1)."""
+    the slot's list become -1).  ``chunked``: a query only ever reads positions of its own chunk of ``window``
+    positions, so what lies wholly below the next query's chunk is given back."""
 
-    def __init__(self, n_pages: int, n_slots: int, max_pages_per_slot: int, window: int | None = None):
+    def __init__(self, n_pages: int, n_slots: int, max_pages_per_slot: int, window: int | None = None, chunked: bool = False):
         self.pages = FreeList(n_pages, "page")
         self.n_slots, self.max_pages_per_slot, self.window = n_slots, max_pages_per_slot, window
+        if chunked and not window:
+            raise ValueError("storage by chunks needs their size")
+        self.chunked = bool(chunked)
         self.slot_pages: list[list[int]] = [[] for _ in range(n_slots)]
         self.dirty: set[int] = set()  # slots whose device copy of the list is stale
 
@@ -104,7 +108,8 @@ class PageTable:
         """After a step: give back pages no later query can read (windowed groups only)."""
         if self.window is None:
             return
-        first_needed = max(0, length - self.window + 1)  # the next query sits at position `length`
+        # the next query sits at position `length`
+        first_needed = length - length % self.window if self.chunked else max(0, length - self.window + 1)
         have = self.slot_pages[slot]
         for j in range(min(first_needed // PAGE_TOKENS, len(have))):
             if have[j] >= 0:

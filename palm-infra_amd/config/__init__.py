@@ -7,8 +7,9 @@ from .sebesun import SebesunConfig
 from .pazilorn import PazilornConfig
 from .matalix import MatalixConfig
 from .biguzen import BiguzenConfig
+from .vovalix import VovalixConfig
 
 __all__ = ["ConfigError", "config_class_for", "config_from_dict", "config_from_dir", "config_source", "preset_dict",
            "preset_names", "register_architecture",
            "registered_architectures", "LayerCall", "ModelSpec", "PartSpec", "Stored", "TensorRef", "joined", "tensor",
-           "Qwen3Config", "SebesunConfig", "PazilornConfig", "MatalixConfig", "BiguzenConfig"]
+           "Qwen3Config", "SebesunConfig", "PazilornConfig", "MatalixConfig", "BiguzenConfig", "VovalixConfig"]

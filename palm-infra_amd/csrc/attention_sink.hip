@@ -1,13 +1,14 @@
 // Causal grouped-query softmax attention over the paged cache with the options that the plain attention kernels do not
 // have: a key size and a value size of their own, an RMS norm over the whole q projection and the whole k projection
-// (or per head, or none), biases on q, k and v, a rotation of the first `rot` dimensions of each head, a sliding
-// window, a sink (a key of a fixed score without a value: it only adds exp(score) to the softmax's denominator), and an
+// (or per head with or without a weight, or none), biases on q, k and v, a rotation of the first `rot` dimensions of each head, a sliding
+// window or chunks of positions that see only themselves, a distance bias (a slope per head), a sink (a key of a fixed score without a value: it only adds exp(score) to the softmax's denominator), and an
 // elementwise sigmoid gate on the heads' outputs (or one gate value for each head).  The sink's score is one number for
 // all heads or a learned one for each.  Between the bias and the norm q, k and v may go through a short causal convolution
 // over time, a channel at a time: y_t = sum_j w[c][j] u_(t - taps + 1 + j) with zeros before the sequence's start; the last
 // taps - 1 inputs u of each sequence are kept as state.  The rotation pairs dimension i with i + rot/2, or 2i with 2i + 1.
 //
-//   p_j = exp(s_j) / (exp(sink) + sum_i exp(s_i)),   s_j = scale * q . k_j,   max(0, pos - window + 1) <= j <= pos
+//   p_j = exp(s_j) / (exp(sink) + sum_i exp(s_i)),   s_j = scale * q . k_j - slope * (pos - j),   low(pos) <= j <= pos
+//   low(pos) = max(0, pos - window + 1), or with `chunked` the first position of pos's chunk of `window` positions
 //   out = (sum_j p_j v_j) * sigmoid(gate)
 //
 // K is [pages, kv_heads, 64, dim]; V is kept transposed, [pages, kv_heads, vdim, 64].
@@ -93,7 +94,7 @@ __global__ __launch_bounds__(1024) void sink_qkv_store_kernel(
         const float* w = nullptr;
         if (norm_mode == SK_NORM_PROJECTION) w = (is_q ? q_w : k_w) + (size_t)hh * dim;
         if (norm_mode == SK_NORM_HEAD) {
-            w = is_q ? q_w : k_w;
+            w = is_q ? q_w : k_w;                              // (null: no weight)
             float ss = 0.f;
             for (int d = lane; d < dim; d += WAVE) { const float v = value(col0 + d, ch0 + d, b ? b + d : nullptr); ss += v * v; }
             inv = 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps);
@@ -175,7 +176,7 @@ PALM_API int palm_sink_qkv_store(hipStream_t stream, const void* rows, int dtype
     PALM_CHECK(n_tokens >= 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0, "sink_qkv_store: tokens=%d heads=%d kv=%d dim=%d vdim=%d",
                n_tokens, heads, kv_heads, dim, vdim);
     PALM_CHECK(norm_mode >= SK_NORM_NONE && norm_mode <= SK_NORM_HEAD, "sink_qkv_store: norm mode %d", norm_mode);
-    PALM_CHECK(norm_mode == SK_NORM_NONE || (q_w && k_w), "sink_qkv_store: a norm needs its weights");
+    PALM_CHECK(norm_mode != SK_NORM_PROJECTION || (q_w && k_w), "sink_qkv_store: a norm over the projections needs its weights");
     PALM_CHECK(rot >= 0 && rot <= dim && rot % 2 == 0, "sink_qkv_store: %d rotated dimensions of %d", rot, dim);
     PALM_CHECK(rot == 0 || (cos_t && sin_t), "sink_qkv_store: a rotation needs its cos and sin rows");
     PALM_CHECK(!write_cache || (k_cache && v_cache && block_table && tok_slot && max_pages > 0), "sink_qkv_store: writing needs cache, pages and slots");
@@ -234,9 +235,9 @@ template <typename T, int MAXQ, int NV>
 __global__ __launch_bounds__(SK_WAVES * WAVE) void sink_attention_kernel(
     const T* __restrict__ q, const T* __restrict__ k_cache, const T* __restrict__ v_cache, const int* __restrict__ block_table,
     int max_pages, const int* __restrict__ seq_slot, const int* __restrict__ seq_start, const int* __restrict__ seq_new,
-    const int* __restrict__ cu_new, int heads, int kv_heads, int dim, int vdim, float scale, int window, int has_sink,
-    float sink_score, const float* __restrict__ sink_scores, const T* __restrict__ gate, int gate_stride, int gate_per_head, int n_slices,
-    float* __restrict__ work, T* __restrict__ out) {
+    const int* __restrict__ cu_new, int heads, int kv_heads, int dim, int vdim, float scale, int window, int chunked,
+    const float* __restrict__ slopes, int has_sink, float sink_score, const float* __restrict__ sink_scores, const T* __restrict__ gate,
+    int gate_stride, int gate_per_head, int n_slices, float* __restrict__ work, T* __restrict__ out) {
     __shared__ float q_s[MAXQ][SK_MAX_DIM];
     __shared__ float m_s[SK_WAVES][MAXQ], l_s[SK_WAVES][MAXQ];
     __shared__ float acc_s[SK_WAVES][MAXQ][SK_MAX_DIM];
@@ -251,7 +252,7 @@ __global__ __launch_bounds__(SK_WAVES * WAVE) void sink_attention_kernel(
     const int nq = min(MAXQ, per_kv - chunk * MAXQ);
     const int t = cu_new[b] + qi;
     const int pos = seq_start[b] + qi;
-    const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+    const int lo = window <= 0 ? 0 : chunked ? pos - pos % window : max(0, pos - window + 1);
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
     const int* pages = block_table + (size_t)seq_slot[b] * max_pages;
 
@@ -261,9 +262,10 @@ __global__ __launch_bounds__(SK_WAVES * WAVE) void sink_attention_kernel(
     }
     __syncthreads();
 
-    float m[MAXQ], l[MAXQ], acc[MAXQ][NV];
+    float m[MAXQ], l[MAXQ], acc[MAXQ][NV], slope[MAXQ];
 #pragma unroll
     for (int qh = 0; qh < MAXQ; ++qh) {
+        slope[qh] = slopes ? slopes[min(h0 + qh, heads - 1)] : 0.f;
         const bool sink_here = has_sink && slice == 0 && wave == 0;
         // one score for all heads, or a learned one for each
         m[qh] = sink_here ? (sink_scores ? sink_scores[min(h0 + qh, heads - 1)] : sink_score) : -INFINITY;
@@ -346,7 +348,7 @@ __global__ __launch_bounds__(SK_WAVES * WAVE) void sink_attention_kernel(
         // the page's maxima of all heads together: every step's exchanges between lanes are under way at once
         float p[MAXQ], top[MAXQ];
 #pragma unroll
-        for (int qh = 0; qh < MAXQ; ++qh) top[qh] = s[qh] = seen ? s[qh] : -INFINITY;
+        for (int qh = 0; qh < MAXQ; ++qh) top[qh] = s[qh] = seen ? fmaf(-slope[qh], (float)(pos - j), s[qh]) : -INFINITY;
 #pragma unroll
         for (int off = WAVE / 2; off > 0; off >>= 1) {
             float other[MAXQ];
@@ -486,13 +488,13 @@ __global__ __launch_bounds__(WAVE) void sink_attention_merge_kernel(const float*
     }
 }
 
-// q [n, heads, dim]; gate: null, or the first gate value of token 0 (rows `gate_stride` elements apart, heads * vdim
+// q [n, heads, dim]; slopes: null, or the distance bias's slope for each head; gate: null, or the first gate value of token 0 (rows `gate_stride` elements apart, heads * vdim
 // values a row, or with gate_per_head one value for each head); sink_scores: null, or a score for each head; work: room for n_tokens * heads * n_slices * (vdim + 2) floats if n_slices > 1; out [n, heads * vdim].
 PALM_API int palm_sink_attention(hipStream_t stream, const void* q, int dtype, const void* k_cache, const void* v_cache,
                                  const int* block_table, int max_pages, const int* seq_slot, const int* seq_start, const int* seq_new,
                                  const int* cu_new, int n_seqs, int max_new, int n_tokens, int heads, int kv_heads, int dim, int vdim,
-                                 float scale, int window, int has_sink, float sink_score, const float* sink_scores, const void* gate,
-                                 int gate_stride, int gate_per_head, int n_slices, float* work, void* out) {
+                                 float scale, int window, int chunked, const float* slopes, int has_sink, float sink_score,
+                                 const float* sink_scores, const void* gate, int gate_stride, int gate_per_head, int n_slices, float* work, void* out) {
     PALM_CHECK(n_seqs >= 0 && max_new >= 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0,
                "sink_attention: seqs=%d max_new=%d heads=%d kv=%d dim=%d vdim=%d", n_seqs, max_new, heads, kv_heads, dim, vdim);
     PALM_CHECK(heads % kv_heads == 0, "sink_attention: %d heads are not a multiple of %d kv heads", heads, kv_heads);
@@ -509,7 +511,7 @@ PALM_API int palm_sink_attention(hipStream_t stream, const void* q, int dtype, c
     dim3 grid(max_new, kv_heads * chunks, n_seqs * n_slices);
     const int nv = (vdim + WAVE - 1) / WAVE;
 #define SK_CASE_V(Q, V) sink_attention_kernel<T, Q, V><<<grid, SK_WAVES * WAVE, 0, stream>>>((const T*)q, (const T*)k_cache, (const T*)v_cache, \
-        block_table, max_pages, seq_slot, seq_start, seq_new, cu_new, heads, kv_heads, dim, vdim, scale, window, has_sink, sink_score, \
+        block_table, max_pages, seq_slot, seq_start, seq_new, cu_new, heads, kv_heads, dim, vdim, scale, window, chunked, slopes, has_sink, sink_score, \
         sink_scores, (const T*)gate, gate_stride, gate_per_head, n_slices, work, (T*)out)
 #define SK_CASE(Q) { if (nv == 1) SK_CASE_V(Q, 1); else if (nv == 2) SK_CASE_V(Q, 2); else if (nv == 3) SK_CASE_V(Q, 3); else SK_CASE_V(Q, 4); }
     PALM_DTYPE_SWITCH(dtype, T, {

@@ -1,4 +1,4 @@
-// Softmax attention with a sink, a window and a gate for prompts on the matrix cores, bfloat16, compiled for one padded
+// Softmax attention with a sink, a window (or chunks), a distance bias and a gate for prompts on the matrix cores, bfloat16, compiled for one padded
 // key size and one padded value size (PALM_SINK_KK: key size / 32 rounded up; PALM_SINK_VT: value size / 16 rounded up).
 //
 // A wave owns one or two tiles of 16 consecutive queries of one head; a block is one wave.  For every page of 64 keys that
@@ -40,9 +40,9 @@ __global__ __launch_bounds__(WAVE) void sink_attention_mfma_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ block_table, int max_pages, const int* __restrict__ seq_slot,
     const int* __restrict__ seq_start, const int* __restrict__ seq_new, const int* __restrict__ cu_new,
-    int heads, int kv_heads, int dim, int vdim, float scale, int window, int has_sink, float sink_score,
-    const float* __restrict__ sink_scores, const bf16_t* __restrict__ gate, int gate_stride, int gate_per_head,
-    bf16_t* __restrict__ out) {
+    int heads, int kv_heads, int dim, int vdim, float scale, int window, int chunked,
+    const float* __restrict__ slopes, int has_sink, float sink_score, const float* __restrict__ sink_scores,
+    const bf16_t* __restrict__ gate, int gate_stride, int gate_per_head, bf16_t* __restrict__ out) {
     const int h = blockIdx.y, b = blockIdx.z;
     if (sink_scores) sink_score = sink_scores[h];                 // a learned score for each head instead of one for all
     const int n_new = seq_new[b];
@@ -53,18 +53,21 @@ __global__ __launch_bounds__(WAVE) void sink_attention_mfma_kernel(
     if (q0 >= n_new) return;
     const int r = lane % 16, g = lane / 16;
     const int start = seq_start[b];
+    // the first key that a query at a position sees (may lie below zero)
+    auto low_of = [&](int pos) { return window <= 0 ? 0 : chunked ? pos - pos % window : pos - window + 1; };
     int qi[QT], qpos[QT], qlow[QT];
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
         qi[t] = min(q0 + 16 * t + r, n_new - 1);                  // a column beyond the run repeats the last query and stores nothing
         qpos[t] = start + qi[t];
-        qlow[t] = window > 0 ? qpos[t] - window + 1 : 0;          // the first key that the query sees (below zero: from the start)
+        qlow[t] = low_of(qpos[t]);
     }
     const int last_pos = start + min(q0 + SM_QUERIES - 1, n_new - 1), first_pos = start + q0;
-    const int first_key = window > 0 ? max(0, first_pos - window + 1) : 0;      // the first key that any query of the wave sees
-    const int last_low = window > 0 ? last_pos - window + 1 : 0;               // the first key that all of them see
+    const int first_key = max(0, low_of(first_pos));                            // the first key that any query of the wave sees
+    const int last_low = low_of(last_pos);                                      // the first key that all of them could see
     const float log2e = 1.4426950408889634f;
     const float scale2 = scale * log2e;
+    const float slope2 = slopes ? slopes[h] * log2e : 0.f;
     const int kvh = h / (heads / kv_heads);
     const int* pages = block_table + (size_t)seq_slot[b] * max_pages;
 
@@ -138,13 +141,15 @@ __global__ __launch_bounds__(WAVE) void sink_attention_mfma_kernel(
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
             float top = -INFINITY;
+            // the distance bias: key 16 n + 4 g + i of the page lies that far beyond the page's first key's distance
+            const float base = slope2 * (float)(pg * PAGE_TOKENS + 4 * g - qpos[t]);
             if (edge) {
 #pragma unroll
                 for (int n = 0; n < 4; ++n)
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         const int j = pg * PAGE_TOKENS + 16 * n + 4 * g + i;
-                        s[t][n][i] = (j <= qpos[t] && j >= qlow[t]) ? s[t][n][i] * scale2 : -INFINITY;
+                        s[t][n][i] = (j <= qpos[t] && j >= qlow[t]) ? fmaf(s[t][n][i], scale2, fmaf(slope2, (float)(16 * n + i), base)) : -INFINITY;
                         top = fmaxf(top, s[t][n][i]);
                     }
             } else {
@@ -152,7 +157,7 @@ __global__ __launch_bounds__(WAVE) void sink_attention_mfma_kernel(
                 for (int n = 0; n < 4; ++n)
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
-                        s[t][n][i] *= scale2;
+                        s[t][n][i] = fmaf(s[t][n][i], scale2, fmaf(slope2, (float)(16 * n + i), base));
                         top = fmaxf(top, s[t][n][i]);
                     }
             }
@@ -229,8 +234,8 @@ __global__ __launch_bounds__(WAVE) void sink_attention_mfma_kernel(
 PALM_API int palm_sink_attention_mfma(hipStream_t stream, const void* q, const void* k_cache, const void* v_cache,
                                       const int* block_table, int max_pages, const int* seq_slot, const int* seq_start,
                                       const int* seq_new, const int* cu_new, int n_seqs, int max_new, int heads, int kv_heads,
-                                      int dim, int vdim, float scale, int window, int has_sink, float sink_score,
-                                      const float* sink_scores, const void* gate, int gate_stride, int gate_per_head, void* out) {
+                                      int dim, int vdim, float scale, int window, int chunked, const float* slopes, int has_sink,
+                                      float sink_score, const float* sink_scores, const void* gate, int gate_stride, int gate_per_head, void* out) {
     PALM_CHECK(n_seqs >= 0 && max_new >= 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0,
                "sink_attention_mfma: seqs=%d max_new=%d heads=%d kv=%d dim=%d vdim=%d", n_seqs, max_new, heads, kv_heads, dim, vdim);
     PALM_CHECK(heads % kv_heads == 0, "sink_attention_mfma: %d heads are not a multiple of %d kv heads", heads, kv_heads);
@@ -244,7 +249,7 @@ PALM_API int palm_sink_attention_mfma(hipStream_t stream, const void* q, const v
     dim3 grid((max_new + SM_QUERIES - 1) / SM_QUERIES, heads, n_seqs);
     sink_attention_mfma_kernel<<<grid, WAVE, 0, stream>>>(
         (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, max_pages, seq_slot, seq_start, seq_new,
-        cu_new, heads, kv_heads, dim, vdim, scale, window, has_sink, sink_score, sink_scores, (const bf16_t*)gate, gate_stride, gate_per_head,
+        cu_new, heads, kv_heads, dim, vdim, scale, window, chunked, slopes, has_sink, sink_score, sink_scores, (const bf16_t*)gate, gate_stride, gate_per_head,
         (bf16_t*)out);
     PALM_LAUNCHED();
     return 0;

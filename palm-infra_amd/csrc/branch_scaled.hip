@@ -7,6 +7,7 @@
 //
 //   y = g * sigmoid(slope * g) * (u + shift),   g = min(gate, limit),   u = clamp(up, -limit, limit)
 #include "common.h"
+#include "expert_form.h"
 
 // Four values of a row at a time (16 bytes of float32, 8 of bfloat16) where the sizes allow.
 __device__ inline void load4(const float* p, float (&o)[4]) {
@@ -104,41 +105,37 @@ PALM_API int palm_add_scaled_normed(hipStream_t stream, float* x, const void* d0
     return 0;
 }
 
-// gate_up [n, 2 ff]: a row's gate values, then its up values.
-__device__ inline float capped(float gate, float up, float limit, float slope, float shift) {
-    const float g = fminf(gate, limit);
-    const float u = fminf(fmaxf(up, -limit), limit);
-    return g * (1.0f / (1.0f + expf(-slope * g))) * (u + shift);
-}
-
-// A row a blockIdx.y; a thread takes four columns at a time if the inner size is a multiple of four, else one.
+// gate_up: rows `stride` elements apart, a row's ff gate values, then its ff up values.
+// A row a blockIdx.y; a thread takes four columns at a time if the inner size and the rows' places are multiples of four
+// (`by_four`), else one.
 template <typename T>
-__global__ void capped_gate_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int ff, float limit, float slope, float shift) {
+__global__ void capped_gate_kernel(const T* __restrict__ gate_up, int stride, int by_four, T* __restrict__ out, int ff, ExpertCap cap) {
     const size_t r = blockIdx.y;
-    const T* row = gate_up + r * 2 * ff;
-    if (ff % 4 == 0) {
+    const T* row = gate_up + r * stride;
+    if (by_four) {
         const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
         if (c >= ff) return;
         float g[4], u[4], y[4];
         load4(row + c, g);
         load4(row + ff + c, u);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) y[i] = capped(g[i], u[i], limit, slope, shift);
+        for (int i = 0; i < 4; ++i) y[i] = expert_capped(g[i], u[i], cap);
         store4(out + r * ff + c, y);
     } else {
         for (int c = blockIdx.x * blockDim.x * 4 + threadIdx.x; c < min(ff, (int)(blockIdx.x + 1) * (int)blockDim.x * 4); c += blockDim.x)
-            out[r * ff + c] = from_float<T>(capped(to_float(row[c]), to_float(row[ff + c]), limit, slope, shift));
+            out[r * ff + c] = from_float<T>(expert_capped(to_float(row[c]), to_float(row[ff + c]), cap));
     }
 }
 
-PALM_API int palm_capped_gate(hipStream_t stream, const void* gate_up, void* out, int dtype, int n, int ff, float limit, float slope,
-                              float shift) {
-    PALM_CHECK(n >= 0 && ff > 0 && limit > 0.f, "capped_gate: rows=%d ff=%d limit=%g", n, ff, (double)limit);
+PALM_API int palm_capped_gate(hipStream_t stream, const void* gate_up, int stride, void* out, int dtype, int n, int ff, float limit,
+                              float slope, float shift) {
+    PALM_CHECK(n >= 0 && ff > 0 && limit > 0.f && stride >= 2 * ff, "capped_gate: rows=%d, %d apart, ff=%d limit=%g", n, stride, ff, (double)limit);
     if (n == 0) return 0;
     PALM_CHECK(n <= 65535, "capped_gate: %d rows are more than one launch takes", n);
     const dim3 grid((ff + 1023) / 1024, n);                      // a block of 256 threads takes 1,024 columns of a row
+    const int by_four = ff % 4 == 0 && stride % 4 == 0 && reinterpret_cast<uintptr_t>(gate_up) % 16 == 0;
     PALM_DTYPE_SWITCH(dtype, T,
-        capped_gate_kernel<T><<<grid, 256, 0, stream>>>((const T*)gate_up, (T*)out, ff, limit, slope, shift));
+        capped_gate_kernel<T><<<grid, 256, 0, stream>>>((const T*)gate_up, stride, by_four, (T*)out, ff, ExpertCap{limit, slope, shift}));
     PALM_LAUNCHED();
     return 0;
 }

@@ -8,9 +8,7 @@
 //
 // S is 32-bit and kept per sequence; step sizes, decays, exponentials and the sums are 32-bit.  Both kernels walk
 // over a sequence's new tokens whatever their number: a prompt leaves what its tokens one by one leave.
-#include "common.h"
-
-constexpr int CONV_MAX_TAPS = 16;
+#include "conv_state.h"
 
 __device__ inline float silu_f(float z) { return z / (1.0f + expf(-z)); }
 __device__ inline float softplus_dt(float z) { return z > 20.f ? z : log1pf(expf(z)); }
@@ -32,30 +30,6 @@ __global__ void causal_conv_kernel(const T* __restrict__ x, int x_stride, const 
         acc = fmaf(w[(size_t)c * taps + j], v, acc);
     }
     out[(row0 + ti) * channels + c] = from_float<T>(silu_f(acc));
-}
-
-// After the convolution has read the old state: the last taps-1 inputs of each sequence, old ones moved up.
-template <typename T>
-__global__ void conv_state_kernel(const T* __restrict__ x, int x_stride, float* __restrict__ conv_state,
-                                  const int* __restrict__ seq_slot, const int* __restrict__ seq_new,
-                                  const int* __restrict__ cu_new, int channels, int taps) {
-    const int c = blockIdx.x * blockDim.x + threadIdx.x, b = blockIdx.y;
-    if (c >= channels) return;
-    const int n_new = seq_new[b];
-    if (n_new <= 0) return;
-    const size_t row0 = (size_t)cu_new[b];
-    float* st = conv_state + (size_t)seq_slot[b] * (taps - 1) * channels;
-    float keep[CONV_MAX_TAPS];
-#pragma unroll
-    for (int j = 0; j < CONV_MAX_TAPS; ++j) {
-        if (j < taps - 1) {
-            const int at = n_new - (taps - 1) + j;
-            keep[j] = at >= 0 ? to_float(x[(row0 + at) * x_stride + c]) : st[(size_t)(taps - 1 + at) * channels + c];
-        }
-    }
-#pragma unroll
-    for (int j = 0; j < CONV_MAX_TAPS; ++j)
-        if (j < taps - 1) st[(size_t)j * channels + c] = keep[j];
 }
 
 PALM_API int palm_causal_conv(hipStream_t stream, const void* x, int dtype, int x_stride, const float* w, const float* bias,

@@ -5,10 +5,13 @@
 //   few rows (a decode step): nothing is planned on the host, every (token, choice) reads its expert's weights itself
 //     expert_gate_up   mid[t, c, f] = silu(G_e h_t)[f] * (U_e h_t)[f],  e = chosen[t, c]           (32-bit)
 //     expert_down      out[t, :] = sum_c weight[t, c] * D_e mid[t, c, :]  in the order of c        (32-bit)
-//   An expert's form: gated (silu(G h) * (U h), the gate rows before the up rows) or plain with the exact gelu (gelu(U h)).
+//   An expert's form: gated (silu(G h) * (U h), the gate rows before the up rows), plain with the exact gelu (gelu(U h)), or
+//   capped gated (g sigmoid(slope g) (u + shift) with g = min(G h, limit), u = clamp(U h, -limit, limit)).
+//   Rows that other branches made (up to two) can be added to the weighted sum where it is written.
 //
-//   route, scored: the scores are sigmoid(logit); the choice is made by score plus a correction per expert; experts lie in
-//              equal groups of neighbours, a group's rank is the sum of its two largest corrected scores, and only experts
+//   route, scored: the scores are sigmoid(logit) or the softmax over all experts; the choice is made by score plus a
+//              correction per expert (or by the score alone); experts lie in
+//              equal groups of neighbours, a group's rank is the sum of its two largest corrected scores, or its largest, and only experts
 //              of the best `keep` groups can be chosen; the weights are the chosen experts' scores (without the correction)
 //              over their sum, times a scale
 //   many rows (a prompt): the host groups the (token, choice) pairs by expert, the products are the library's
@@ -16,6 +19,7 @@
 //     scatter_add      out[rows[i], :] += weight[i] * y[i, :]      (an expert's rows are distinct tokens: no two
 //                      threads meet, and the experts are added one after the other)
 #include "common.h"
+#include "expert_form.h"
 
 constexpr int ROUTE_MAX_PER_LANE = 8;            // up to 512 experts
 
@@ -62,7 +66,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
         const float p = expf(best - first);                  // the first is the largest
         sum += p;
         if (lane == c) mine = p;                             // lane c keeps choice c's weight
-        if (lane == 0) chosen[t * top + c] = at;
+        if (lane == 0) chosen[t * top + c] = min(at, experts - 1);     // (logits that are no numbers choose nobody: an expert that exists is named all the same)
 #pragma unroll
         for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
             if (i * WAVE + lane == at) z[i] = -INFINITY;
@@ -71,33 +75,44 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
 }
 
 // One wave per token.  logits: rows `stride` apart (other columns may follow the experts').
-__device__ inline float moe_gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
-
 __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __restrict__ logits, int stride, int experts, int top,
                                                                 const float* __restrict__ correction, int groups, int keep, float scale,
-                                                                int* __restrict__ chosen, float* __restrict__ weight) {
+                                                                int softmax, int group_largest, int* __restrict__ chosen, float* __restrict__ weight) {
     __shared__ float choice_s[ROUTE_MAX_PER_LANE * WAVE];
     __shared__ float group_s[ROUTE_MAX_PER_LANE * WAVE];
     const size_t t = blockIdx.x;
     const int lane = threadIdx.x;
     float s[ROUTE_MAX_PER_LANE], z[ROUTE_MAX_PER_LANE];
+    float high = -INFINITY, total = 0.f;
 #pragma unroll
     for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
         const int e = i * WAVE + lane;
-        s[i] = e < experts ? 1.0f / (1.0f + expf(-logits[t * stride + e])) : 0.f;
+        s[i] = e < experts ? logits[t * stride + e] : -INFINITY;
+        high = fmaxf(high, s[i]);
+    }
+    if (softmax) {
+        high = wave_max(high);
+#pragma unroll
+        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) { s[i] = expf(s[i] - high); total += s[i]; }
+        total = wave_sum(total);
+    }
+#pragma unroll
+    for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+        const int e = i * WAVE + lane;
+        s[i] = e >= experts ? 0.f : softmax ? s[i] / total : 1.0f / (1.0f + expf(-s[i]));
         z[i] = e < experts ? s[i] + (correction ? correction[e] : 0.f) : -INFINITY;
         if (e < experts) choice_s[e] = z[i];
     }
     if (groups > 1) {
         const int size = experts / groups;
         __syncthreads();
-        for (int g = lane; g < groups; g += WAVE) {                    // the sum of the group's two largest
+        for (int g = lane; g < groups; g += WAVE) {                    // the sum of the group's two largest, or its largest
             float a = -INFINITY, b = -INFINITY;
             for (int j = 0; j < size; ++j) {
                 const float v = choice_s[g * size + j];
                 if (v > a) { b = a; a = v; } else if (v > b) b = v;
             }
-            group_s[g] = size > 1 ? a + b : a;
+            group_s[g] = size > 1 && !group_largest ? a + b : a;
         }
         __syncthreads();
 #pragma unroll
@@ -128,7 +143,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __r
         }
         sum += score;
         if (lane == c) mine = score;
-        if (lane == 0) chosen[t * top + c] = at;
+        if (lane == 0) chosen[t * top + c] = min(at, experts - 1);
 #pragma unroll
         for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
             if (i * WAVE + lane == at) z[i] = -INFINITY;
@@ -142,14 +157,14 @@ constexpr int MOE_THREADS = 256;
 template <typename T, typename TW>
 __global__ __launch_bounds__(MOE_THREADS) void expert_gate_up_kernel(const T* __restrict__ h, const TW* __restrict__ gate_up,
                                                                      const int* __restrict__ chosen, int top, int width, int ff,
-                                                                     int rows_per_block, int form, float* __restrict__ mid) {
+                                                                     int rows_per_block, int form, ExpertCap cap, float* __restrict__ mid) {
     extern __shared__ float h_s[];                  // [width]
     const int t = blockIdx.z, c = blockIdx.y;
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, n_waves = MOE_THREADS / WAVE;
     for (int d = threadIdx.x; d < width; d += MOE_THREADS) h_s[d] = to_float(h[(size_t)t * width + d]);
     __syncthreads();
     const int e = chosen[(size_t)t * top + c];
-    const bool gated = form == 0;                   // else: up rows alone, through the exact gelu
+    const bool gated = form != EXPERT_GELU;         // else: up rows alone, through the exact gelu
     const TW* w = gate_up + (size_t)e * (gated ? 2 : 1) * ff * width;
     const int f_end = min(ff, (int)(blockIdx.x + 1) * rows_per_block);
     // Two rows of the first matrix are under way at a time in both forms: an inner value's gate row and up row, or (plain)
@@ -184,20 +199,22 @@ __global__ __launch_bounds__(MOE_THREADS) void expert_gate_up_kernel(const T* __
         if (lane == 0) {
             float* m = mid + ((size_t)t * top + c) * ff;
             if (gated) {
-                m[f] = g / (1.0f + expf(-g)) * u;
+                m[f] = form == EXPERT_CAPPED ? expert_capped(g, u, cap) : expert_silu_gated(g, u);
             } else {
-                m[f] = moe_gelu_erf(u);
-                if (f2 < f_end) m[f2] = moe_gelu_erf(g);
+                m[f] = expert_gelu(u);
+                if (f2 < f_end) m[f2] = expert_gelu(g);
             }
         }
     }
 }
 
 // grid (blocks of output rows, tokens); a wave computes one output value at a time, the choices one after the other.
-template <typename TW>
+// `add0`, `add1`: null, or rows [n, width] that other branches made, added to the sum.
+template <typename T, typename TW>
 __global__ __launch_bounds__(MOE_THREADS) void expert_down_kernel(const float* __restrict__ mid, const TW* __restrict__ down,
                                                                   const int* __restrict__ chosen, const float* __restrict__ weight,
                                                                   int top, int width, int ff, int rows_per_block,
+                                                                  const T* __restrict__ add0, const T* __restrict__ add1,
                                                                   float* __restrict__ out) {
     extern __shared__ float m_s[];                  // [top][ff]
     const int t = blockIdx.y;
@@ -222,7 +239,11 @@ __global__ __launch_bounds__(MOE_THREADS) void expert_down_kernel(const float* _
             }
             total = fmaf(weight[(size_t)t * top + c], wave_sum(acc), total);
         }
-        if (lane == 0) out[(size_t)t * width + r] = total;
+        if (lane == 0) {
+            if (add0) total += to_float(add0[(size_t)t * width + r]);
+            if (add1) total += to_float(add1[(size_t)t * width + r]);
+            out[(size_t)t * width + r] = total;
+        }
     }
 }
 
@@ -253,7 +274,8 @@ PALM_API int palm_moe_route(hipStream_t stream, const float* logits, int n_token
 }
 
 PALM_API int palm_moe_route_scored(hipStream_t stream, const float* logits, int stride, int n_tokens, int experts, int top,
-                                   const float* correction, int groups, int keep, float scale, int* chosen, float* weight) {
+                                   const float* correction, int groups, int keep, float scale, int softmax, int group_largest, int* chosen,
+                                   float* weight) {
     PALM_CHECK(n_tokens >= 0 && experts > 0 && top > 0 && top <= experts && stride >= experts, "moe_route_scored: n=%d experts=%d top=%d stride=%d",
                n_tokens, experts, top, stride);
     PALM_CHECK(experts <= ROUTE_MAX_PER_LANE * WAVE, "moe_route_scored: %d experts exceed %d", experts, ROUTE_MAX_PER_LANE * WAVE);
@@ -263,7 +285,7 @@ PALM_API int palm_moe_route_scored(hipStream_t stream, const float* logits, int 
     PALM_CHECK((long long)keep * (experts / groups) >= top, "moe_route_scored: %d groups of %d experts cannot give %d choices", keep,
                experts / groups, top);
     if (n_tokens == 0) return 0;
-    moe_route_scored_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, stride, experts, top, correction, groups, keep, scale, chosen, weight);
+    moe_route_scored_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, stride, experts, top, correction, groups, keep, scale, softmax, group_largest, chosen, weight);
     PALM_LAUNCHED();
     return 0;
 }
@@ -285,13 +307,14 @@ PALM_API int palm_add_gated_rows(hipStream_t stream, float* out, const void* y, 
     return 0;
 }
 
-// h [n, width]; gate_up [experts, 2 ff, width] (an expert's gate rows, then its up rows; form 1: [experts, ff, width], up rows
-// alone); down [experts, width, ff];
+// h [n, width]; gate_up [experts, 2 ff, width] (an expert's gate rows, then its up rows; the gelu form: [experts, ff, width], up
+// rows alone); add0, add1: null or rows [n, width] of h's type; down [experts, width, ff];
 // chosen, weight [n, top]; mid: room for n * top * ff floats; out float32 [n, width].
 PALM_API int palm_moe_experts(hipStream_t stream, const void* h, int dtype, const void* gate_up, const void* down, int w_dtype,
                               const int* chosen, const float* weight, int n_tokens, int top, int width, int ff, float* mid,
-                              float* out, int form) {
-    PALM_CHECK(form == 0 || form == 1, "moe_experts: form %d is neither gated silu (0) nor plain gelu (1)", form);
+                              float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1) {
+    PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_CAPPED, "moe_experts: form %d is neither gated silu (0) nor plain gelu (1) nor capped gated (2)", form);
+    PALM_CHECK(form != EXPERT_CAPPED || limit > 0.f, "moe_experts: the cap %g must be positive", (double)limit);
     PALM_CHECK(n_tokens >= 0 && top > 0 && width > 0 && ff > 0, "moe_experts: n=%d top=%d width=%d ff=%d", n_tokens, top, width, ff);
     PALM_CHECK(width <= 16384 && (long long)top * ff <= 16384, "moe_experts: width %d / top x ff %d x %d exceed what a block holds", width, top, ff);
     PALM_CHECK(n_tokens <= 65535 && top <= 65535, "moe_experts: %d tokens x %d choices are more than one launch takes", n_tokens, top);
@@ -302,9 +325,9 @@ PALM_API int palm_moe_experts(hipStream_t stream, const void* h, int dtype, cons
     PALM_DTYPE_SWITCH(dtype, T, {
         PALM_DTYPE_SWITCH(w_dtype, TW, {
             expert_gate_up_kernel<T, TW><<<dim3(up_blocks, top, n_tokens), MOE_THREADS, width * sizeof(float), stream>>>(
-                (const T*)h, (const TW*)gate_up, chosen, top, width, ff, up_rows, form, mid);
-            expert_down_kernel<TW><<<dim3(down_blocks, n_tokens), MOE_THREADS, (size_t)top * ff * sizeof(float), stream>>>(
-                mid, (const TW*)down, chosen, weight, top, width, ff, down_rows, out);
+                (const T*)h, (const TW*)gate_up, chosen, top, width, ff, up_rows, form, ExpertCap{limit, slope, shift}, mid);
+            expert_down_kernel<T, TW><<<dim3(down_blocks, n_tokens), MOE_THREADS, (size_t)top * ff * sizeof(float), stream>>>(
+                mid, (const TW*)down, chosen, weight, top, width, ff, down_rows, (const T*)add0, (const T*)add1, out);
         });
     });
     PALM_LAUNCHED();

@@ -8,8 +8,10 @@
 //             y = D_e mid.  The weights are the first operand of the matrix instruction, so that a lane ends with four
 //             neighbouring features of one row; a wave owns 32 features x 64 rows and reads its fragments from memory itself
 //             (a weight fragment feeds four products, a row fragment two or four)
-//   combine   out[t] = sum_c weight[t, c] * y[place of pair (t, c)], in the order of c, 32-bit
+//   combine   out[t] = sum_c weight[t, c] * y[place of pair (t, c)], in the order of c, 32-bit, plus up to two rows that other
+//             branches made
 #include "mfma.h"
+#include "expert_form.h"
 
 constexpr int GT_TOKENS = 64;                     // rows of a tile
 constexpr int GT_RUNS = GT_TOKENS / 16;           // runs of 16 rows: what one matrix instruction takes
@@ -94,13 +96,13 @@ __global__ __launch_bounds__(PLAN_THREADS) void moe_place_kernel(const int* __re
 
 // grid (tiles, blocks of GT_FEATURES features).  a: the rows [*, k_dim]; row_of_slot: null (the rows lie in slot order) or
 // slot -> pair, the pair's row being pair / top.  w: [experts, n_w_rows, k_dim]; FORM 1 (gated): n_w_rows = 2 n_features, an
-// expert's gate rows first, and the result is silu(gate) * up; FORM 2: the product through the exact gelu; FORM 0: the product
-// as it is.  out: bfloat16 [slots, n_features].
+// expert's gate rows first, and the result is silu(gate) * up; FORM 3: the same rows, capped gated; FORM 2: the product through
+// the exact gelu; FORM 0: the product as it is.  out: bfloat16 [slots, n_features].
 template <int FORM>
 __global__ __launch_bounds__(GT_WAVES * WAVE) void moe_grouped_kernel(const bf16_t* __restrict__ a, const int* __restrict__ slot_pair, int top,
                                                                       const bf16_t* __restrict__ w, const int* __restrict__ tile_expert,
-                                                                      int n_features, int k_dim, bf16_t* __restrict__ out) {
-    constexpr bool GATED = FORM == 1;
+                                                                      int n_features, int k_dim, ExpertCap cap, bf16_t* __restrict__ out) {
+    constexpr bool GATED = FORM == 1 || FORM == 3;
     const int tile = blockIdx.x;
     const int e = tile_expert[tile];
     if (e < 0) return;
@@ -154,11 +156,9 @@ __global__ __launch_bounds__(GT_WAVES * WAVE) void moe_grouped_kernel(const bf16
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 if (GATED) {
-                    const float gt = acc[ft][tt][i];
-                    v[i] = gt / (1.0f + expf(-gt)) * acc[2 + ft][tt][i];
+                    v[i] = FORM == 3 ? expert_capped(acc[ft][tt][i], acc[2 + ft][tt][i], cap) : expert_silu_gated(acc[ft][tt][i], acc[2 + ft][tt][i]);
                 } else if (FORM == 2) {
-                    const float z = acc[ft][tt][i];
-                    v[i] = 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
+                    v[i] = expert_gelu(acc[ft][tt][i]);
                 } else {
                     v[i] = acc[ft][tt][i];
                 }
@@ -172,25 +172,28 @@ __global__ __launch_bounds__(GT_WAVES * WAVE) void moe_grouped_kernel(const bf16
 
 // One block per token.
 __global__ void moe_combine_kernel(const bf16_t* __restrict__ y, const int* __restrict__ pair_slot, const float* __restrict__ weight, int top,
-                                   int width, float* __restrict__ out) {
+                                   int width, const bf16_t* __restrict__ add0, const bf16_t* __restrict__ add1, float* __restrict__ out) {
     const size_t t = blockIdx.x;
     for (int d = threadIdx.x; d < width; d += blockDim.x) {
         float total = 0.f;
         for (int c = 0; c < top; ++c) total = fmaf(weight[t * top + c], to_float(y[(size_t)pair_slot[t * top + c] * width + d]), total);
+        if (add0) total += to_float(add0[t * width + d]);
+        if (add1) total += to_float(add1[t * width + d]);
         out[t * width + d] = total;
     }
 }
 
 PALM_API int palm_moe_tile_tokens() { return GT_TOKENS; }
 
-// chosen, weight [n, top]; h bfloat16 [n, width]; gate_up bfloat16 [experts, 2 ff, width] (form 1: [experts, ff, width], up rows
-// alone, through the exact gelu); down bfloat16 [experts, width, ff].
+// chosen, weight [n, top]; h bfloat16 [n, width]; gate_up bfloat16 [experts, 2 ff, width] (the gelu form: [experts, ff, width], up
+// rows alone); add0, add1: null or bfloat16 rows [n, width]; down bfloat16 [experts, width, ff].
 // Room, with max_tiles = ceil(n top / tile) + experts and slots = max_tiles * tile: plan: (2 experts + 1 + max_tiles + slots
 // + n top) ints; mid: slots * ff bfloat16; y: slots * width bfloat16.  out float32 [n, width].
 PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gate_up, const void* down, const int* chosen,
                               const float* weight, int n_tokens, int top, int experts, int width, int ff, int* plan, void* mid, void* y,
-                              float* out, int form) {
-    PALM_CHECK(form == 0 || form == 1, "moe_grouped: form %d is neither gated silu (0) nor plain gelu (1)", form);
+                              float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1) {
+    PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_CAPPED, "moe_grouped: form %d is neither gated silu (0) nor plain gelu (1) nor capped gated (2)", form);
+    PALM_CHECK(form != EXPERT_CAPPED || limit > 0.f, "moe_grouped: the cap %g must be positive", (double)limit);
     PALM_CHECK(n_tokens >= 0 && top > 0 && experts > 0 && width > 0 && ff > 0, "moe_grouped: n=%d top=%d experts=%d width=%d ff=%d", n_tokens,
                top, experts, width, ff);
     PALM_CHECK(width % 8 == 0 && ff % 8 == 0, "moe_grouped: width %d and inner size %d must be multiples of eight", width, ff);
@@ -206,15 +209,17 @@ PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gat
     moe_count_kernel<<<experts, PLAN_THREADS, 0, stream>>>(chosen, (int)n_pairs, counts);
     moe_runs_kernel<<<1, PLAN_THREADS, 0, stream>>>(counts, experts, max_tiles, starts, tile_expert);
     moe_place_kernel<<<experts, PLAN_THREADS, 0, stream>>>(chosen, (int)n_pairs, starts, slot_pair, pair_slot);
-    if (form == 0)
-        moe_grouped_kernel<1><<<dim3(max_tiles, (ff + GT_FEATURES - 1) / GT_FEATURES), GT_WAVES * WAVE, 0, stream>>>(
-            (const bf16_t*)h, slot_pair, top, (const bf16_t*)gate_up, tile_expert, ff, width, (bf16_t*)mid);
-    else
-        moe_grouped_kernel<2><<<dim3(max_tiles, (ff + GT_FEATURES - 1) / GT_FEATURES), GT_WAVES * WAVE, 0, stream>>>(
-            (const bf16_t*)h, slot_pair, top, (const bf16_t*)gate_up, tile_expert, ff, width, (bf16_t*)mid);
+    const ExpertCap cap{limit, slope, shift};
+    const dim3 up_grid(max_tiles, (ff + GT_FEATURES - 1) / GT_FEATURES);
+#define MOE_UP(FORM) moe_grouped_kernel<FORM><<<up_grid, GT_WAVES * WAVE, 0, stream>>>((const bf16_t*)h, slot_pair, top, (const bf16_t*)gate_up, \
+        tile_expert, ff, width, cap, (bf16_t*)mid)
+    if (form == EXPERT_GATED_SILU) MOE_UP(1);
+    else if (form == EXPERT_GELU) MOE_UP(2);
+    else MOE_UP(3);
+#undef MOE_UP
     moe_grouped_kernel<0><<<dim3(max_tiles, (width + GT_FEATURES - 1) / GT_FEATURES), GT_WAVES * WAVE, 0, stream>>>(
-        (const bf16_t*)mid, nullptr, top, (const bf16_t*)down, tile_expert, width, ff, (bf16_t*)y);
-    moe_combine_kernel<<<n_tokens, 256, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, out);
+        (const bf16_t*)mid, nullptr, top, (const bf16_t*)down, tile_expert, width, ff, cap, (bf16_t*)y);
+    moe_combine_kernel<<<n_tokens, 256, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, (const bf16_t*)add0, (const bf16_t*)add1, out);
     PALM_LAUNCHED();
     return 0;
 }

@@ -12,26 +12,9 @@
 // written as they are, 32-bit, and a pass of its own norms a token's joined heads together, with a weight, and gates
 // them (palm_joined_norm_gate).
 //
-// A first pass rotates q and k of all the step's tokens into 32-bit rows.  Then one block per (head, sequence), one
-// thread per value dimension v: the thread keeps column v of S in registers and walks over the sequence's new
-// tokens.  A token's rotated q and k are the same for every thread of the block: each wave reads the two rows once,
-// one value a lane, and broadcasts value d to all its lanes as a scalar operand of the multiply-adds (no LDS and no
-// barrier in the recurrence); the per-token sums of squares over v are reduced a tile of tokens at a time.  A prompt and a single token run the same code, so a prompt leaves the state that its tokens
-// one by one leave.
-//
-// A long run of new tokens would keep only (heads x sequences) blocks busy, one after the other token.  Such a run is
-// cut into chunks of `chunk` tokens, and the recurrence's linearity does the rest in three launches:
-//   1. every chunk alone from a zero state: its own sum  L_c = sum_t g^(end - t) k_t v_t^T         (all chunks at once)
-//   2. the chunks' starting states, one after the other: S_(c+1) = g^len_c S_c + L_c, S_0 the kept state   (elementwise)
-//   3. every chunk from its starting state, now with outputs                                        (all chunks at once)
-// The arithmetic of a token is the same in all three; only the order of the 32-bit sums over the past differs.
-#include "common.h"
-
-constexpr int RET_TILE = 8;
-
-enum RetentionMode : int { RET_WHOLE = 0, RET_LOCAL = 1, RET_FROM_STARTS = 2 };
-
-__device__ inline float ret_silu(float z) { return z / (1.0f + expf(-z)); }
+// A first pass rotates q and k of all the step's tokens into 32-bit rows; the walk over the tokens, and how a long run of
+// them is cut into chunks that run side by side, is linear_recurrence.h's.
+#include "linear_recurrence.h"
 
 // q and k of every token and head, rotated (k also scaled), 32-bit: qk[row][head][0 = q, 1 = k][pad], pad >= dim the
 // key size that the main kernel is compiled for; the columns beyond dim are zero, so that the main kernel's loops
@@ -50,169 +33,19 @@ __global__ void retention_rotate_kernel(const T* __restrict__ qkvg, int row_stri
     const T* qr = qkvg + row * row_stride + q_off + h * dim;
     const T* kr = qkvg + row * row_stride + k_off + h * dim;
     float qv = to_float(qr[d]), kv = to_float(kr[d]);
-    if (act) { qv = ret_silu(qv); kv = ret_silu(kv); }
+    if (act) { qv = rec_silu(qv); kv = rec_silu(kv); }
     if (d < rot) {
         const int i = d < half ? d : d - half;
         const float c = cos_t[row * half + i], sn = sin_t[row * half + i];
         const int partner = d < half ? d + half : d - half;
         float qp = to_float(qr[partner]), kp = to_float(kr[partner]);
-        if (act) { qp = ret_silu(qp); kp = ret_silu(kp); }
+        if (act) { qp = rec_silu(qp); kp = rec_silu(kp); }
         // the pair (u, w) becomes (u c - w s, w c + u s)
         qv = d < half ? qv * c - qp * sn : qv * c + qp * sn;
         kv = d < half ? kv * c - kp * sn : kv * c + kp * sn;
     }
     o[0] = qv;
     o[pad] = kv * k_scale;
-}
-
-// MAXT: the most threads of a block (the value size, rounded up to whole waves): what the compiler may assume when it
-// hands out registers.  A thread keeps DMAX values of S; up to 256 threads a block they all stay in registers.
-template <typename T, int DMAX, int MAXT>
-__global__ __launch_bounds__(MAXT) void retention_kernel(int mode, int chunk, int max_chunks, float* __restrict__ starts, const T* __restrict__ qkvg,
-                                 int row_stride, int v_off, int g_off, const float* __restrict__ qk,
-                                 const float* __restrict__ decay, float eps,
-                                 float* __restrict__ state, const int* __restrict__ seq_slot,
-                                 const int* __restrict__ seq_new, const int* __restrict__ cu_new,
-                                 int heads, int dim, int vdim, T* __restrict__ out, int act, int joined, float* __restrict__ raw) {
-    __shared__ float red[RET_TILE][16];
-    __shared__ float o_s[RET_TILE][MAXT];
-    constexpr int QREGS = (DMAX + WAVE - 1) / WAVE;
-    const int h = blockIdx.x, b = blockIdx.y / max_chunks, c = blockIdx.y % max_chunks;
-    const int v = threadIdx.x;
-    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, n_waves = blockDim.x / WAVE;
-    // this block's run of tokens: the sequence's new ones, or one chunk of them
-    const int seq_tokens = seq_new[b];
-    if (c * chunk >= seq_tokens) return;
-    const int n_new = mode == RET_WHOLE ? seq_tokens : min(chunk, seq_tokens - c * chunk);
-    const int row0 = cu_new[b] + (mode == RET_WHOLE ? 0 : c * chunk);
-    const bool mine = v < vdim;
-    const float g = decay[h];
-    float* sp = mode == RET_WHOLE ? state + (((size_t)seq_slot[b] * heads + h) * dim) * vdim + v
-                                  : starts + ((((size_t)b * max_chunks + c) * heads + h) * dim) * vdim + v;
-
-    // the reads are unconditional (of a row and a column that exist) and what does not belong is set to zero after:
-    // no branch between them, so that they are all under way at once
-    float S[DMAX];
-    {
-        const float* at = sp - v + min(v, vdim - 1);
-        const bool zero = mode == RET_LOCAL || !mine;
-        if (dim == DMAX) {                                        // the usual case: every row exists, one stride for all reads
-            const size_t stride = (size_t)vdim;
-#pragma unroll
-            for (int d = 0; d < DMAX; ++d) S[d] = at[d * stride];
-            if (zero) {
-#pragma unroll
-                for (int d = 0; d < DMAX; ++d) S[d] = 0.f;
-            }
-        } else {
-#pragma unroll
-            for (int d = 0; d < DMAX; ++d) {
-                const float s0 = at[(size_t)min(d, dim - 1) * vdim];
-                S[d] = (zero || d >= dim) ? 0.f : s0;
-            }
-        }
-    }
-
-    // A token's inputs: the thread's value, and of the token's q and k rows (the same for all threads) one value a
-    // lane, which the wave hands to all its lanes as scalars.  The next token's are read while this one's are used.
-    const int vc = min(v, vdim - 1);
-    auto read_token = [&](int t, float& vv, float (&qv)[QREGS], float (&kv)[QREGS]) {
-        const size_t row = (size_t)(row0 + t);
-        vv = to_float(qkvg[row * row_stride + v_off + h * vdim + vc]);
-        if (act) vv = ret_silu(vv);
-        const float* __restrict__ qr = qk + ((row * heads + h) * 2) * DMAX;
-#pragma unroll
-        for (int c = 0; c < QREGS; ++c) {
-            const int at = min(c * WAVE + lane, DMAX - 1);             // (a key size of 32: the upper lanes repeat)
-            qv[c] = qr[at];
-            kv[c] = qr[DMAX + at];
-        }
-    };
-    float vv, qv[QREGS], kv[QREGS];
-    if (n_new > 0) read_token(0, vv, qv, kv);
-    for (int t0 = 0; t0 < n_new; t0 += RET_TILE) {
-        const int tt = min(RET_TILE, n_new - t0);
-        for (int ti = 0; ti < tt; ++ti) {                        // not unrolled: the body is DMAX steps long already
-            float vn, qn[QREGS], kn[QREGS];
-            read_token(min(t0 + ti + 1, n_new - 1), vn, qn, kn);
-            if (!mine) vv = 0.f;
-            float acc = 0.f;
-#pragma unroll
-            for (int d = 0; d < DMAX; ++d) {
-                const float qd = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, qv[d / WAVE]), d % WAVE));
-                const float kd = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, kv[d / WAVE]), d % WAVE));
-                S[d] = fmaf(g, S[d], kd * vv);
-                acc = fmaf(S[d], qd, acc);
-            }
-            if (mode != RET_LOCAL && joined) {
-                if (mine) raw[(size_t)(row0 + t0 + ti) * ((size_t)heads * vdim) + h * vdim + v] = acc;
-            } else if (mode != RET_LOCAL) {
-                o_s[ti][v] = acc;
-                const float ss = wave_sum(acc * acc);
-                if (lane == 0) red[ti][wave] = ss;
-            }
-            vv = vn;
-#pragma unroll
-            for (int c = 0; c < QREGS; ++c) { qv[c] = qn[c]; kv[c] = kn[c]; }
-        }
-        if (mode == RET_LOCAL || joined) continue;
-        __syncthreads();
-        for (int ti = 0; ti < tt; ++ti) {
-            float total = 0.f;
-            for (int w = 0; w < n_waves; ++w) total += red[ti][w];
-            const float inv = 1.0f / sqrtf(total / (float)vdim + eps);
-            const size_t row = (size_t)(row0 + t0 + ti);
-            const float gate = to_float(qkvg[row * row_stride + g_off + h * vdim + vc]);
-            if (mine) out[row * ((size_t)heads * vdim) + h * vdim + v] = from_float<T>(o_s[ti][v] * inv * (gate / (1.0f + expf(-gate))));
-        }
-        __syncthreads();
-    }
-    if (mine && n_new > 0 && mode != RET_FROM_STARTS) {
-        if (dim == DMAX) {
-#pragma unroll
-            for (int d = 0; d < DMAX; ++d) sp[(size_t)d * vdim] = S[d];
-        } else {
-#pragma unroll
-            for (int d = 0; d < DMAX; ++d)
-                if (d < dim) sp[(size_t)d * vdim] = S[d];
-        }
-    }
-}
-
-// Step 2 above: one thread per element of (sequence, head, dim, vdim).  starts[b][c] holds L_c and leaves as S_c.
-__global__ void retention_starts_kernel(float* __restrict__ starts, float* __restrict__ state, const float* __restrict__ decay,
-                                        const int* __restrict__ seq_slot, const int* __restrict__ seq_new, int chunk,
-                                        int max_chunks, int heads, int per_head) {
-    const int e = blockIdx.x * blockDim.x + threadIdx.x, b = blockIdx.y;
-    if (e >= heads * per_head) return;
-    const int n_new = seq_new[b];
-    if (n_new <= 0) return;
-    const float g = decay[e / per_head];
-    float* st = state + (size_t)seq_slot[b] * heads * per_head + e;
-    float s = *st;
-    for (int c = 0; c * chunk < n_new; ++c) {
-        float* at = starts + ((size_t)b * max_chunks + c) * heads * per_head + e;
-        const float local = *at;
-        *at = s;
-        s = fmaf(powf(g, (float)min(chunk, n_new - c * chunk)), s, local);
-    }
-    *st = s;
-}
-
-template <typename T>
-static void retention_launch(hipStream_t stream, dim3 grid, int threads, int mode, int chunk, int max_chunks, float* starts,
-                             const T* qkvg, int row_stride, int v_off, int g_off, const float* qk, const float* decay,
-                             float eps, float* state, const int* seq_slot, const int* seq_new,
-                             const int* cu_new, int heads, int dim, int vdim, T* out, int act, int joined, float* raw) {
-#define RET_CASE(D) { if (threads <= 256) retention_kernel<T, D, 256><<<grid, threads, 0, stream>>>(mode, chunk, max_chunks, starts, qkvg, \
-            row_stride, v_off, g_off, qk, decay, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, out, act, joined, raw); \
-        else retention_kernel<T, D, 1024><<<grid, threads, 0, stream>>>(mode, chunk, max_chunks, starts, qkvg, \
-            row_stride, v_off, g_off, qk, decay, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, out, act, joined, raw); }
-    if (dim <= 32) RET_CASE(32)
-    else if (dim <= 64) RET_CASE(64)
-    else if (dim <= 128) RET_CASE(128)
-    else RET_CASE(256)
-#undef RET_CASE
 }
 
 // qk: room for n_tokens * heads * 2 * pad floats (the rotated q and k; pad = palm_retention_pad(dim)).  chunk == 0: every sequence's run in one block
@@ -236,26 +69,19 @@ PALM_API int palm_retention(hipStream_t stream, const void* qkvg, int dtype, int
     const int max_chunks = chunk > 0 ? (max_new + chunk - 1) / chunk : 1;
     PALM_CHECK(heads <= 65535 && (long long)n_seqs * max_chunks <= 65535, "retention: %d heads / %d sequences x %d chunks are more than one launch takes",
                heads, n_seqs, max_chunks);
-    const int threads = (vdim + WAVE - 1) / WAVE * WAVE;
-    dim3 grid(heads, n_seqs * max_chunks);
     const int pad = palm_retention_pad(dim);
     const long long rot_threads = (long long)n_tokens * heads * pad;
+#define RET_CASE(D) linear_recurrence_sized<T, D, false>(stream, n_seqs, max_new, chunk, starts, nullptr, (const T*)qkvg, row_stride, v_off, g_off, qk, \
+            decay, nullptr, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, act, joined, raw)
     PALM_DTYPE_SWITCH(dtype, T, {
         retention_rotate_kernel<T><<<(unsigned)((rot_threads + 255) / 256), 256, 0, stream>>>((const T*)qkvg, row_stride, q_off, k_off, cos_t,
                                                                                              sin_t, rot, k_scale, act, n_tokens, heads, dim, pad, qk);
-        if (chunk == 0) {
-            retention_launch<T>(stream, grid, threads, RET_WHOLE, 1 << 30, 1, nullptr, (const T*)qkvg, row_stride, v_off, g_off, qk, decay,
-                                eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, act, joined, raw);
-        } else {
-            retention_launch<T>(stream, grid, threads, RET_LOCAL, chunk, max_chunks, starts, (const T*)qkvg, row_stride, v_off, g_off, qk,
-                                decay, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, act, joined, raw);
-            const int elems = heads * dim * vdim;
-            retention_starts_kernel<<<dim3((elems + 255) / 256, n_seqs), 256, 0, stream>>>(starts, state, decay, seq_slot, seq_new, chunk,
-                                                                                         max_chunks, heads, dim * vdim);
-            retention_launch<T>(stream, grid, threads, RET_FROM_STARTS, chunk, max_chunks, starts, (const T*)qkvg, row_stride, v_off, g_off,
-                                qk, decay, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, act, joined, raw);
-        }
+        if (pad == 32) RET_CASE(32);
+        else if (pad == 64) RET_CASE(64);
+        else if (pad == 128) RET_CASE(128);
+        else RET_CASE(256);
     });
+#undef RET_CASE
     PALM_LAUNCHED();
     return 0;
 }

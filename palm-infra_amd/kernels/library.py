@@ -20,6 +20,8 @@ Libraries:
                         rows), and the stream of blocks that norm a branch's output; loaded when a model has such a part
   ``feedforward``       routed experts (routing by softmax or by scores in groups, experts gated or plain) and the
                         activations of plain feed-forwards
+  ``gla_d<N>``          gated linear attention (a decay for every key channel and token), compiled for key sizes up to N
+  ``delta_head_d<N>``   the delta rule with one decay a head behind short convolutions, compiled for key sizes up to N
   ``streams``           a residual stream in several copies with learned weights between them, and its norms
   ``mlstm``             a matrix memory with input and forget gates per head and token
   ``latent_attention_k<K>_v<V>``  attention over compressed rows for prompts on the matrix cores, compiled for rows up to
@@ -64,10 +66,16 @@ FEEDFORWARD_SOURCES = ["moe.hip", "moe_grouped.hip", "activation.hip"]
 STREAMS_SOURCES = ["streams.hip"]
 MLSTM_SOURCES = ["mlstm.hip"]
 RECURRENT_SOURCES = ["retention.hip"]
+GLA_SOURCES = ["gla.hip"]
+DELTA_HEAD_SOURCES = ["delta_head.hip"]
 SINK_ATTENTION_SOURCES = ["attention_sink.hip"]
 SINK_ATTENTION_MFMA_SOURCES = ["attention_sink_mfma.hip"]
 BRANCH_SOURCES = ["branch_scaled.hip"]
 HEADERS = ["common.h", "mfma.h", "linear_thin.h", "linear_wide.h", "attention_api.h"]
+# headers of a few sources only: a change of one rebuilds the libraries of the sources that include it
+OWN_HEADERS = {"retention.hip": ["linear_recurrence.h"], "gla.hip": ["linear_recurrence.h"], "delta_rule.hip": ["delta_rule.h"],
+               "delta_head.hip": ["delta_rule.h", "conv_state.h"], "mamba.hip": ["conv_state.h"], "moe.hip": ["expert_form.h"],
+               "moe_grouped.hip": ["expert_form.h"], "branch_scaled.hip": ["expert_form.h"]}
 
 
 class KernelBuildError(RuntimeError):
@@ -116,7 +124,8 @@ def _existing(names) -> list[str]:
 def _digest(sources, defines) -> str:
     h = hashlib.sha256()
     h.update(" ".join(FLAGS + sorted(defines)).encode())
-    for name in sorted(_existing(list(sources) + HEADERS)):
+    own = {h for s in sources for h in OWN_HEADERS.get(s, ())}
+    for name in sorted(_existing(list(sources) + HEADERS + sorted(own))):
         h.update(name.encode())
         h.update((CSRC / name).read_bytes())
     return h.hexdigest()[:16]
@@ -211,6 +220,10 @@ def _spec(name: str):
         return STREAMS_SOURCES, ()
     if name == "mlstm":
         return MLSTM_SOURCES, ()
+    if name.startswith("gla_d"):
+        return GLA_SOURCES, (f"PALM_GLA_DIM={int(name[len('gla_d'):])}",)
+    if name.startswith("delta_head_d"):
+        return DELTA_HEAD_SOURCES, (f"PALM_DELTA_DIM={int(name[len('delta_head_d'):])}",)
     if name.startswith("sink_attention_k"):
         kk, vt = name[len("sink_attention_k"):].split("_v")
         return SINK_ATTENTION_MFMA_SOURCES, (f"PALM_SINK_KK={int(kk)}", f"PALM_SINK_VT={int(vt)}")

@@ -812,18 +812,18 @@ _SINK_SIGNATURES = {
                             c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                             c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int],
     "palm_sink_attention": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
-                            c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_float, c_void_p, c_void_p, c_int,
-                            c_int, c_int, c_void_p, c_void_p],
+                            c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_int, c_float, c_void_p,
+                            c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
 }
 _FEEDFORWARD_SIGNATURES = {
     "palm_moe_route": [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
-    "palm_moe_route_scored": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_float, c_void_p, c_void_p],
+    "palm_moe_route_scored": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p],
     "palm_add_gated_rows": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int],
     "palm_moe_experts": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                         c_void_p, c_void_p, c_int],
+                         c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p],
     "palm_moe_tile_tokens": [],
     "palm_moe_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
-                         c_void_p, c_void_p, c_int],
+                         c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p],
     "palm_gather_rows": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
     "palm_scatter_add": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "palm_activation": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_longlong],
@@ -842,7 +842,19 @@ _MLSTM_SIGNATURES = {
 _BRANCH_SIGNATURES = {
     "palm_add_scaled_normed": [c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_float, c_int, c_void_p, c_void_p, c_float, c_void_p,
                                c_int, c_int, c_int, c_void_p, c_int],
-    "palm_capped_gate": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_float],
+    "palm_capped_gate": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_float, c_float],
+}
+_GLA_SIGNATURES = {
+    "palm_gla_pad": [],
+    "palm_gla": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_float, c_float,
+                 c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_void_p,
+                 c_void_p, c_int, c_void_p],
+}
+_DELTA_HEAD_SIGNATURES = {
+    "palm_delta_head_pad": [],
+    "palm_delta_head": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                        c_void_p, c_void_p, c_void_p, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                        c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p],
 }
 _small_libraries: dict = {}
 
@@ -881,6 +893,21 @@ def streams_lib():
 
 def mlstm_lib():
     return _small("mlstm", _MLSTM_SIGNATURES)
+
+
+def padded_key_size(dim: int) -> int:
+    """The key size that a recurrence over keys of ``dim`` is compiled for."""
+    _need(1 <= dim <= 256, f"a key size of {dim} lies outside 1 to 256")
+    return 32 if dim <= 32 else 64 if dim <= 64 else 128 if dim <= 128 else 256
+
+
+def gla_lib(dim: int):
+    """The library compiled for this key size (built when a model of this size first runs)."""
+    return _small(f"gla_d{padded_key_size(dim)}", _GLA_SIGNATURES)
+
+
+def delta_head_lib(dim: int):
+    return _small(f"delta_head_d{padded_key_size(dim)}", _DELTA_HEAD_SIGNATURES)
 
 
 def add_normed(x: torch.Tensor, delta: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
@@ -982,6 +1009,42 @@ def retention(qkvg: torch.Tensor, heads: int, dim: int, vdim: int, decay: torch.
         library.call(recurrent(), "palm_joined_norm_gate", _stream(), _p(raw), _p(joined_norm), float(eps),
                      qkvg.data_ptr() + g_off * qkvg.element_size(), _code(qkvg, "retention"), qkvg.shape[1], int(gate_sigmoid), n,
                      heads * vdim, _p(out))
+    return out
+
+
+def gla(rows: torch.Tensor, low: torch.Tensor, w2: torch.Tensor, bias: torch.Tensor, tau: float, norm_w: torch.Tensor, heads: int, dim: int,
+        vdim: int, q_scale: float, eps: float, state: torch.Tensor, ctx, col0: int = 0, chunk: int | None = None) -> torch.Tensor:
+    """The step's tokens through gated linear attention.  rows [n, >= col0 + heads * (2 dim + 2 vdim)]: q | k | v | gate from
+    column col0; low float32 [n, rank] (a view of wider rows is fine), w2 float32 [rank, heads * dim] and bias float32
+    [heads * dim]: the decays are sigmoid(low w2 + bias)^(1/tau), one for every key channel; state float32 [slots, heads, dim,
+    vdim], read and left updated.  Returns [n, heads * vdim]: every head's output normed over vdim with ``norm_w`` and times
+    silu of the gate.  ``chunk``: see ``retention_chunk`` (None: chosen here)."""
+    what = "gla"
+    _dev(what, rows, w2, bias, norm_w, state, ctx.seq_slot, ctx.seq_new, ctx.cu_new)
+    _i32(what, ctx.seq_slot, ctx.seq_new, ctx.cu_new)
+    n, rank = rows.shape[0], w2.shape[0]
+    _need(rows.dim() == 2 and col0 >= 0 and rows.shape[1] >= col0 + heads * (2 * dim + 2 * vdim) and n == ctx.n_tokens,
+          f"{what}: rows {tuple(rows.shape)} from column {col0} are not [{ctx.n_tokens}, {heads} * (2*{dim} + 2*{vdim})]")
+    _need(low.is_cuda and low.dtype == F32 and low.shape == (n, rank) and (n == 0 or low.stride(1) == 1),
+          f"{what}: the decays' inputs are float32 [{n}, {rank}] with contiguous rows, not {low.dtype} {tuple(low.shape)}")
+    _need(w2.shape == (rank, heads * dim) and w2.dtype == F32 and bias.shape == (heads * dim,) and bias.dtype == F32 and norm_w.shape == (vdim,)
+          and norm_w.dtype == F32, f"{what}: the decays' weights [{rank}, {heads * dim}] and bias and the norm's weight [{vdim}] are float32")
+    _need(state.dim() == 4 and state.shape[1:] == (heads, dim, vdim) and state.dtype == F32,
+          f"{what}: state {tuple(state.shape)} {state.dtype} is not float32 [slots, {heads}, {dim}, {vdim}]")
+    lib = gla_lib(dim)
+    out = torch.empty((n, heads * vdim), dtype=rows.dtype, device=rows.device)
+    prep = torch.empty((n, heads, 3, lib.palm_gla_pad()), dtype=F32, device=rows.device)
+    chunk = retention_chunk(ctx.n_seqs, heads, ctx.max_new) if chunk is None else int(chunk)
+    starts = keeps = None
+    if chunk:
+        chunks = ctx.n_seqs * (-(-ctx.max_new // chunk))
+        starts = torch.empty((chunks, heads, dim, vdim), dtype=F32, device=rows.device)
+        keeps = torch.empty((chunks, heads, dim), dtype=F32, device=rows.device)
+    q_off, v_off = col0, col0 + 2 * heads * dim
+    library.call(lib, "palm_gla", _stream(), _p(rows), _code(rows, what), rows.shape[1], q_off, q_off + heads * dim, v_off, v_off + heads * vdim,
+                 _p(low), low.stride(0), _p(w2), _p(bias), rank, float(tau), float(q_scale), _p(norm_w), float(eps), _p(state), _p(ctx.seq_slot),
+                 _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs, heads, dim, vdim, _p(out), int(ctx.max_new), chunk, _p(starts), _p(keeps), n,
+                 _p(prep))
     return out
 
 
@@ -1237,6 +1300,49 @@ def delta_rule(u: torch.Tensor, offsets: tuple, b: torch.Tensor, a: torch.Tensor
     return out
 
 
+def delta_head(rows: torch.Tensor, ab: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor,
+               norm_w: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, q_scale: float, unit_eps: float, eps: float,
+               state: torch.Tensor, ctx, col0: int = 0, chunk: int | None = None) -> torch.Tensor:
+    """The step's tokens through a gated delta rule with one decay a head, from the projections to the gated heads.
+
+    rows [n, >= col0 + 2 kv_heads dim + 2 heads vdim]: q | k | v | gate from column col0; ab float32 [n, 2 heads] (a view of wider
+    rows is fine): the write strengths before their sigmoid, then the decays before bias and softplus; conv_w float32 [channels
+    of q | k | v, taps] with conv_state float32 [slots, taps - 1, channels], and state float32 [slots, heads, dim, vdim], both
+    read and left updated.  Returns [n, heads * vdim]: the heads' outputs, each normed over vdim with ``norm_w`` and times silu
+    of the gate.  ``chunk``: see ``delta_chunk`` (None: chosen here)."""
+    what = "delta_head"
+    _dev(what, rows, conv_w, conv_state, a_log, dt_bias, norm_w, state, ctx.tok_slot, ctx.seq_slot, ctx.seq_new, ctx.cu_new)
+    _i32(what, ctx.tok_slot, ctx.seq_slot, ctx.seq_new, ctx.cu_new)
+    n, channels = rows.shape[0], 2 * kv_heads * dim + heads * vdim
+    taps = conv_w.shape[1]
+    _need(rows.dim() == 2 and col0 >= 0 and rows.shape[1] >= col0 + channels + heads * vdim and n == ctx.n_tokens,
+          f"{what}: rows {tuple(rows.shape)} from column {col0} do not hold q, k ({kv_heads} x {dim}), v and gate ({heads} x {vdim}) of {ctx.n_tokens} tokens")
+    _need(ab.is_cuda and ab.dtype == F32 and ab.shape == (n, 2 * heads) and (n == 0 or ab.stride(1) == 1),
+          f"{what}: write strengths and decays are float32 [{n}, {2 * heads}] with contiguous rows, not {ab.dtype} {tuple(ab.shape)}")
+    _need(conv_w.shape == (channels, taps) and conv_w.dtype == F32 and conv_state.dim() == 3 and conv_state.shape[1:] == (taps - 1, channels)
+          and conv_state.dtype == F32, f"{what}: convolution {tuple(conv_w.shape)} with kept inputs {tuple(conv_state.shape)} for {channels} channels")
+    for t, shape, nm in ((a_log, (heads,), "A_log"), (dt_bias, (heads,), "dt_bias"), (norm_w, (vdim,), "the norm's weight")):
+        _need(tuple(t.shape) == shape and t.dtype == F32, f"{what}: {nm} is float32 {shape}, not {t.dtype} {tuple(t.shape)}")
+    _need(state.dim() == 4 and state.shape[1:] == (heads, dim, vdim) and state.dtype == F32,
+          f"{what}: state {tuple(state.shape)} {state.dtype} is not float32 [slots, {heads}, {dim}, {vdim}]")
+    lib, dev = delta_head_lib(dim), rows.device
+    out = torch.empty((n, heads * vdim), dtype=rows.dtype, device=dev)
+    prep = torch.empty((n, kv_heads, 2, lib.palm_delta_head_pad()), dtype=F32, device=dev)
+    values = torch.empty((n, heads * vdim), dtype=F32, device=dev)
+    beta, decay = torch.empty((2, n, heads), dtype=F32, device=dev)
+    chunk = delta_chunk(ctx.n_seqs, heads, ctx.max_new) if chunk is None else int(chunk)
+    ext = starts = None
+    if chunk:
+        chunks = ctx.n_seqs * (-(-ctx.max_new // chunk))
+        ext = torch.empty((chunks, heads, dim, vdim + dim), dtype=F32, device=dev)
+        starts = torch.empty((chunks, heads, dim, vdim), dtype=F32, device=dev)
+    library.call(lib, "palm_delta_head", _stream(), _p(rows), _code(rows, what), rows.shape[1], col0, col0 + channels, _p(conv_w), taps,
+                 _p(conv_state) if taps > 1 else None, _p(ctx.tok_slot), _p(ab), ab.stride(0), 0, heads, _p(a_log), _p(dt_bias), _p(norm_w),
+                 float(q_scale), float(unit_eps), float(eps), _p(state), _p(ctx.seq_slot), _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs, n,
+                 heads, kv_heads, dim, vdim, _p(out), _p(prep), _p(values), _p(beta), _p(decay), int(ctx.max_new), chunk, _p(ext), _p(starts))
+    return out
+
+
 # ---- attention over one compressed row per position -----------------------------------------------------------------
 
 def latent_prep(down: torch.Tensor, q_rank: int, kv_off: int, kv_rank: int, rot_dim: int, q_norm_w, kv_norm_w, eps: float,
@@ -1402,44 +1508,68 @@ def moe_route(logits: torch.Tensor, top: int):
     return chosen, weight
 
 
-EXPERT_FORMS = {"gated_silu": 0, "gelu": 1}
+EXPERT_FORMS = {"gated_silu": 0, "gelu": 1, "capped_gated": 2}
+NO_CAP = (1.0, 1.0, 0.0)           # limit, slope, shift: what the other forms pass and do not read
+
+
+def expert_rows(form: str) -> int:
+    """Rows of an expert's first matrix for each inner value: gated experts have a gate row and an up row."""
+    return 1 if form == "gelu" else 2
+
+
+def _addends(what: str, add, h):
+    """Up to two tensors of rows that other branches made, as addresses (None where there is none)."""
+    _need(len(add) <= 2, f"{what}: {len(add)} rows to add (at most two)")
+    for y in add:
+        _dev(what, y)
+        _need(y.shape == h.shape and y.dtype == h.dtype, f"{what}: rows to add are {h.dtype} {tuple(h.shape)}, not {y.dtype} {tuple(y.shape)}")
+    return [_p(y) for y in add] + [None] * (2 - len(add))
 
 
 def _expert_shapes(what, h, up, down, ff, form):
     """-> (experts, rows of an expert's first matrix): gated experts keep their gate rows before their up rows."""
     _need(form in EXPERT_FORMS, f"{what}: an expert's form {form!r} is not one of {sorted(EXPERT_FORMS)}")
-    per = (2 if form == "gated_silu" else 1) * ff
+    per = expert_rows(form) * ff
     width = h.shape[1]
     _need(up.dim() == 2 and up.shape[1] == width and up.shape[0] % per == 0 and down.shape == (up.shape[0] // per * width, ff)
           and up.dtype == down.dtype, f"{what}: first matrices {tuple(up.shape)}, down {tuple(down.shape)} for width {width}, inner size {ff}")
     return up.shape[0] // per
 
 
-def moe_route_scored(logits: torch.Tensor, experts: int, top: int, correction: torch.Tensor | None, groups: int, keep: int, scale: float):
-    """logits float32 [n, >= experts] (the experts' columns first) -> (chosen int32 [n, top], weight float32 [n, top]).  The
-    scores are sigmoid(logit); the choice is made by score + ``correction``; the experts lie in ``groups`` equal groups of
-    neighbours, a group ranks by the sum of its two largest corrected scores, and only experts of the best ``keep`` groups can
+ROUTER_SCORES = {"sigmoid": 0, "softmax": 1}
+GROUP_SCORES = {"two_largest": 0, "largest": 1}
+
+
+def moe_route_scored(logits: torch.Tensor, experts: int, top: int, correction: torch.Tensor | None, groups: int, keep: int, scale: float,
+                     score: str = "sigmoid", group_score: str = "two_largest"):
+    """logits float32 [n, >= experts] (the experts' columns first; a view of wider rows is fine) -> (chosen int32 [n, top], weight float32 [n, top]).  The
+    scores are sigmoid(logit), or with ``score`` "softmax" the softmax over all experts; the choice is made by score +
+    ``correction`` (None: the score); the experts lie in ``groups`` equal groups of neighbours, a group ranks by the sum of its
+    two largest corrected scores (``group_score`` "largest": by its largest), and only experts of the best ``keep`` groups can
     be chosen (the lower index wins a tie); the weights are the chosen scores over their sum (+ 1e-20), times ``scale``."""
-    _dev("moe_route_scored", logits, correction)
-    _need(logits.dim() == 2 and logits.dtype == F32 and logits.shape[1] >= experts, f"moe_route_scored: router logits are float32 [n, >= {experts}], "
+    _dev("moe_route_scored", correction)
+    _need(logits.is_cuda and logits.dim() == 2 and (logits.shape[0] == 0 or logits.stride(1) == 1) and logits.dtype == F32 and logits.shape[1] >= experts, f"moe_route_scored: router logits are float32 [n, >= {experts}], "
           f"not {logits.dtype} {tuple(logits.shape)}")
+    _need(score in ROUTER_SCORES and group_score in GROUP_SCORES, f"moe_route_scored: score {score!r} is one of {sorted(ROUTER_SCORES)}, group_score "
+          f"{group_score!r} one of {sorted(GROUP_SCORES)}")
     _need(correction is None or (correction.shape == (experts,) and correction.dtype == F32), f"moe_route_scored: the correction is float32 [{experts}]")
     n = logits.shape[0]
     chosen = torch.empty((n, top), dtype=torch.int32, device=logits.device)
     weight = torch.empty((n, top), dtype=F32, device=logits.device)
-    library.call(feedforward(), "palm_moe_route_scored", _stream(), _p(logits), logits.shape[1], n, int(experts), int(top), _p(correction),
-                 int(groups), int(keep), float(scale), _p(chosen), _p(weight))
+    library.call(feedforward(), "palm_moe_route_scored", _stream(), _p(logits), logits.stride(0), n, int(experts), int(top), _p(correction),
+                 int(groups), int(keep), float(scale), ROUTER_SCORES[score], GROUP_SCORES[group_score], _p(chosen), _p(weight))
     return chosen, weight
 
 
 def add_gated_rows(out: torch.Tensor, y: torch.Tensor, logits: torch.Tensor, column: int) -> torch.Tensor:
     """out[t] += sigmoid(logits[t, column]) * y[t]: out float32 [n, width] in place, logits float32 [n, *]."""
-    _dev("add_gated_rows", out, y, logits)
+    _dev("add_gated_rows", out, y)
+    _need(logits.is_cuda and (logits.shape[0] == 0 or logits.stride(1) == 1), "add_gated_rows: the gate's rows are contiguous and on the GPU")
     _need(out.dim() == 2 and out.dtype == F32 and y.shape == out.shape and logits.dim() == 2 and logits.dtype == F32
           and logits.shape[0] == out.shape[0] and 0 <= column < logits.shape[1],
           f"add_gated_rows: out {tuple(out.shape)} {out.dtype}, y {tuple(y.shape)}, gate column {column} of {tuple(logits.shape)} {logits.dtype}")
     library.call(feedforward(), "palm_add_gated_rows", _stream(), _p(out), _p(y), _code(y, "add_gated_rows"),
-                 logits.data_ptr() + column * 4, logits.shape[1], out.shape[0], out.shape[1])
+                 logits.data_ptr() + column * 4, logits.stride(0), out.shape[0], out.shape[1])
     return out
 
 
@@ -1456,10 +1586,11 @@ def activation(z: torch.Tensor, kind: str) -> torch.Tensor:
 
 
 def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, ff: int,
-                form: str = "gated_silu") -> torch.Tensor:
+                form: str = "gated_silu", cap=NO_CAP, add=()) -> torch.Tensor:
     """Every row through its chosen experts, nothing planned on the host: h [n, width]; gate_up [experts * 2 ff, width] (an
-    expert's gate rows, then its up rows; ``form`` "gelu": [experts * ff, width], up rows alone, through the exact gelu);
-    down [experts * width, ff].  Returns float32 [n, width], the weighted sum."""
+    expert's gate rows, then its up rows; ``form`` "gelu": [experts * ff, width], up rows alone, through the exact gelu; ``form``
+    "capped_gated": gate and up rows, capped as ``cap`` = (limit, slope, shift) says); down [experts * width, ff].  Returns float32
+    [n, width], the weighted sum plus the rows ``add`` (up to two [n, width] of h's type that other branches made)."""
     what = "moe_experts"
     _dev(what, h, gate_up, down, chosen, weight)
     _i32(what, chosen)
@@ -1470,7 +1601,7 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chos
     mid = torch.empty((n, top, ff), dtype=F32, device=h.device)
     out = torch.empty((n, width), dtype=F32, device=h.device)
     library.call(feedforward(), "palm_moe_experts", _stream(), _p(h), _code(h, what), _p(gate_up), _p(down), _code(gate_up, what + " weights"),
-                 _p(chosen), _p(weight), n, top, width, ff, _p(mid), _p(out), EXPERT_FORMS[form])
+                 _p(chosen), _p(weight), n, top, width, ff, _p(mid), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h))
     return out
 
 
@@ -1480,7 +1611,7 @@ def moe_grouped_serves(h: torch.Tensor, gate_up: torch.Tensor, ff: int) -> bool:
 
 
 def moe_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, ff: int,
-                form: str = "gated_silu") -> torch.Tensor:
+                form: str = "gated_silu", cap=NO_CAP, add=()) -> torch.Tensor:
     """Every row through its chosen experts, for many rows, planned on the device: the (row, choice) pairs grouped by expert,
     two grouped products on the matrix cores, the weighted sum in the order of the choices.  Shapes as ``moe_experts``;
     returns float32 [n, width]."""
@@ -1501,7 +1632,7 @@ def moe_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chos
     y = torch.empty((slots, width), dtype=BF16, device=h.device)
     out = torch.empty((n, width), dtype=F32, device=h.device)
     library.call(feedforward(), "palm_moe_grouped", _stream(), _p(h), _p(gate_up), _p(down), _p(chosen), _p(weight), n, top, experts, width, ff,
-                 _p(plan), _p(mid), _p(y), _p(out), EXPERT_FORMS[form])
+                 _p(plan), _p(mid), _p(y), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h))
     return out
 
 
@@ -1527,7 +1658,7 @@ def scatter_add(out: torch.Tensor, y: torch.Tensor, rows: torch.Tensor, weight: 
 
 # ---- softmax attention with a sink, a window and a gate (library ``sink_attention``) -------------------------------
 
-SINK_NORMS = {None: 0, "projection": 1, "head": 2}
+SINK_NORMS = {None: 0, "projection": 1, "head": 2, "head_unit": 2}       # (head_unit: per head, without a weight)
 SINK_BLOCKS_WANTED = 1024         # a decode step's key ranges are cut into slices until about this many blocks run
 
 
@@ -1540,7 +1671,7 @@ def sink_qkv_store(rows: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim
     """q, k and v of the step's tokens from ``rows`` [n, >= heads*dim + kv_heads*dim + kv_heads*vdim] (q | k | v | whatever
     follows): ``bias`` (float32 over q | k | v, or None) is added, q and k are normed (``norm``: "projection": one RMS norm
     over the whole q row and one over the whole k row, weights of those sizes; "head": per head, weights of the key size;
-    None), their first ``rot`` dimensions are rotated by the tokens' cos and sin rows (``pairing``: dimension i with i + rot/2,
+    "head_unit": per head, no weights; None), their first ``rot`` dimensions are rotated by the tokens' cos and sin rows (``pairing``: dimension i with i + rot/2,
     or 2i with 2i + 1), k and v go to their pages, and q comes back as [n, heads, dim].  ``col0``: q begins at this column of
     the rows.
 
@@ -1562,7 +1693,9 @@ def sink_qkv_store(rows: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim
     _need(pairing in ROTARY_PAIRINGS, f"sink_qkv_store: pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
     if bias is not None:
         _need(bias.shape == (channels,) and bias.dtype == F32, f"sink_qkv_store: the bias is float32 [{channels}]")
-    if norm is not None:
+    if norm == "head_unit":
+        _need(q_w is None and k_w is None, "sink_qkv_store: unit heads have no weights")
+    elif norm is not None:
         want = (q_size, kv_heads * dim) if norm == "projection" else (dim, dim)
         _need(q_w is not None and k_w is not None and q_w.shape == (want[0],) and k_w.shape == (want[1],) and q_w.dtype == F32
               and k_w.dtype == F32, f"sink_qkv_store: the norm weights are float32 [{want[0]}] and [{want[1]}]")
@@ -1607,9 +1740,10 @@ def sink_slices(ctx, heads: int, kv_heads: int, window: int | None) -> int:
 
 def sink_attention_exact(q: torch.Tensor, k_cache, v_cache, block_table, ctx, heads: int, kv_heads: int, dim: int, vdim: int,
                          scale: float, window: int | None, sink, gate: torch.Tensor | None, gate_off: int = 0,
-                         slices: int | None = None, gate_per_head: bool = False) -> torch.Tensor:
+                         slices: int | None = None, gate_per_head: bool = False, chunked: bool = False, slopes=None) -> torch.Tensor:
     """Attention of the step's queries q [n, heads, dim] over the cached keys of their sequences up to their own positions
-    (the last ``window`` if given), with a sink in the denominator: ``sink`` is its score for all heads, or a float32 tensor
+    (the last ``window`` if given; with ``chunked`` those of the query's own chunk of ``window`` positions, counted from the
+    sequence's start), head h's scores less slopes[h] times the distance (``slopes`` float32 [heads] or None), with a sink in the denominator: ``sink`` is its score for all heads, or a float32 tensor
     [heads] of learned scores, or None.  ``gate``: a tensor [n, >= gate_off + heads*vdim] whose columns from ``gate_off`` on
     gate the output through a sigmoid (None: no gate); with ``gate_per_head`` one column for each head.  Returns
     [n, heads * vdim].  32-bit arithmetic whatever the elements' type."""
@@ -1621,12 +1755,13 @@ def sink_attention_exact(q: torch.Tensor, k_cache, v_cache, block_table, ctx, he
           and v_cache.shape[1:] == (kv_heads, vdim, PAGE_TOKENS), f"sink_attention: cache {tuple(k_cache.shape)} / {tuple(v_cache.shape)}")
     gate_ptr, gate_stride = _sink_gate("sink_attention", gate, gate_off, n, heads, vdim, q.dtype, gate_per_head)
     sink_score, sink_scores = _sink_scores("sink_attention", sink, heads, q.device)
+    _sink_slopes("sink_attention", slopes, heads, window, chunked)
     slices = sink_slices(ctx, heads, kv_heads, window) if slices is None else int(slices)
     work = torch.empty((n * heads * slices * (vdim + 2),), dtype=F32, device=q.device) if slices > 1 else None
     out = torch.empty((n, heads * vdim), dtype=q.dtype, device=q.device)
     library.call(sink_attention_lib(), "palm_sink_attention", _stream(), _p(q), _code(q, "sink_attention"), _p(k_cache), _p(v_cache),
                  _p(block_table), block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs,
-                 int(ctx.max_new), n, heads, kv_heads, dim, vdim, float(scale), int(window or 0), int(sink is not None),
+                 int(ctx.max_new), n, heads, kv_heads, dim, vdim, float(scale), int(window or 0), int(chunked), _p(slopes), int(sink is not None),
                  sink_score, _p(sink_scores), gate_ptr, gate_stride, int(gate_per_head), slices, _p(work), _p(out))
     return out
 
@@ -1650,8 +1785,15 @@ def _sink_scores(what: str, sink, heads: int, device):
     return float(sink or 0.0), None
 
 
+def _sink_slopes(what: str, slopes, heads: int, window, chunked: bool) -> None:
+    if slopes is not None:
+        _dev(what, slopes)
+        _need(slopes.shape == (heads,) and slopes.dtype == F32, f"{what}: the distance bias's slopes are float32 [{heads}], not {slopes.dtype} {tuple(slopes.shape)}")
+    _need(window or not chunked, f"{what}: chunks need their size")
+
+
 _SINK_MFMA_SIGNATURE = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
-                        c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_void_p]
+                        c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_void_p]
 _sink_mfma_libs: dict = {}
 
 
@@ -1673,7 +1815,7 @@ def sink_attention_mfma_lib(dim: int, vdim: int):
 
 def sink_attention_mfma(q: torch.Tensor, k_cache, v_cache, block_table, ctx, heads: int, kv_heads: int, dim: int, vdim: int,
                         scale: float, window: int | None, sink, gate: torch.Tensor | None, gate_off: int = 0,
-                        gate_per_head: bool = False) -> torch.Tensor:
+                        gate_per_head: bool = False, chunked: bool = False, slopes=None) -> torch.Tensor:
     """``sink_attention_exact`` for prompts in bfloat16 on the matrix cores (scores, weights and sums 32-bit)."""
     _dev("sink_attention_mfma", q, k_cache, v_cache, block_table, gate, ctx.seq_slot, ctx.seq_start, ctx.seq_new, ctx.cu_new)
     _i32("sink_attention_mfma", block_table, ctx.seq_slot, ctx.seq_start, ctx.seq_new, ctx.cu_new)
@@ -1684,23 +1826,24 @@ def sink_attention_mfma(q: torch.Tensor, k_cache, v_cache, block_table, ctx, hea
           and v_cache.shape[1:] == (kv_heads, vdim, PAGE_TOKENS), f"sink_attention_mfma: cache {tuple(k_cache.shape)} / {tuple(v_cache.shape)}")
     gate_ptr, gate_stride = _sink_gate("sink_attention_mfma", gate, gate_off, n, heads, vdim, BF16, gate_per_head)
     sink_score, sink_scores = _sink_scores("sink_attention_mfma", sink, heads, q.device)
+    _sink_slopes("sink_attention_mfma", slopes, heads, window, chunked)
     out = torch.empty((n, heads * vdim), dtype=BF16, device=q.device)
     library.call(sink_attention_mfma_lib(dim, vdim), "palm_sink_attention_mfma", _stream(), _p(q), _p(k_cache), _p(v_cache), _p(block_table),
                  block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs, int(ctx.max_new),
-                 heads, kv_heads, dim, vdim, float(scale), int(window or 0), int(sink is not None), sink_score, _p(sink_scores), gate_ptr,
-                 gate_stride, int(gate_per_head), _p(out))
+                 heads, kv_heads, dim, vdim, float(scale), int(window or 0), int(chunked), _p(slopes), int(sink is not None), sink_score,
+                 _p(sink_scores), gate_ptr, gate_stride, int(gate_per_head), _p(out))
     return out
 
 
 def sink_attention(q, k_cache, v_cache, block_table, ctx, heads, kv_heads, dim, vdim, scale, window, sink, gate, gate_off=0,
-                   gate_per_head=False):
+                   gate_per_head=False, chunked=False, slopes=None):
     """The kernel that serves: the matrix cores for prompts in bfloat16, the exact one for the float32 mode, for single
     tokens, and for sizes that the matrix-core kernel does not take."""
     if not ctx.is_decode and sink_mfma_serves(q, dim, vdim):
         return sink_attention_mfma(q, k_cache, v_cache, block_table, ctx, heads, kv_heads, dim, vdim, scale, window, sink, gate, gate_off,
-                                   gate_per_head=gate_per_head)
+                                   gate_per_head=gate_per_head, chunked=chunked, slopes=slopes)
     return sink_attention_exact(q, k_cache, v_cache, block_table, ctx, heads, kv_heads, dim, vdim, scale, window, sink, gate, gate_off,
-                                gate_per_head=gate_per_head)
+                                gate_per_head=gate_per_head, chunked=chunked, slopes=slopes)
 
 
 # ---- branches scaled by a learned vector; the capped feed-forward gate (library ``branches``) ---------------------
@@ -1730,12 +1873,13 @@ def add_scaled_normed(x: torch.Tensor, terms, weights, scale: torch.Tensor | Non
 
 
 def capped_gate(gate_up: torch.Tensor, limit: float, slope: float, shift: float) -> torch.Tensor:
-    """[n, 2 ff] (gate | up) -> [n, ff]: g * sigmoid(slope * g) * (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit)."""
-    _dev("capped_gate", gate_up)
-    _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, f"capped_gate: rows {tuple(gate_up.shape)} are not [n, 2 ff]")
+    """[n, 2 ff] (gate | up; a view of wider rows is fine) -> [n, ff]: g * sigmoid(slope * g) * (u + shift), g = min(gate, limit),
+    u = clamp(up, -limit, limit)."""
+    _need(gate_up.is_cuda and gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0 and (gate_up.shape[0] == 0 or gate_up.stride(1) == 1),
+          f"capped_gate: rows {tuple(gate_up.shape)} on {gate_up.device} are not [n, 2 ff] with contiguous rows")
     n, ff = gate_up.shape[0], gate_up.shape[1] // 2
     out = torch.empty((n, ff), dtype=gate_up.dtype, device=gate_up.device)
-    library.call(branches(), "palm_capped_gate", _stream(), _p(gate_up), _p(out), _code(gate_up, "capped_gate"), n, ff, float(limit),
+    library.call(branches(), "palm_capped_gate", _stream(), _p(gate_up), gate_up.stride(0), _p(out), _code(gate_up, "capped_gate"), n, ff, float(limit),
                  float(slope), float(shift))
     return out
 

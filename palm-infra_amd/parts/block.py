@@ -25,11 +25,19 @@ one kernel.
 ``hyper_connections``: the residual stream runs in S copies x_1 .. x_S.  A sublayer reads u = sum_s in[s] x_s through its norm
 (a ``streams_in`` reader), and its output y goes into all streams at once, x_t <- sum_s mix[s, t] x_s + out[t] y (every new
 stream from the old ones).  A layer may have no feed-forward.  The write of one sublayer and the read of the next are one kernel.
+
+``parallel_pre_norm``: h = norm(x); x += mixer(h) + feed_forward(h): one norm, whose output both branches read.  A layer may have
+no feed-forward.  With the tensors ``in`` and ``in_exact`` (the branches' input matrices joined along their rows, the mixer's
+first; the second product's result is 32-bit) two products serve both branches, each of which takes its columns.  A feed-forward
+that takes an addend adds the mixer's output where it writes its own, so that the norm that reads x next adds one delta.
 """
 from __future__ import annotations
 
+import torch
+
 from ..kernels import ops
 from .base import cache_needs, cache_needs_beside_shared, register_part
+from .linear import Linear
 from .norm import PassThrough, StreamsReader
 from .residual import ResidualSink, WeightedSum, as_tensor, run_branch
 
@@ -251,3 +259,55 @@ class HyperConnectionsBlock:
         h = self._write(x, y, self.mixer_mix, self.mixer_out, self.feed_forward_norm, None)
         y = as_tensor(self.feed_forward.forward(h, ctx))
         return self._write(x, y, self.feed_forward_mix, self.feed_forward_out, sink.norm, sink.rows)
+
+
+@register_part("block", "parallel_pre_norm")
+class ParallelPreNormBlock:
+    def __init__(self, spec, builder):
+        self.norm = builder.build(spec.parts["norm"])
+        self.mixer = builder.build(spec.parts["mixer"])
+        self.feed_forward = builder.build(spec.parts["feed_forward"]) if "feed_forward" in spec.parts else None
+        self.shared = Linear(builder.tensor(spec, "in")) if "in" in spec.tensors else None
+        self.exact = Linear(builder.tensor(spec, "in_exact")) if "in_exact" in spec.tensors else None
+        branches = [p for p in (self.mixer, self.feed_forward) if p is not None]
+        if (self.shared is not None) != all(getattr(p, "shared_input", False) for p in branches):
+            raise ValueError("parallel branches: a shared input product and branches that take their rows from it come together")
+        if self.shared is not None:
+            for what, product, field in (("in", self.shared, "in_rows"), ("in_exact", self.exact, "exact_rows")):
+                rows = [getattr(p, field, 0) for p in branches]
+                if sum(rows) != (product.out_features if product is not None else 0):
+                    raise ValueError(f"parallel branches: the product {what!r} makes {product.out_features if product is not None else 0} columns, "
+                                     f"the branches take {rows}")
+
+    @property
+    def capturable(self) -> bool:
+        return all(getattr(p, "capturable", False) for p in (self.norm, self.mixer, self.feed_forward) if p is not None)
+
+    @staticmethod
+    def cache_needs(spec):
+        return cache_needs(spec.parts["mixer"])
+
+    @property
+    def entry_norm(self):
+        return self.norm
+
+    def forward(self, x, h, ctx, sink):
+        h = as_tensor(h)
+        mixer, ff = self.mixer, self.feed_forward
+        if self.shared is not None:
+            rows = self.shared(h)
+            exact = self.exact(h, out_dtype=torch.float32) if self.exact is not None else None
+            mixer_exact = getattr(mixer, "exact_rows", 0)
+            y = mixer.forward_rows(rows, 0, ctx, exact, 0) if mixer_exact else mixer.forward_rows(rows, 0, ctx)
+            run_ff = lambda **kw: ff.forward_rows(h, rows, mixer.in_rows, ctx, exact, mixer_exact, **kw)
+        else:
+            y = mixer.forward(h, ctx)
+            run_ff = lambda **kw: ff.forward(h, ctx, **kw)
+        y = as_tensor(y)
+        if ff is None:
+            return sink.finish(y)
+        if getattr(ff, "takes_addend", False):
+            return sink.finish(run_ff(addend=y))
+        delta = as_tensor(run_ff())
+        ops.add_scaled_normed(x, [y], [1.0], None, None, 0.0)              # x += y; the feed-forward's output goes in with the next norm
+        return sink.finish(delta)

@@ -75,3 +75,60 @@ class DeltaRule:
                            self.a_log, self.dt_bias, self.norm_w, self.nh, self.nqk, self.dk, self.dv, self.dk ** -0.5, UNIT_EPS,
                            self.eps, lc.states["delta"], ctx)
         return self.out(o)
+
+
+@register_part("mixer", "delta_rule_head")
+class DeltaRuleHeadDecay:
+    """The same rule with one decay a head instead of one for each key channel:
+
+        S <- g_t S;   u_t = beta_t (v_t - S^T k_t);   S <- S + k_t u_t^T;   o_t = S^T q_t
+
+    with g_t = exp(-exp(A_log_h) softplus(W_a h + dt_bias_h)) and beta_t = sigmoid(W_b h), both one number a head; each head's o_t
+    is normed over value_dim (one weight vector for all heads) and multiplied by silu of a whole gate projection.  One joined
+    product makes q | k | v | gate, one with a 32-bit result the rows of W_b and W_a; the convolutions (whose values stay 32-bit),
+    unit vectors, decays and write strengths are one pass before the recurrence."""
+    capturable = True
+
+    def __init__(self, spec, builder):
+        p = spec.params
+        self.hidden = int(p["hidden_size"])
+        self.nh, self.nqk, self.dk, self.dv = int(p["num_heads"]), int(p["num_qk_heads"]), int(p["key_dim"]), int(p["value_dim"])
+        self.taps, self.eps = int(p["taps"]), float(p["eps"])
+        if self.nh % self.nqk:
+            raise ValueError(f"delta rule: {self.nh} heads are not a multiple of {self.nqk} q/k heads")
+        t = lambda name: builder.tensor(spec, name)
+        self.channels = 2 * self.nqk * self.dk + self.nh * self.dv
+        # the input products are this part's own, or wider ones that the block makes for all its branches (``input`` "shared")
+        self.shared_input = p.get("input") == "shared"
+        self.in_rows, self.exact_rows = self.channels + self.nh * self.dv, 2 * self.nh
+        self.qkvg = None if self.shared_input else Linear(t("qkvg"))
+        self.ba = None if self.shared_input else Linear(t("ba"))
+        self.out = Linear(t("out"))
+        self.conv, self.a_log, self.dt_bias, self.norm_w = t("conv"), t("a_log"), t("dt_bias"), t("norm")
+        want = {"out": (self.out.weight, (self.hidden, self.nh * self.dv)), "conv": (self.conv, (self.channels, self.taps)),
+                "a_log": (self.a_log, (self.nh,)), "dt_bias": (self.dt_bias, (self.nh,)), "norm": (self.norm_w, (self.dv,))}
+        if not self.shared_input:
+            want.update({"qkvg": (self.qkvg.weight, (self.in_rows, self.hidden)), "ba": (self.ba.weight, (2 * self.nh, self.hidden))})
+        for name, (tensor, shape) in want.items():
+            if tuple(tensor.shape) != shape:
+                raise ValueError(f"delta rule: {name} is {tuple(tensor.shape)}, expected {shape}")
+
+    @staticmethod
+    def cache_needs(spec):
+        return DeltaRule.cache_needs(spec)
+
+    def forward(self, h, ctx):
+        if self.shared_input:
+            raise RuntimeError("a delta rule whose input products are shared gets its rows from the part that makes them")
+        return self.forward_rows(self.qkvg(h), 0, ctx, self.ba(h, out_dtype=torch.float32), 0)
+
+    def forward_rows(self, rows, col0, ctx, exact, exact_col0):
+        """``rows`` [n, >= col0 + in_rows]: q | k | v | gate from column ``col0``; ``exact`` float32: the rows of W_b, then of W_a,
+        from ``exact_col0``."""
+        lc = ctx.layer_cache
+        if lc is None or not lc.states or "delta" not in lc.states:
+            raise RuntimeError("the delta rule needs its state; the step gave it no cache")
+        o = ops.delta_head(rows, exact[:, exact_col0:exact_col0 + 2 * self.nh], self.conv, lc.states["delta_conv"], self.a_log, self.dt_bias,
+                           self.norm_w, self.nh, self.nqk, self.dk, self.dv, self.dk ** -0.5, UNIT_EPS, self.eps, lc.states["delta"], ctx,
+                           col0=col0)
+        return self.out(o)

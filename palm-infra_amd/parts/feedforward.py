@@ -18,13 +18,20 @@ limit); gate and up joined into one [2I, H] product.
 ``activation``, float32 [2]): for z > 0, softplus(p) z^2 + z/2; for z <= 0, (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2.
 ``relu_squared`` is max(z, 0)^2, ``gelu_erf`` the exact gelu, ``gelu_tanh`` its tanh form.
 
-``routed_scored``: ``experts`` plain feed-forwards down(gelu(up(h))) (the exact gelu, no biases) of which every token goes
+``routed_scored`` (as follows, with the options named at the end): ``experts`` plain feed-forwards down(gelu(up(h))) (the exact gelu, no biases) of which every token goes
 through ``top``.  The router's logits are 32-bit, the scores their sigmoid; the choice is made by score plus the tensor
 ``correction``, the weights by the scores without it: the chosen experts' scores over their sum (+ 1e-20), times ``scale``.
 With ``groups`` the experts lie in that many equal groups of neighbours, a group ranks by the sum of its two largest
 corrected scores, and only experts of the best ``keep`` groups can be chosen.  With ``shared_size`` one more expert of that
 inner size runs for every token and is added, times the sigmoid of one more router row (the last row of the tensor
-``router``), one number per token.  The experts run as those of ``routed_gated_silu`` do."""
+``router``), one number per token.  The experts run as those of ``routed_gated_silu`` do.
+
+Options of ``routed_scored``: ``form`` "capped_gated": the experts are those of ``capped_gated`` (tensors ``up`` and ``shared_up``
+then hold gate rows before up rows, expert by expert), with ``limit`` and for the shared expert ``shared_limit``; ``score``
+"softmax": the scores are the softmax over all experts' logits; ``group_score`` "largest": a group ranks by its largest score;
+``shared_gate`` false: the shared expert's output is added as it is.  ``input`` "shared": the shared expert's first product and
+the router's are columns of wider products that the block makes for all its branches (``forward_rows``); rows that another
+branch of the block made can be added where the experts' weighted sum is written (``addend``)."""
 from __future__ import annotations
 
 import numpy as np
@@ -106,13 +113,15 @@ class DenseFeedForward:
 
 class RoutedExperts:
     """The experts of a routed feed-forward and how a step's rows go through them, whatever chose them.  ``form``:
-    "gated_silu" (an expert's first matrix holds its gate rows, then its up rows) or "gelu" (up rows alone)."""
+    "gated_silu" (an expert's first matrix holds its gate rows, then its up rows), "gelu" (up rows alone), or "capped_gated"
+    (gate rows and up rows, capped as ``cap`` = (limit, slope, shift) says)."""
     DIRECT_ROWS = 128            # as many rows as a recorded step holds at most
 
-    def _set_experts(self, first, down, experts: int, inter: int, hidden: int, form: str):
+    def _set_experts(self, first, down, experts: int, inter: int, hidden: int, form: str, cap=ops.NO_CAP):
+        self.cap = cap
         self.first, self.down_all, self.form = first, down, form
         self.experts, self.inter, self.hidden = experts, inter, hidden
-        per = (2 if form == "gated_silu" else 1) * inter
+        per = ops.expert_rows(form) * inter
         if first.shape != (experts * per, hidden) or down.shape != (experts * hidden, inter):
             raise ValueError(f"routed feed-forward: weights {tuple(first.shape)}, {tuple(down.shape)} do not fit {experts} experts of inner "
                              f"size {inter} over hidden {hidden}")
@@ -121,15 +130,18 @@ class RoutedExperts:
         self.expert_down = [Linear(down[e * hidden:(e + 1) * hidden]) for e in range(experts)]
 
     def _mid(self, e: int, xs):
-        return self.expert_first[e].gated(xs) if self.form == "gated_silu" else ops.activation(self.expert_first[e](xs), "gelu_erf")
+        if self.form == "gated_silu":
+            return self.expert_first[e].gated(xs)
+        z = self.expert_first[e](xs)
+        return ops.capped_gate(z, *self.cap) if self.form == "capped_gated" else ops.activation(z, "gelu_erf")
 
-    def run_experts(self, h, chosen, weight):
-        """float32 [n, hidden]: sum_c weight[t, c] * expert chosen[t, c] of h[t]."""
+    def run_experts(self, h, chosen, weight, add=()):
+        """float32 [n, hidden]: sum_c weight[t, c] * expert chosen[t, c] of h[t], plus the rows ``add`` (up to two)."""
         top = chosen.shape[1]
         if h.shape[0] <= self.DIRECT_ROWS:
-            return ops.moe_experts(h, self.first, self.down_all, chosen, weight, self.inter, self.form)
+            return ops.moe_experts(h, self.first, self.down_all, chosen, weight, self.inter, self.form, self.cap, add)
         if ops.moe_grouped_serves(h, self.first, self.inter):
-            return ops.moe_grouped(h, self.first, self.down_all, chosen, weight, self.inter, self.form)
+            return ops.moe_grouped(h, self.first, self.down_all, chosen, weight, self.inter, self.form, self.cap, add)
         # group the (token, choice) pairs by expert; within an expert in the order of the tokens
         flat = chosen.to("cpu").numpy().reshape(-1)
         order = np.argsort(flat, kind="stable").astype(np.int32)
@@ -139,6 +151,11 @@ class RoutedExperts:
         xs = ops.gather_rows(h, src)
         ws = ops.gather_rows(pair_weight.reshape(-1, 1), torch.from_numpy(order).to(h.device)).reshape(-1)
         out = torch.zeros((h.shape[0], self.hidden), dtype=torch.float32, device=h.device)
+        if add:
+            every = torch.arange(h.shape[0], dtype=torch.int32, device=h.device)
+            ones = torch.ones((h.shape[0],), dtype=torch.float32, device=h.device)
+            for y in add:
+                ops.scatter_add(out, y, every, ones)
         at = 0
         for e in range(self.experts):
             n = int(counts[e])
@@ -176,33 +193,63 @@ class RoutedGatedSiluFeedForward(RoutedExperts):
 @register_part("feed_forward", "routed_scored")
 class RoutedScoredFeedForward(RoutedExperts):
     capturable = True
+    FORMS = ("gelu", "capped_gated")
 
     def __init__(self, spec, builder):
         p = spec.params
         W, E = int(p["hidden_size"]), int(p["num_experts"])
         self.top, self.scale = int(p["top"]), float(p.get("scale", 1.0))
         self.groups, self.keep = int(p.get("groups") or 1), int(p.get("keep") or 1)
+        self.score, self.group_score = str(p.get("score", "sigmoid")), str(p.get("group_score", "two_largest"))
+        form = str(p.get("form", "gelu"))
+        if form not in self.FORMS:
+            raise ValueError(f"routed feed-forward: form {form!r} is not one of {self.FORMS}")
         if not 1 <= self.top <= E or E % self.groups or not 1 <= self.keep <= self.groups or self.keep * (E // self.groups) < self.top:
             raise ValueError(f"routed feed-forward: {self.top} of {E} experts a token, from {self.keep} of {self.groups} groups")
+        cap = lambda limit: (float(p[limit]), float(p.get("slope", 1.0)), float(p.get("shift", 0.0))) if form == "capped_gated" else ops.NO_CAP
         self.shared = int(p["shared_size"]) if p.get("shared_size") else None
-        self.router = Linear(builder.tensor(spec, "router"))          # the experts' rows, then the shared expert's gate row
-        if self.router.weight.shape != (E + (1 if self.shared else 0), W):
+        self.shared_gate = bool(self.shared) and bool(p.get("shared_gate", True))
+        self.shared_input = p.get("input") == "shared"
+        self._set_experts(builder.tensor(spec, "up"), builder.tensor(spec, "down"), E, int(p["intermediate_size"]), W, form, cap("limit"))
+        per = ops.expert_rows(form)
+        # what the block's wider products make for this part: the shared expert's first rows; the router's logits
+        self.in_rows, self.exact_rows = per * (self.shared or 0), E + (1 if self.shared_gate else 0)
+        self.router = None if self.shared_input else Linear(builder.tensor(spec, "router"))   # the experts' rows (, the shared expert's gate row)
+        if self.router is not None and self.router.weight.shape != (self.exact_rows, W):
             raise ValueError(f"routed feed-forward: router {tuple(self.router.weight.shape)} does not fit {E} experts"
-                             + (" and a shared expert's gate" if self.shared else ""))
+                             + (" and a shared expert's gate" if self.shared_gate else ""))
         self.correction = builder.tensor(spec, "correction") if "correction" in spec.tensors else None
-        self._set_experts(builder.tensor(spec, "up"), builder.tensor(spec, "down"), E, int(p["intermediate_size"]), W, "gelu")
         if self.shared:
-            self.shared_up, self.shared_down = Linear(builder.tensor(spec, "shared_up")), Linear(builder.tensor(spec, "shared_down"))
-            if self.shared_up.weight.shape != (self.shared, W) or self.shared_down.weight.shape != (W, self.shared):
-                raise ValueError(f"routed feed-forward: the shared expert's weights {tuple(self.shared_up.weight.shape)}, "
-                                 f"{tuple(self.shared_down.weight.shape)} do not fit inner size {self.shared} over hidden {W}")
+            self.shared_cap = cap("shared_limit")
+            self.shared_up = None if self.shared_input else Linear(builder.tensor(spec, "shared_up"))
+            self.shared_down = Linear(builder.tensor(spec, "shared_down"))
+            if (self.shared_up is not None and self.shared_up.weight.shape != (self.in_rows, W)) or self.shared_down.weight.shape != (W, self.shared):
+                raise ValueError(f"routed feed-forward: the shared expert's weights do not fit inner size {self.shared} over hidden {W}: down "
+                                 f"{tuple(self.shared_down.weight.shape)}")
 
-    def forward(self, h, ctx):
+    def forward(self, h, ctx, addend=None):
         h = as_tensor(h)
-        logits = self.router(h, out_dtype=torch.float32)
-        chosen, weight = ops.moe_route_scored(logits, self.experts, self.top, self.correction, self.groups, self.keep, self.scale)
-        out = self.run_experts(h, chosen, weight)
+        if self.shared_input:
+            raise RuntimeError("a routed feed-forward whose input products are shared gets its rows from the part that makes them")
+        return self._run(h, self.router(h, out_dtype=torch.float32), self.shared_up(h) if self.shared else None, addend)
+
+    def forward_rows(self, h, rows, col0, ctx, exact, exact_col0, addend=None):
+        """``rows`` [n, >= col0 + in_rows]: the shared expert's first product from column ``col0``; ``exact`` float32: the router's
+        logits from ``exact_col0`` on."""
+        return self._run(h, exact[:, exact_col0:], rows[:, col0:col0 + self.in_rows] if self.shared else None, addend)
+
+    takes_addend = True
+
+    def _run(self, h, logits, first, addend):
+        chosen, weight = ops.moe_route_scored(logits, self.experts, self.top, self.correction, self.groups, self.keep, self.scale,
+                                              self.score, self.group_score)
+        add = [] if addend is None else [addend]
         if self.shared:
-            y = self.shared_down(ops.activation(self.shared_up(h), "gelu_erf"))
+            mid = ops.capped_gate(first, *self.shared_cap) if self.form == "capped_gated" else ops.activation(first.contiguous(), "gelu_erf")
+            y = self.shared_down(mid)
+            if not self.shared_gate:
+                add.append(y)
+        out = self.run_experts(h, chosen, weight, add)
+        if self.shared_gate:
             ops.add_gated_rows(out, y, logits, self.experts)
         return out

@@ -1,7 +1,8 @@
 """RMSNorm: y = x * (1 / sqrt(mean(x^2) + eps)) * w, statistics in 32-bit (kernels/norm.cpp:13-31).
 The residual add that precedes a norm in a block is fused into the same pass
 (engine/cuda_ops.cu:140-170 has the same fusion).  With ``offset`` c the checkpoint stores w - c (a weight kept around
-zero for c = 1): the sum is made once, in 32-bit, when the part is built.
+zero for c = 1): the sum is made once, in 32-bit, when the part is built; so is a ``gain`` on the norm's result (a fixed
+scale of what reads it: a product of scaled rows is the scaled product).
 
 ``dyt`` (Dynamic Tanh): y = tanh(alpha x) w + b with one learned slope alpha, a weight and a bias over the width: no mean and
 no variance, nothing crosses the columns.
@@ -30,6 +31,9 @@ class RMSNorm:
         offset = float(spec.params.get("offset", 0.0))
         if offset:
             self.weight = self.weight + offset
+        gain = float(spec.params.get("gain", 1.0))
+        if gain != 1.0:
+            self.weight = self.weight * gain
         self.dtype = builder.dtype
         if self.weight.shape != (self.width,):
             raise ValueError(f"RMSNorm of width {self.width} got a weight of shape {tuple(self.weight.shape)}")

@@ -4,7 +4,7 @@ of their own.
 One joined product makes q | k | v (| gate).  ``qkv_bias`` (float32 over q | k | v) is added where the sums are still
 32-bit.  q and k are normed as ``qk_norm`` says ("projection": one RMS norm over the whole q row, all heads at once, and
 one over the whole k row, with plain weights of those sizes; "head": per head with one weight vector of the key size for
-all heads; None), then the first ``rotary_dim`` dimensions of every head are rotated.  Query head h reads key/value head
+all heads; "head_unit": per head without a weight; None), then the first ``rotary_dim`` dimensions of every head are rotated.  Query head h reads key/value head
 h // (heads / kv_heads); a query at position p sees the keys max(0, p - window + 1) .. p.  With ``sink`` the softmax has
 one more term in its denominator, exp(sink_score), that belongs to no value:
 
@@ -21,15 +21,22 @@ may be "interleaved" (dimension 2i with 2i + 1).  ``kv`` "borrowed": the part ha
 biases, convolutions or norms of them); its run-order entry reads the keys and values that another entry wrote
 (``cache_of``), with its own queries, window, sink and gate, and keeps only its own convolution's state.  ``storage_window``:
 the window by which the keys and values are kept if other entries read them with a longer one (None: every position).
+``mask`` "chunked": the sequence is cut into chunks of ``window`` positions, counted from its first one, and a query sees the
+keys up to its own position of its own chunk only; what lies below a sequence's current chunk is given back.  ``distance_bias``
+"halving": head h's score loses slope_h * (query's position - key's position), slope_h = 2^(-8 (h + 1) / heads).
 """
 from __future__ import annotations
+
+import torch
 
 from ..cache import KVNeed, StateNeed
 from ..kernels import ops
 from .base import register_part
 from .linear import Linear
 
-QK_NORMS = (None, "projection", "head")
+QK_NORMS = (None, "projection", "head", "head_unit")
+MASKS = ("sliding", "chunked")
+DISTANCE_BIASES = (None, "halving")
 GATES = (None, "sigmoid", "head_sigmoid")
 
 
@@ -44,6 +51,14 @@ class SinkAttention:
         self.dk, self.dv = int(p["key_dim"]), int(p["value_dim"])
         self.scale, self.eps = float(p["scale"]), float(p.get("eps", 1e-6))
         self.window = int(p["window"]) if p.get("window") else None
+        self.chunked = p.get("mask", "sliding") == "chunked"
+        if p.get("mask", "sliding") not in MASKS or (self.chunked and not self.window):
+            raise ValueError(f"sink attention: mask {p.get('mask')!r} is one of {MASKS}, and chunks have a size (window)")
+        if p.get("distance_bias") not in DISTANCE_BIASES:
+            raise ValueError(f"sink attention: distance_bias {p.get('distance_bias')!r} is not one of {DISTANCE_BIASES}")
+        self.slopes = None
+        if p.get("distance_bias"):
+            self.slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / self.nh) for h in range(self.nh)], dtype=torch.float32).to(builder.device)
         self.sink = float(p.get("sink_score", 0.0)) if p.get("sink") else None
         if p.get("sink") == "learned":
             self.sink = builder.tensor(spec, "sink_scores")
@@ -77,8 +92,9 @@ class SinkAttention:
                              f"heads of key size {self.dk} and value size {self.dv} over hidden {self.hidden}")
         if self.out.weight.shape != (self.hidden, self.nh * self.dv):
             raise ValueError(f"sink attention: output weight {tuple(self.out.weight.shape)} does not fit")
-        self.q_w = builder.tensor(spec, "q_norm") if self.qk_norm else None
-        self.k_w = builder.tensor(spec, "k_norm") if self.qk_norm and not self.borrows else self.q_w
+        weighted = self.qk_norm in ("projection", "head")
+        self.q_w = builder.tensor(spec, "q_norm") if weighted else None
+        self.k_w = builder.tensor(spec, "k_norm") if weighted and not self.borrows else self.q_w
         self.position = builder.build(spec.parts["position"]) if "position" in spec.parts else None
         if self.position is not None and self.position.rotary_dim > self.dk:
             raise ValueError("sink attention: the rotation lies within the key size")
@@ -105,7 +121,10 @@ class SinkAttention:
         window = int(p["window"]) if p.get("window") else None
         if "storage_window" in p:                       # others read these keys, by windows of their own
             window = int(p["storage_window"]) if p["storage_window"] else None
-        return [KVNeed(int(p["num_kv_heads"]), int(p["key_dim"]), window, value_dim=int(p["value_dim"]))] + SinkAttention._conv_need(spec)
+        chunked = p.get("mask") == "chunked"
+        if chunked and window != int(p["window"]):
+            raise ValueError("sink attention: keys kept by another window than the part's own are read through a sliding one")
+        return [KVNeed(int(p["num_kv_heads"]), int(p["key_dim"]), window, value_dim=int(p["value_dim"]), chunked=chunked)] + SinkAttention._conv_need(spec)
 
     @staticmethod
     def cache_needs_beside_shared(spec):
@@ -137,5 +156,6 @@ class SinkAttention:
                                cos, sin, rot, lc.k, lc.v, table, ctx, write_cache=not self.borrows, col0=col0, pairing=pairing,
                                conv=self.conv, conv_state=state)
         o = ops.sink_attention(q, lc.k, lc.v, table, ctx, self.nh, self.nkv, self.dk, self.dv, self.scale, self.window, self.sink,
-                               rows if self.gate else None, col0 + self.gate_off, gate_per_head=self.head_gate)
+                               rows if self.gate else None, col0 + self.gate_off, gate_per_head=self.head_gate, chunked=self.chunked,
+                               slopes=self.slopes)
         return self.out(o)
