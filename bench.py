@@ -352,6 +352,22 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
             if f and f["kind"] == "moe" and "palm_moe_experts" not in out:                 # plain experts: two matrices each
                 out["palm_moe_experts"] = (None, None, 2.0 * batch * f["router"]["top"] * 2 * f["expert"]["ff"] * raw["width"], hbm)
                 out["palm_moe_grouped"] = (2.0 * tokens * f["router"]["top"] * 2 * f["expert"]["ff"] * raw["width"], mfma, None, None)
+    elif raw.get("architecture") == "Vovalix":
+        for layer in raw["layers"]:
+            m, f = layer["mixer"], layer.get("mlp")
+            per = m["heads"] * m["dim"] * m["vdim"]
+            if layer["type"] == "attention" and "palm_sink_attention" not in out:
+                size = m["mask"]["size"] if m.get("mask") else max(tokens, context + 1)
+                seen = sum(p % size + 1 for p in range(tokens))
+                out["palm_sink_attention_mfma"] = (2.0 * m["heads"] * (m["dim"] + m["vdim"]) * seen, mfma, None, None)
+                out["palm_sink_attention"] = (None, None, 2.0 * batch * (context % size + 1) * m["kv_heads"] * (m["dim"] + m["vdim"]), hbm)
+            elif layer["type"] == "gla":                                # two multiply-adds for every element of S and token
+                out["palm_gla"] = (4.0 * tokens * per, vec, 2.0 * 4 * batch * per, hbm)
+            elif layer["type"] == "delta":                              # four
+                out["palm_delta_head"] = (8.0 * tokens * per, vec, 2.0 * 4 * batch * per, hbm)
+            if f and "palm_moe_experts" not in out:
+                amount = 2.0 * f["router"]["top"] * 3 * f["expert"]["ff"] * raw["width"]
+                out["palm_moe_experts"], out["palm_moe_grouped"] = (None, None, batch * amount, hbm), (tokens * amount, mfma, None, None)
     elif "layers" in raw:
         for layer in raw["layers"]:
             m = layer["mixer"]
@@ -486,7 +502,18 @@ def _biguzen_bench(args, record) -> dict:
     return record["sizes"]["biguzen-2048"]["biguzen"]
 
 
-DESIGNS = {"biguzen": ("Biguzen presets beside Matalix presets of equal width and depth", _biguzen_bench),
+def _vovalix_bench(args, record) -> dict:
+    """The Vovalix presets beside the Biguzen and the Pazilorn presets of the same width and depth (the closest designs here:
+    Biguzen has the same attention kernels, experts chosen in groups with a shared one and a recurrence over a matrix per head,
+    Pazilorn the other delta rule and gated experts)."""
+    for width in ("2048", "4096"):
+        record["sizes"][f"vovalix-{width}"] = {
+            name: design_points(preset_dict(f"{name}-{width}"), args, PREFILL_TOKENS, BATCH, CONTEXT) for name in ("vovalix", "biguzen", "pazilorn")}
+    return record["sizes"]["vovalix-2048"]["vovalix"]
+
+
+DESIGNS = {"vovalix": ("Vovalix presets beside Biguzen and Pazilorn presets of equal width and depth", _vovalix_bench),
+           "biguzen": ("Biguzen presets beside Matalix presets of equal width and depth", _biguzen_bench),
            "matalix": ("Matalix presets beside Sebesun presets of equal width and depth", _matalix_bench),
            "sebesun": ("Sebesun presets beside Qwen3 models of equal width and depth", _sebesun_bench),
            "pazilorn": ("Pazilorn presets beside Sebesun presets of equal width and depth", _pazilorn_bench)}
@@ -524,7 +551,8 @@ def main(argv=None) -> int:
     ap.add_argument("--prefill-tokens", type=int, default=PREFILL_TOKENS,
                     help="tokens of the timed prompt (2,048 is the workload's; others serve profiles of longer prompts)")
     ap.add_argument("--design", help="instead of the default workload: another design's presets beside its closest relative "
-                    "of equal width and depth ('sebesun' beside Qwen3, 'pazilorn' and 'matalix' beside Sebesun, 'biguzen' beside Matalix)")
+                    "of equal width and depth ('sebesun' beside Qwen3, 'pazilorn' and 'matalix' beside Sebesun, 'biguzen' beside Matalix, "
+                    "'vovalix' beside Biguzen and Pazilorn)")
     args = ap.parse_args(argv)
     if args.design:
         if args.gpus != 1:

@@ -107,7 +107,7 @@ def build_dir() -> Path:
     local = CSRC / "_build"
     try:
         local.mkdir(parents=True, exist_ok=True)
-        probe = local / f".probe{os.getpid()}"
+        probe = local / f".probe{os.getpid()}_{threading.get_ident()}"          # (libraries may be built side by side)
         probe.write_text("")
         probe.unlink()
         return local
@@ -244,6 +244,12 @@ def build(name: str, force: bool = False) -> Path:
     sources, defines = _spec(name)
     with _lock:
         return _compile(name, sources, defines, force)
+
+
+def build_all(names, force: bool = False) -> list[Path]:
+    """Several libraries side by side."""
+    with _lock, ThreadPoolExecutor(max_workers=8) as pool:
+        return list(pool.map(lambda name: _compile(name, *_spec(name), force), names))
 
 
 def load(name: str) -> ctypes.CDLL:

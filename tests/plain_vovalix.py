@@ -184,6 +184,19 @@ def route(z, r):
     return chosen, picked / (picked.sum(dim=1, keepdim=True) + 1e-20)
 
 
+def route_margins(z, r):
+    """How far each token's choice is from another one [T]: the smallest difference of router logits between an expert that is
+    chosen and one that could be, and between the largest of a kept group and of one that is not."""
+    E, top = int(r["experts"]), int(r["top"])
+    count, keep = (int(r["groups"]["count"]), int(r["groups"]["keep"])) if r.get("groups") else (1, 1)
+    by_group = z.reshape(z.shape[0], count, E // count)
+    best = by_group.max(dim=2).values
+    ranked = best.sort(dim=1, descending=True).values
+    out = ranked[:, keep - 1] - ranked[:, keep] if keep < count else torch.full((z.shape[0],), math.inf, dtype=F64)
+    inside = by_group.masked_fill((best < ranked[:, keep - 1:keep])[:, :, None], -math.inf).reshape(z.shape[0], E).sort(dim=1, descending=True).values
+    return torch.minimum(out, inside[:, top - 1] - inside[:, top]) if top < E else out
+
+
 def routed_feed_forward(h, w, p, f):
     chosen, weights = route(h @ w[p + "router"].T, f["router"])
     out = torch.zeros_like(h)
@@ -202,9 +215,9 @@ def routed_feed_forward(h, w, p, f):
 MIXERS = {"gla": gla_mixer, "attention": attention_mixer, "delta": delta_mixer}
 
 
-def forward(raw, tensors, ids, layer_results=None):
+def forward(raw, tensors, ids, layer_results=None, margins=None):
     """Logits [T, vocab] of one sequence from its first token.  ``layer_results``: a list that gets the residual stream
-    after every layer."""
+    after every layer; ``margins``: one that gets every router's ``route_margins``."""
     w = {k: t.to(F64) for k, t in tensors.items()}
     eps = float(raw["norm"]["eps"])
     x = w["embed"][torch.tensor(ids, dtype=torch.long)]
@@ -217,6 +230,8 @@ def forward(raw, tensors, ids, layer_results=None):
         y = MIXERS[layer["type"]](h, w, p + "mix.", layer["mixer"], eps)
         if layer.get("mlp") is not None:
             y = y + routed_feed_forward(h, w, p + "mlp.", layer["mlp"])
+            if margins is not None:
+                margins.append(route_margins(h @ w[p + "mlp.router"].T, layer["mlp"]["router"]))
         x = x + y
         if layer_results is not None:
             layer_results.append(x)
