@@ -8,7 +8,8 @@
 // A first pass makes the step's decays and writes q (times its scale), k and the decays as 32-bit rows padded to the key size
 // that the walk is compiled for (PALM_GLA_DIM: one library for each); the padding's q and k are zero and its decay one.  The
 // decay is the exponential of the logarithm of the sigmoid over tau, so that neither a decay near one nor one near zero loses
-// its digits.  The walk over the tokens, and how a long run of them is cut into chunks that run side by side, is
+// its digits.  Where every sequence brings one token the walk's waves make q, k and decays of their head themselves, while the
+// state is on its way to the registers, and the first pass is not needed.  The walk over the tokens, and how a long run of them is cut into chunks that run side by side, is
 // linear_recurrence.h's.
 #include "linear_recurrence.h"
 
@@ -39,6 +40,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const T* __restrict__ row
     float z[GLA_TOKENS];
 #pragma unroll
     for (int i = 0; i < GLA_TOKENS; ++i) z[i] = bias[channel];
+#pragma unroll 4
     for (int r = 0; r < rank; ++r) {
         const float w = w2[(size_t)r * heads * dim + channel];
 #pragma unroll
@@ -56,11 +58,50 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(const T* __restrict__ row
     }
 }
 
+// A step of single tokens: a lane makes its key channels' q, k and decay.
+template <typename T>
+struct GlaDirect {
+    static constexpr bool SINGLE = true;
+    static constexpr int QREGS = (GLA_DIM + WAVE - 1) / WAVE;
+    const T* rows;
+    const float* low;
+    const float* w2;
+    const float* bias;
+    int row_stride, q_off, k_off, low_stride, rank, heads, dim;
+    float q_scale, inv_tau;
+    __device__ void read(size_t row, int h, int lane, float (&in)[3][QREGS]) const {
+        const T* __restrict__ src = rows + row * row_stride;
+        const float* __restrict__ lo = low + row * low_stride;
+        const float* __restrict__ w = w2;
+        int channel[QREGS];
+        float z[QREGS];
+#pragma unroll
+        for (int c = 0; c < QREGS; ++c) {
+            channel[c] = h * dim + min(c * WAVE + lane, dim - 1);
+            z[c] = bias[channel[c]];
+        }
+#pragma unroll 8
+        for (int r = 0; r < rank; ++r) {
+            const float l = lo[r];
+#pragma unroll
+            for (int c = 0; c < QREGS; ++c) z[c] = fmaf(l, w[(size_t)r * heads * dim + channel[c]], z[c]);
+        }
+#pragma unroll
+        for (int c = 0; c < QREGS; ++c) {
+            const bool there = c * WAVE + lane < dim;
+            const float q = to_float(src[q_off + channel[c]]) * q_scale, k = to_float(src[k_off + channel[c]]);
+            in[0][c] = there ? q : 0.f;
+            in[1][c] = there ? k : 0.f;
+            in[2][c] = there ? expf(gla_logsigmoid(z[c]) * inv_tau) : 1.f;
+        }
+    }
+};
+
 PALM_API int palm_gla_pad() { return GLA_DIM; }
 
 // rows [n, row_stride]: q at q_off, k at k_off (heads * dim each), v at v_off, the gate at g_off (heads * vdim each); low float32
 // [n, low_stride], `rank` values a token; state float32 [slots, heads, dim, vdim]; norm_w float32 [vdim]; out [n, heads * vdim].
-// Room: prep n * heads * 3 * palm_gla_pad() floats; with chunks (chunk > 0), max_chunks = ceil(max_new / chunk): starts n_seqs *
+// Room: prep n * heads * 3 * palm_gla_pad() floats (not needed if max_new is one); with chunks (chunk > 0), max_chunks = ceil(max_new / chunk): starts n_seqs *
 // max_chunks * heads * dim * vdim floats and chunk_keep n_seqs * max_chunks * heads * dim floats.
 PALM_API int palm_gla(hipStream_t stream, const void* rows, int dtype, int row_stride, int q_off, int k_off, int v_off, int g_off,
                       const float* low, int low_stride, const float* w2, const float* bias, int rank, float tau, float q_scale,
@@ -73,16 +114,25 @@ PALM_API int palm_gla(hipStream_t stream, const void* rows, int dtype, int row_s
     PALM_CHECK(vdim <= 1024, "gla: a value size of %d exceeds 1024", vdim);
     PALM_CHECK(tau > 0.f, "gla: tau %g must be positive", (double)tau);
     PALM_CHECK(chunk >= 0 && (chunk == 0 || (starts && chunk_keep && max_new > 0)), "gla: chunks of %d tokens need their starting states", chunk);
-    PALM_CHECK(n_tokens == 0 || (rows && low && w2 && bias && norm_w && state && prep && out), "gla: rows, decays' weights and state are needed");
+    PALM_CHECK(n_tokens == 0 || (rows && low && w2 && bias && norm_w && state && (prep || max_new == 1) && out), "gla: rows, decays' weights and state are needed");
     if (n_seqs == 0 || n_tokens == 0) return 0;
     const int max_chunks = chunk > 0 ? (max_new + chunk - 1) / chunk : 1;
     PALM_CHECK(heads <= 65535 && (long long)n_seqs * max_chunks <= 65535 && n_tokens <= 65535 * GLA_TOKENS,
                "gla: %d heads / %d sequences x %d chunks / %d tokens are more than one launch takes", heads, n_seqs, max_chunks, n_tokens);
+    if (max_new == 1) {
+        PALM_DTYPE_SWITCH(dtype, T, {
+            const GlaDirect<T> direct{(const T*)rows, low, w2, bias, row_stride, q_off, k_off, low_stride, rank, heads, dim, q_scale, 1.0f / tau};
+            linear_recurrence_sized<T, GLA_DIM, true>(stream, n_seqs, 1, 0, nullptr, nullptr, (const T*)rows, row_stride, v_off, g_off, direct, nullptr,
+                                                      norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, 0, 0, nullptr);
+        });
+        PALM_LAUNCHED();
+        return 0;
+    }
     PALM_DTYPE_SWITCH(dtype, T, {
         gla_prep_kernel<T><<<dim3((heads * GLA_DIM + 255) / 256, (n_tokens + GLA_TOKENS - 1) / GLA_TOKENS), 256, 0, stream>>>(
             (const T*)rows, row_stride, q_off, k_off, q_scale, low, low_stride, w2, bias, rank, 1.0f / tau, n_tokens, heads, dim, prep);
         linear_recurrence_sized<T, GLA_DIM, true>(stream, n_seqs, max_new, chunk, starts, chunk_keep, (const T*)rows, row_stride, v_off, g_off,
-                                                  prep, nullptr, norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, 0, 0,
+                                                  PreparedRows<GLA_DIM, 3>{prep, heads}, nullptr, norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, 0, 0,
                                                   nullptr);
     });
     PALM_LAUNCHED();

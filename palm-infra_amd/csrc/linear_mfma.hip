@@ -58,7 +58,8 @@ __global__ __launch_bounds__(NW * WAVE) void linear_thin_kernel(const bf16_t* __
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const bool ok = k0 + j * 32 + g * 8 < K;            // K is a multiple of 8: a chunk is whole or absent
-                const int at = ok ? k0 + j * 32 : 0;                // an absent chunk reads the row's start and is zeroed
+                const int at = ok ? k0 + j * 32 : -g * 8;           // an absent chunk reads the row's start and is zeroed (the lane's own
+                                                                    // place in a first chunk may lie beyond a K below 32)
 #pragma unroll
                 for (int rt = 0; rt < RT; ++rt) {
                     const bf16x8 v = load_bf16x8(wp[rt] + at);
@@ -184,7 +185,7 @@ __global__ __launch_bounds__(NW * WAVE) void linear_stream_kernel(const bf16_t* 
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const bool ok = EXACT || (k0 + j * 32 + g * 8 < K);
-            const int at = ok ? k0 + j * 32 : 0;             // an absent chunk reads the row's start and is masked
+            const int at = ok ? k0 + j * 32 : -g * 8;        // an absent chunk reads the row's start and is masked
             wv[u][j] = load_bf16x8(ask_row + at);
             if (!AREG) xv[u][j] = load_bf16x8(xp + at);
             mask |= (ok ? 1 : 0) << j;
@@ -207,7 +208,7 @@ __global__ __launch_bounds__(NW * WAVE) void linear_stream_kernel(const bf16_t* 
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const bool ok = EXACT || (k0 + j * 32 + g * 8 < K);
-                const bf16x8 v = load_bf16x8(xp + (ok ? k0 + j * 32 : 0));
+                const bf16x8 v = load_bf16x8(xp + (ok ? k0 + j * 32 : -g * 8));
                 xa[t][j] = ok ? v : zero_bf16x8();
             }
         }

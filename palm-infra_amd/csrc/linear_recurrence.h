@@ -27,14 +27,34 @@ enum RecurrenceMode : int { REC_WHOLE = 0, REC_LOCAL = 1, REC_FROM_STARTS = 2 };
 
 __device__ inline float rec_silu(float z) { return z / (1.0f + expf(-z)); }
 
+// Where a token's q, k (and decays) come from.  `read` brings the values of lane, lane + 64, .. of a token's row and head into
+// in[0 = q, 1 = k, 2 = decay], q and k zero beyond the key size.  PreparedRows: [row][head][0 = q, 1 = k, 2 = decay][DMAX], 32-bit,
+// made by a pass before the walk.  A type with SINGLE set serves runs of one token: nothing is read ahead.
+template <int DMAX, int PREP>
+struct PreparedRows {
+    static constexpr bool SINGLE = false;
+    static constexpr int QREGS = (DMAX + WAVE - 1) / WAVE;
+    const float* rows;
+    int heads;
+    __device__ void read(size_t row, int h, int lane, float (&in)[PREP][QREGS]) const {
+        const float* __restrict__ qr = rows + ((row * heads + h) * PREP) * DMAX;
+#pragma unroll
+        for (int c = 0; c < QREGS; ++c) {
+            const int at = min(c * WAVE + lane, DMAX - 1);             // (a key size of 32: the upper lanes repeat)
+#pragma unroll
+            for (int i = 0; i < PREP; ++i) in[i][c] = qr[i * DMAX + at];
+        }
+    }
+};
+
 // CHANNEL: every token has a decay for each key channel (the third of its prepared rows), else one fixed decay a head.
 // MAXT: the most threads of a block (the value size, rounded up to whole waves): what the compiler may assume when it
 // hands out registers.  A thread keeps DMAX values of S; up to 256 threads a block they all stay in registers.
-// qk: [row][head][0 = q, 1 = k, CHANNEL: 2 = decay][DMAX], 32-bit, q and k zero beyond dim.  rows: v at v_off, the gate at g_off.
-template <typename T, int DMAX, int MAXT, bool CHANNEL>
+// inputs: q, k and decays.  rows: v at v_off, the gate at g_off.
+template <typename T, int DMAX, int MAXT, bool CHANNEL, typename In>
 __global__ __launch_bounds__(MAXT) void linear_recurrence_kernel(int mode, int chunk, int max_chunks, float* __restrict__ starts,
                                  float* __restrict__ chunk_keep, const T* __restrict__ rows,
-                                 int row_stride, int v_off, int g_off, const float* __restrict__ qk,
+                                 int row_stride, int v_off, int g_off, const In inputs,
                                  const float* __restrict__ decay, const float* __restrict__ norm_w, float eps,
                                  float* __restrict__ state, const int* __restrict__ seq_slot,
                                  const int* __restrict__ seq_new, const int* __restrict__ cu_new,
@@ -86,13 +106,7 @@ __global__ __launch_bounds__(MAXT) void linear_recurrence_kernel(int mode, int c
         const size_t row = (size_t)(row0 + t);
         vv = to_float(rows[row * row_stride + v_off + h * vdim + vc]);
         if (act) vv = rec_silu(vv);
-        const float* __restrict__ qr = qk + ((row * heads + h) * PREP) * DMAX;
-#pragma unroll
-        for (int c = 0; c < QREGS; ++c) {
-            const int at = min(c * WAVE + lane, DMAX - 1);             // (a key size of 32: the upper lanes repeat)
-#pragma unroll
-            for (int i = 0; i < PREP; ++i) in[i][c] = qr[i * DMAX + at];
-        }
+        inputs.read(row, h, lane, in);
     };
     auto from_lane = [](float x, int d) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, x), d % WAVE)); };
     float vv, in[PREP][QREGS], kept[QREGS];
@@ -102,8 +116,8 @@ __global__ __launch_bounds__(MAXT) void linear_recurrence_kernel(int mode, int c
     for (int t0 = 0; t0 < n_new; t0 += REC_TILE) {
         const int tt = min(REC_TILE, n_new - t0);
         for (int ti = 0; ti < tt; ++ti) {                        // not unrolled: the body is DMAX steps long already
-            float vn, next[PREP][QREGS];
-            read_token(min(t0 + ti + 1, n_new - 1), vn, next);
+            float vn = vv, next[PREP][QREGS];
+            if constexpr (!In::SINGLE) read_token(min(t0 + ti + 1, n_new - 1), vn, next);
             if (!mine) vv = 0.f;
             float acc = 0.f;
 #pragma unroll
@@ -124,11 +138,13 @@ __global__ __launch_bounds__(MAXT) void linear_recurrence_kernel(int mode, int c
                 const float ss = wave_sum(acc * acc);
                 if (lane == 0) red[ti][wave] = ss;
             }
-            vv = vn;
+            if constexpr (!In::SINGLE) {
+                vv = vn;
 #pragma unroll
-            for (int i = 0; i < PREP; ++i)
+                for (int i = 0; i < PREP; ++i)
 #pragma unroll
-                for (int c = 0; c < QREGS; ++c) in[i][c] = next[i][c];
+                    for (int c = 0; c < QREGS; ++c) in[i][c] = next[i][c];
+            }
         }
         if (mode == REC_LOCAL || joined) continue;
         __syncthreads();
@@ -187,9 +203,9 @@ __global__ void linear_recurrence_starts_kernel(float* __restrict__ starts, cons
 }
 
 // All launches of a step for one padded key size: chunk == 0 walks over every run in one block a head.
-template <typename T, int DMAX, bool CHANNEL>
+template <typename T, int DMAX, bool CHANNEL, typename In>
 static void linear_recurrence_sized(hipStream_t stream, int n_seqs, int max_new, int chunk, float* starts, float* chunk_keep, const T* rows,
-                                    int row_stride, int v_off, int g_off, const float* qk, const float* decay, const float* norm_w, float eps,
+                                    int row_stride, int v_off, int g_off, const In& inputs, const float* decay, const float* norm_w, float eps,
                                     float* state, const int* seq_slot, const int* seq_new, const int* cu_new, int heads, int dim, int vdim,
                                     T* out, int act, int joined, float* raw) {
     const int threads = (vdim + WAVE - 1) / WAVE * WAVE;
@@ -198,11 +214,11 @@ static void linear_recurrence_sized(hipStream_t stream, int n_seqs, int max_new,
     auto walk = [&](int mode) {
         const int run = chunk > 0 ? chunk : 1 << 30;
         if (threads <= 256)
-            linear_recurrence_kernel<T, DMAX, 256, CHANNEL><<<grid, threads, 0, stream>>>(mode, run, max_chunks, starts, chunk_keep, rows, row_stride,
-                v_off, g_off, qk, decay, norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, out, act, joined, raw);
+            linear_recurrence_kernel<T, DMAX, 256, CHANNEL, In><<<grid, threads, 0, stream>>>(mode, run, max_chunks, starts, chunk_keep, rows, row_stride,
+                v_off, g_off, inputs, decay, norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, out, act, joined, raw);
         else
-            linear_recurrence_kernel<T, DMAX, 1024, CHANNEL><<<grid, threads, 0, stream>>>(mode, run, max_chunks, starts, chunk_keep, rows, row_stride,
-                v_off, g_off, qk, decay, norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, out, act, joined, raw);
+            linear_recurrence_kernel<T, DMAX, 1024, CHANNEL, In><<<grid, threads, 0, stream>>>(mode, run, max_chunks, starts, chunk_keep, rows, row_stride,
+                v_off, g_off, inputs, decay, norm_w, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, out, act, joined, raw);
     };
     if (chunk == 0) {
         walk(REC_WHOLE);

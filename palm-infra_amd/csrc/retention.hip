@@ -71,7 +71,8 @@ PALM_API int palm_retention(hipStream_t stream, const void* qkvg, int dtype, int
                heads, n_seqs, max_chunks);
     const int pad = palm_retention_pad(dim);
     const long long rot_threads = (long long)n_tokens * heads * pad;
-#define RET_CASE(D) linear_recurrence_sized<T, D, false>(stream, n_seqs, max_new, chunk, starts, nullptr, (const T*)qkvg, row_stride, v_off, g_off, qk, \
+#define RET_CASE(D) linear_recurrence_sized<T, D, false>(stream, n_seqs, max_new, chunk, starts, nullptr, (const T*)qkvg, row_stride, v_off, g_off, \
+            PreparedRows<D, 2>{qk, heads}, \
             decay, nullptr, eps, state, seq_slot, seq_new, cu_new, heads, dim, vdim, (T*)out, act, joined, raw)
     PALM_DTYPE_SWITCH(dtype, T, {
         retention_rotate_kernel<T><<<(unsigned)((rot_threads + 255) / 256), 256, 0, stream>>>((const T*)qkvg, row_stride, q_off, k_off, cos_t,

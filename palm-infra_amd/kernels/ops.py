@@ -1033,7 +1033,7 @@ def gla(rows: torch.Tensor, low: torch.Tensor, w2: torch.Tensor, bias: torch.Ten
           f"{what}: state {tuple(state.shape)} {state.dtype} is not float32 [slots, {heads}, {dim}, {vdim}]")
     lib = gla_lib(dim)
     out = torch.empty((n, heads * vdim), dtype=rows.dtype, device=rows.device)
-    prep = torch.empty((n, heads, 3, lib.palm_gla_pad()), dtype=F32, device=rows.device)
+    prep = torch.empty((n, heads, 3, lib.palm_gla_pad()), dtype=F32, device=rows.device) if ctx.max_new > 1 else None
     chunk = retention_chunk(ctx.n_seqs, heads, ctx.max_new) if chunk is None else int(chunk)
     starts = keeps = None
     if chunk:

@@ -1,6 +1,7 @@
 """y = x W^T for a weight in the checkpoint's [out, in] layout: the one place that picks the kernel.
 
   float32 run, or a 32-bit weight under bfloat16 activations   the exact FMA kernel
+  bfloat16 x bfloat16, an inner size that is no multiple of 8    the exact FMA kernel (rows do not start on 16 bytes)
   bfloat16 x bfloat16, up to 16 rows (decode)                   the matrix-core kernel for thin products
   bfloat16 x bfloat16, 17 to 256 rows (decode batches, short    the kernel that brings both operands through rings in
   prompts)                                                      LDS, where it beats the others (ops.mid_pays); where
@@ -68,7 +69,7 @@ class Linear:
                 return ops.linear_thin(x.values, w, out_dtype or x.dtype, planes_ok=planes_ok, row_ss=x.ss, row_eps=x.eps)
             x = x.materialize()
         out_dtype = out_dtype or x.dtype
-        if x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16:
+        if x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and self.in_features % 8 == 0:
             rows = x.shape[0]
             if x.is_contiguous() and ops.mid_pays(rows, self.out_features, self.in_features, planes_ok=planes_ok, out_dtype=out_dtype):
                 return ops.linear_mid(x, w, out_dtype, planes_ok=planes_ok)

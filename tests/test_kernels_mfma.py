@@ -23,7 +23,7 @@ def rand(*shape, seed=0, scale=1.0, dtype=BF16):
 
 
 @pytest.mark.parametrize("M", [1, 8, 16, 17, 33, 64, 70, 128, 150])
-@pytest.mark.parametrize("N,K", [(7, 8), (130, 64), (515, 80), (1000, 224), (96, 4096), (4096, 1536), (300, 12288),
+@pytest.mark.parametrize("N,K", [(7, 8), (64, 8), (96, 16), (33, 24), (130, 64), (515, 80), (1000, 224), (96, 4096), (4096, 1536), (300, 12288),
                                  (1000, 2048), (515, 2056), (130, 5000), (9000, 2048), (8200, 3080), (64, 8192), (48, 7000),
                                  (4200, 5120)])
 def test_linear_thin_against_the_plain_product(ops, M, N, K):
