@@ -4,7 +4,7 @@
 //              weights the softmax over those logits alone
 //   few rows (a decode step): nothing is planned on the host, every (token, choice) reads its expert's weights itself
 //     expert_gate_up   mid[t, c, f] = silu(G_e h_t)[f] * (U_e h_t)[f],  e = chosen[t, c]           (32-bit)
-//     expert_down      out[t, :] = sum_c weight[t, c] * D_e mid[t, c, :]  in the order of c        (32-bit)
+//     expert_down      out[t, :] = sum_c weight[t, c] * D_e mid[t, c, :]                          (32-bit)
 //   An expert's form: gated (silu(G h) * (U h), the gate rows before the up rows), plain with the exact gelu (gelu(U h)), or
 //   capped gated (g sigmoid(slope g) (u + shift) with g = min(G h, limit), u = clamp(U h, -limit, limit)).
 //   Rows that other branches made (up to two) can be added to the weighted sum where it is written.
@@ -36,14 +36,15 @@ __device__ inline void load8(const float* p, float (&v)[8]) {
     v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
 }
 
-// One wave per token.
+// One wave per token.  PER: experts a lane holds.
+template <int PER>
 __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict__ logits, int experts, int top,
                                                          int* __restrict__ chosen, float* __restrict__ weight) {
     const size_t t = blockIdx.x;
     const int lane = threadIdx.x;
-    float z[ROUTE_MAX_PER_LANE];
+    float z[PER];
 #pragma unroll
-    for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+    for (int i = 0; i < PER; ++i) {
         const int e = i * WAVE + lane;
         z[i] = e < experts ? logits[t * experts + e] : -INFINITY;
     }
@@ -52,7 +53,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
         float best = -INFINITY;
         int at = 0x7fffffff;
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+        for (int i = 0; i < PER; ++i) {
             const int e = i * WAVE + lane;
             if (e < experts && (z[i] > best || (z[i] == best && e < at))) { best = z[i]; at = e; }
         }
@@ -68,24 +69,25 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
         if (lane == c) mine = p;                             // lane c keeps choice c's weight
         if (lane == 0) chosen[t * top + c] = min(at, experts - 1);     // (logits that are no numbers choose nobody: an expert that exists is named all the same)
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
+        for (int i = 0; i < PER; ++i)
             if (i * WAVE + lane == at) z[i] = -INFINITY;
     }
     if (lane < top) weight[t * top + lane] = mine / sum;
 }
 
 // One wave per token.  logits: rows `stride` apart (other columns may follow the experts').
+template <int PER>
 __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __restrict__ logits, int stride, int experts, int top,
                                                                 const float* __restrict__ correction, int groups, int keep, float scale,
                                                                 int softmax, int group_largest, int* __restrict__ chosen, float* __restrict__ weight) {
-    __shared__ float choice_s[ROUTE_MAX_PER_LANE * WAVE];
-    __shared__ float group_s[ROUTE_MAX_PER_LANE * WAVE];
+    __shared__ float choice_s[PER * WAVE];
+    __shared__ float group_s[PER * WAVE];
     const size_t t = blockIdx.x;
     const int lane = threadIdx.x;
-    float s[ROUTE_MAX_PER_LANE], z[ROUTE_MAX_PER_LANE];
+    float s[PER], z[PER];
     float high = -INFINITY, total = 0.f;
 #pragma unroll
-    for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+    for (int i = 0; i < PER; ++i) {
         const int e = i * WAVE + lane;
         s[i] = e < experts ? logits[t * stride + e] : -INFINITY;
         high = fmaxf(high, s[i]);
@@ -93,11 +95,11 @@ __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __r
     if (softmax) {
         high = wave_max(high);
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) { s[i] = expf(s[i] - high); total += s[i]; }
+        for (int i = 0; i < PER; ++i) { s[i] = expf(s[i] - high); total += s[i]; }
         total = wave_sum(total);
     }
 #pragma unroll
-    for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+    for (int i = 0; i < PER; ++i) {
         const int e = i * WAVE + lane;
         s[i] = e >= experts ? 0.f : softmax ? s[i] / total : 1.0f / (1.0f + expf(-s[i]));
         z[i] = e < experts ? s[i] + (correction ? correction[e] : 0.f) : -INFINITY;
@@ -116,7 +118,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __r
         }
         __syncthreads();
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+        for (int i = 0; i < PER; ++i) {
             const int e = i * WAVE + lane;
             if (e >= experts) continue;
             const int g = e / size;
@@ -131,7 +133,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __r
         float best = -INFINITY, score = 0.f;
         int at = 0x7fffffff;
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+        for (int i = 0; i < PER; ++i) {
             const int e = i * WAVE + lane;
             if (e < experts && (z[i] > best || (z[i] == best && e < at))) { best = z[i]; at = e; score = s[i]; }
         }
@@ -145,7 +147,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __r
         if (lane == c) mine = score;
         if (lane == 0) chosen[t * top + c] = min(at, experts - 1);
 #pragma unroll
-        for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
+        for (int i = 0; i < PER; ++i)
             if (i * WAVE + lane == at) z[i] = -INFINITY;
     }
     if (lane < top) weight[t * top + lane] = mine / (sum + 1e-20f) * scale;
@@ -208,7 +210,9 @@ __global__ __launch_bounds__(MOE_THREADS) void expert_gate_up_kernel(const T* __
     }
 }
 
-// grid (blocks of output rows, tokens); a wave computes one output value at a time, the choices one after the other.
+// grid (blocks of output rows, tokens); a wave computes one output value at a time, DOWN_CHOICES choices at once.
+constexpr int DOWN_CHOICES = 4;
+
 // `add0`, `add1`: null, or rows [n, width] that other branches made, added to the sum.
 template <typename T, typename TW>
 __global__ __launch_bounds__(MOE_THREADS) void expert_down_kernel(const float* __restrict__ mid, const TW* __restrict__ down,
@@ -217,28 +221,50 @@ __global__ __launch_bounds__(MOE_THREADS) void expert_down_kernel(const float* _
                                                                   const T* __restrict__ add0, const T* __restrict__ add1,
                                                                   float* __restrict__ out) {
     extern __shared__ float m_s[];                  // [top][ff]
+    __shared__ int expert_s[WAVE];
+    __shared__ float weight_s[WAVE];
     const int t = blockIdx.y;
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, n_waves = MOE_THREADS / WAVE;
     for (int i = threadIdx.x; i < top * ff; i += MOE_THREADS) m_s[i] = mid[(size_t)t * top * ff + i];
+    if (threadIdx.x < top) {
+        expert_s[threadIdx.x] = chosen[(size_t)t * top + threadIdx.x];
+        weight_s[threadIdx.x] = weight[(size_t)t * top + threadIdx.x];
+    }
     __syncthreads();
     const int r_end = min(width, (int)(blockIdx.x + 1) * rows_per_block);
     for (int r = blockIdx.x * rows_per_block + wave; r < r_end; r += n_waves) {
-        float total = 0.f;
-        for (int c = 0; c < top; ++c) {
-            const TW* wr = down + ((size_t)chosen[(size_t)t * top + c] * width + r) * ff;
-            float acc = 0.f;
+        // the rows of four choices are under way together, and a row's lanes are added once for all choices
+        float part = 0.f;
+        for (int c0 = 0; c0 < top; c0 += DOWN_CHOICES) {
+            const TW* wr[DOWN_CHOICES];
+            float acc[DOWN_CHOICES];
+#pragma unroll
+            for (int i = 0; i < DOWN_CHOICES; ++i) {                        // (beyond the last choice: the last one again, not counted)
+                wr[i] = down + ((size_t)expert_s[min(c0 + i, top - 1)] * width + r) * ff;
+                acc[i] = 0.f;
+            }
             if (ff % 8 == 0) {
                 for (int f = lane * 8; f < ff; f += WAVE * 8) {
-                    float wv[8];
-                    load8(wr + f, wv);
+                    float wv[DOWN_CHOICES][8];
 #pragma unroll
-                    for (int i = 0; i < 8; ++i) acc = fmaf(wv[i], m_s[c * ff + f + i], acc);
+                    for (int i = 0; i < DOWN_CHOICES; ++i) load8(wr[i] + f, wv[i]);
+#pragma unroll
+                    for (int i = 0; i < DOWN_CHOICES; ++i) {
+                        const float* m = m_s + min(c0 + i, top - 1) * ff + f;
+#pragma unroll
+                        for (int j = 0; j < 8; ++j) acc[i] = fmaf(wv[i][j], m[j], acc[i]);
+                    }
                 }
             } else {
-                for (int f = lane; f < ff; f += WAVE) acc = fmaf(to_float(wr[f]), m_s[c * ff + f], acc);
+                for (int f = lane; f < ff; f += WAVE)
+#pragma unroll
+                    for (int i = 0; i < DOWN_CHOICES; ++i) acc[i] = fmaf(to_float(wr[i][f]), m_s[min(c0 + i, top - 1) * ff + f], acc[i]);
             }
-            total = fmaf(weight[(size_t)t * top + c], wave_sum(acc), total);
+#pragma unroll
+            for (int i = 0; i < DOWN_CHOICES; ++i)
+                if (c0 + i < top) part = fmaf(weight_s[c0 + i], acc[i], part);
         }
+        float total = wave_sum(part);
         if (lane == 0) {
             if (add0) total += to_float(add0[(size_t)t * width + r]);
             if (add1) total += to_float(add1[(size_t)t * width + r]);
@@ -268,7 +294,8 @@ PALM_API int palm_moe_route(hipStream_t stream, const float* logits, int n_token
     PALM_CHECK(experts <= ROUTE_MAX_PER_LANE * WAVE, "moe_route: %d experts exceed %d", experts, ROUTE_MAX_PER_LANE * WAVE);
     PALM_CHECK(top <= WAVE, "moe_route: %d choices a token exceed %d", top, WAVE);
     if (n_tokens == 0) return 0;
-    moe_route_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, experts, top, chosen, weight);
+    if (experts <= WAVE) moe_route_kernel<1><<<n_tokens, WAVE, 0, stream>>>(logits, experts, top, chosen, weight);
+    else moe_route_kernel<ROUTE_MAX_PER_LANE><<<n_tokens, WAVE, 0, stream>>>(logits, experts, top, chosen, weight);
     PALM_LAUNCHED();
     return 0;
 }
@@ -285,7 +312,12 @@ PALM_API int palm_moe_route_scored(hipStream_t stream, const float* logits, int 
     PALM_CHECK((long long)keep * (experts / groups) >= top, "moe_route_scored: %d groups of %d experts cannot give %d choices", keep,
                experts / groups, top);
     if (n_tokens == 0) return 0;
-    moe_route_scored_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, stride, experts, top, correction, groups, keep, scale, softmax, group_largest, chosen, weight);
+    if (experts <= WAVE)
+        moe_route_scored_kernel<1><<<n_tokens, WAVE, 0, stream>>>(logits, stride, experts, top, correction, groups, keep, scale, softmax, group_largest,
+                                                                 chosen, weight);
+    else
+        moe_route_scored_kernel<ROUTE_MAX_PER_LANE><<<n_tokens, WAVE, 0, stream>>>(logits, stride, experts, top, correction, groups, keep, scale, softmax,
+                                                                                  group_largest, chosen, weight);
     PALM_LAUNCHED();
     return 0;
 }
@@ -317,7 +349,7 @@ PALM_API int palm_moe_experts(hipStream_t stream, const void* h, int dtype, cons
     PALM_CHECK(form != EXPERT_CAPPED || limit > 0.f, "moe_experts: the cap %g must be positive", (double)limit);
     PALM_CHECK(n_tokens >= 0 && top > 0 && width > 0 && ff > 0, "moe_experts: n=%d top=%d width=%d ff=%d", n_tokens, top, width, ff);
     PALM_CHECK(width <= 16384 && (long long)top * ff <= 16384, "moe_experts: width %d / top x ff %d x %d exceed what a block holds", width, top, ff);
-    PALM_CHECK(n_tokens <= 65535 && top <= 65535, "moe_experts: %d tokens x %d choices are more than one launch takes", n_tokens, top);
+    PALM_CHECK(n_tokens <= 65535 && top <= WAVE, "moe_experts: %d tokens x %d choices are more than one launch takes", n_tokens, top);
     if (n_tokens == 0) return 0;
     // blocks enough to fill the chip, but no fewer than four rows a wave
     const int up_rows = max(16, (ff + 15) / 16), up_blocks = (ff + up_rows - 1) / up_rows;
