@@ -9,10 +9,12 @@
 // expanded, all heads read the same rows.  Scores, softmax and sums are 32-bit.
 //
 //   latent_prep        the joined down projection's rows -> the normed query latent; the normed latent and the
-//                      rotated key part into the position's cache row (and, where the caller keeps one for the prompt
-//                      kernel of latent_attention_mfma.hip, the latent into a bfloat16 copy with the positions innermost)
-//   latent_query       q rows -> [a_h | rotated q_rot,h] per head, 32-bit
-//   latent_attention   softmax over the visible rows (causal, optional window), o_lat,h = sum_j p_j c_j, 32-bit
+//                      rotated key part into the position's cache row (and, where the caller keeps one for the kernels
+//                      of latent_attention_mfma.hip, the latent into a bfloat16 copy with the positions innermost)
+//   latent_query       q rows -> [a_h | rotated q_rot,h] per head, 32-bit; where the queries come straight from the layer's
+//                      input (no query latent to be normed first) the same launch writes the positions' cache rows
+//   latent_attention   softmax over the visible rows (causal, optional window, optionally one more term exp(sink_h) in the
+//                      denominator), o_lat,h = sum_j p_j c_j, 32-bit
 //   latent_output      head h: sigmoid(gate_h) * U_v,h o_lat,h
 #include "common.h"
 
@@ -33,6 +35,10 @@ __device__ inline void lat_load8(const float* p, float (&v)[8]) {
     v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
 }
 
+// The two members of rotated pair i of `half` pairs: (i, i + half), or neighbours (2i, 2i + 1).
+__device__ inline int pair_first(int i, int neighbours) { return neighbours ? 2 * i : i; }
+__device__ inline int pair_second(int i, int half, int neighbours) { return neighbours ? 2 * i + 1 : half + i; }
+
 // One block per token.  down: [n, stride] holding the query latent at 0 (q_rank), the key/value latent at kv_off
 // (kv_rank) and the key part to rotate behind it (rot_dim).  rows_cache: [pages, PAGE_TOKENS, kv_rank + rot_dim].
 template <typename T>
@@ -41,7 +47,7 @@ __global__ __launch_bounds__(LAT_THREADS) void latent_prep_kernel(
     const float* __restrict__ kv_norm_w, float eps, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
     const int* __restrict__ positions, const int* __restrict__ tok_slot, const int* __restrict__ block_table, int max_pages,
     T* __restrict__ rows_cache, int write_cache, T* __restrict__ cq, bf16_t* __restrict__ rows_t,
-    const int* __restrict__ block_table_t) {
+    const int* __restrict__ block_table_t, int neighbours) {
     __shared__ float scratch[16];
     const size_t row = blockIdx.x;
     const T* dr = down + row * stride;
@@ -74,42 +80,91 @@ __global__ __launch_bounds__(LAT_THREADS) void latent_prep_kernel(
     const int half = rot_dim / 2;
     for (int i = threadIdx.x; i < half; i += LAT_THREADS) {
         const float c = cos_t[row * half + i], s = sin_t[row * half + i];
-        const float a = to_float(dr[kv_off + kv_rank + i]), b = to_float(dr[kv_off + kv_rank + half + i]);
-        cr[kv_rank + i] = from_float<T>(a * c - b * s);
-        cr[kv_rank + half + i] = from_float<T>(b * c + a * s);
+        const int i0 = kv_rank + pair_first(i, neighbours), i1 = kv_rank + pair_second(i, half, neighbours);
+        const float a = to_float(dr[kv_off + i0]), b = to_float(dr[kv_off + i1]);
+        cr[i0] = from_float<T>(a * c - b * s);
+        cr[i1] = from_float<T>(b * c + a * s);
     }
 }
 
-// One block per (tile of LQ_TILE tokens, head, run of LQ_COLS latent columns).  q: [n, heads * (dim + rot_dim)], a head's
-// plain part first.  uk: [heads * dim, kv_rank].  qa: float32 [n, heads, kv_rank + rot_dim].  A thread owns a column of
-// the key matrix and walks down it (neighbouring threads read neighbouring values); the first run's block also rotates.
+// What latent_query writes to the cache beside its queries: src rows hold the latent at column 0 and the key part behind it.
+template <typename T> struct LatentStore {
+    const T* src;                    // null: nothing is written
+    int stride;
+    const float* norm_w;
+    float eps;
+    const int *positions, *tok_slot, *block_table;
+    int max_pages;
+    T* rows;
+    bf16_t* rows_t;                  // null, or the transposed copy with its page table
+    const int* block_table_t;
+};
+
+// One wave writes the cache row of token `row`, as latent_prep does.
+template <typename T>
+__device__ inline void latent_store_row(const LatentStore<T>& st, size_t row, int kv_rank, int rot_dim, const float* __restrict__ cos_t,
+                                        const float* __restrict__ sin_t, int neighbours, int lane) {
+    const T* dr = st.src + row * st.stride;
+    float ss = 0.f;
+    for (int d = lane; d < kv_rank; d += WAVE) {
+        const float v = to_float(dr[d]);
+        ss = fmaf(v, v, ss);
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)kv_rank + st.eps);
+    const int pos = st.positions[row];
+    const size_t entry = (size_t)st.tok_slot[row] * st.max_pages + pos / PAGE_TOKENS;
+    T* cr = st.rows + ((size_t)st.block_table[entry] * PAGE_TOKENS + pos % PAGE_TOKENS) * (kv_rank + rot_dim);
+    bf16_t* ct = st.rows_t ? st.rows_t + (size_t)st.block_table_t[entry] * kv_rank * PAGE_TOKENS + pos % PAGE_TOKENS : nullptr;
+    for (int d = lane; d < kv_rank; d += WAVE) {
+        const float v = (to_float(dr[d]) * inv) * st.norm_w[d];
+        cr[d] = from_float<T>(v);
+        if (ct) ct[(size_t)d * PAGE_TOKENS] = f32_to_bf16(v);
+    }
+    const int half = rot_dim / 2;
+    for (int i = lane; i < half; i += WAVE) {
+        const float c = cos_t[row * half + i], s = sin_t[row * half + i];
+        const int i0 = kv_rank + pair_first(i, neighbours), i1 = kv_rank + pair_second(i, half, neighbours);
+        const float a = to_float(dr[i0]), b = to_float(dr[i1]);
+        cr[i0] = from_float<T>(a * c - b * s);
+        cr[i1] = from_float<T>(b * c + a * s);
+    }
+}
+
+// One block per (tile of LQ_TILE tokens, head, run of LQ_COLS latent columns).  q: [n, heads * (dim + rot_dim)] (rows
+// q_stride apart), a head's plain part first.  uk: [heads * dim, kv_rank].  qa: float32 [n, heads, kv_rank + rot_dim].  A thread owns a column of
+// the key matrix and walks down it (neighbouring threads read neighbouring values); the first run's block also rotates, and
+// (st) the first runs' blocks share out the tile's cache rows, a token for each head in turn.
 constexpr int LQ_TILE = 8;
 constexpr int LQ_COLS = 64;
 constexpr int LQ_MAX_DIM = 512;
 
 template <typename T, typename TW>
 __global__ __launch_bounds__(LQ_COLS) void latent_query_kernel(
-    const T* __restrict__ q, const TW* __restrict__ uk, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
-    int n_tokens, int heads, int dim, int rot_dim, int kv_rank, float* __restrict__ qa) {
+    const T* __restrict__ q, int q_stride, const TW* __restrict__ uk, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+    int n_tokens, int heads, int dim, int rot_dim, int kv_rank, int neighbours, LatentStore<T> st, float* __restrict__ qa) {
     __shared__ float q_s[LQ_TILE][LQ_MAX_DIM];
     const int t0 = blockIdx.x * LQ_TILE, h = blockIdx.y;
     const int tt = min(LQ_TILE, n_tokens - t0);
     const int hd = dim + rot_dim, dk = kv_rank + rot_dim, half = rot_dim / 2;
     for (int idx = threadIdx.x; idx < LQ_TILE * dim; idx += LQ_COLS) {
         const int ti = idx / dim, d = idx % dim;
-        q_s[ti][d] = ti < tt ? to_float(q[((size_t)(t0 + ti) * heads + h) * hd + d]) : 0.f;
+        q_s[ti][d] = ti < tt ? to_float(q[(size_t)(t0 + ti) * q_stride + (size_t)h * hd + d]) : 0.f;
     }
     if (blockIdx.z == 0) {
         for (int idx = threadIdx.x; idx < tt * half; idx += LQ_COLS) {
             const int ti = idx / half, i = idx % half;
             const size_t row = t0 + ti;
-            const T* qr = q + (row * heads + h) * hd + dim;
+            const T* qr = q + row * q_stride + (size_t)h * hd + dim;
             const float c = cos_t[row * half + i], s = sin_t[row * half + i];
-            const float a = to_float(qr[i]), b = to_float(qr[half + i]);
+            const int i0 = pair_first(i, neighbours), i1 = pair_second(i, half, neighbours);
+            const float a = to_float(qr[i0]), b = to_float(qr[i1]);
             float* o = qa + (row * heads + h) * dk + kv_rank;
-            o[i] = a * c - b * s;
-            o[half + i] = b * c + a * s;
+            o[i0] = a * c - b * s;
+            o[i1] = b * c + a * s;
         }
+        if (st.src)
+            for (int ti = h; ti < tt; ti += gridDim.y)
+                latent_store_row(st, (size_t)(t0 + ti), kv_rank, rot_dim, cos_t, sin_t, neighbours, threadIdx.x);
     }
     __syncthreads();
     const TW* w = uk + (size_t)h * dim * kv_rank;
@@ -142,7 +197,8 @@ template <typename T, int HG, int ACC>
 __global__ __launch_bounds__(LA_WAVES * WAVE) void latent_attention_kernel(
     const float* __restrict__ qa, const T* __restrict__ rows_cache, const int* __restrict__ block_table, int max_pages,
     const int* __restrict__ seq_slot, const int* __restrict__ seq_start, const int* __restrict__ seq_new,
-    const int* __restrict__ cu_new, int heads, int kv_rank, int rot_dim, float scale, int window, float* __restrict__ out) {
+    const int* __restrict__ cu_new, int heads, int kv_rank, int rot_dim, float scale, int window,
+    const float* __restrict__ sink_scores, float* __restrict__ out) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int dk = kv_rank + rot_dim;
     float* q_s = lds;                                  // [HG][dk]
@@ -168,8 +224,10 @@ __global__ __launch_bounds__(LA_WAVES * WAVE) void latent_attention_kernel(
     float m[HG], l[HG], acc[HG][ACC];
 #pragma unroll
     for (int g = 0; g < HG; ++g) {
-        m[g] = -INFINITY;
-        l[g] = 0.f;
+        // the sink is a key of a learned score without a value: the first wave's running maximum and sum start from it
+        const bool sink_here = sink_scores && wave == 0;
+        m[g] = sink_here ? sink_scores[min(h0 + g, heads - 1)] : -INFINITY;
+        l[g] = sink_here ? 1.f : 0.f;
 #pragma unroll
         for (int i = 0; i < ACC; ++i) acc[g][i] = 0.f;
     }
@@ -321,7 +379,8 @@ __global__ __launch_bounds__(LAT_THREADS) void latent_output_kernel(
 PALM_API int palm_latent_prep(hipStream_t stream, const void* down, int dtype, int stride, int q_rank, int kv_off, int kv_rank,
                               int rot_dim, const float* q_norm_w, const float* kv_norm_w, float eps, const float* cos_t,
                               const float* sin_t, const int* positions, const int* tok_slot, const int* block_table, int max_pages,
-                              void* rows_cache, int write_cache, void* cq, int n_tokens, void* rows_t, const int* block_table_t) {
+                              void* rows_cache, int write_cache, void* cq, int n_tokens, void* rows_t, const int* block_table_t,
+                              int pairing) {
     PALM_CHECK(n_tokens >= 0 && q_rank > 0 && kv_rank > 0 && rot_dim >= 0 && rot_dim % 2 == 0, "latent_prep: n=%d q_rank=%d kv_rank=%d rot_dim=%d",
                n_tokens, q_rank, kv_rank, rot_dim);
     PALM_CHECK(stride >= kv_off + kv_rank + rot_dim && kv_off >= q_rank, "latent_prep: rows of %d do not hold %d + %d + %d", stride, q_rank,
@@ -329,29 +388,42 @@ PALM_API int palm_latent_prep(hipStream_t stream, const void* down, int dtype, i
     PALM_CHECK(rot_dim == 0 || (cos_t && sin_t), "latent_prep: a rotation needs its cos and sin rows");
     PALM_CHECK(max_pages > 0, "latent_prep: max_pages %d", max_pages);
     PALM_CHECK(!rows_t || block_table_t, "latent_prep: the transposed copy needs its page table");
+    PALM_CHECK(pairing == 0 || pairing == 1, "latent_prep: pairing %d is neither halves (0) nor neighbours (1)", pairing);
     if (n_tokens == 0) return 0;
     PALM_DTYPE_SWITCH(dtype, T,
         latent_prep_kernel<T><<<n_tokens, LAT_THREADS, 0, stream>>>((const T*)down, stride, q_rank, kv_off, kv_rank, rot_dim, q_norm_w,
                                                                    kv_norm_w, eps, cos_t, sin_t, positions, tok_slot, block_table,
                                                                    max_pages, (T*)rows_cache, write_cache, (T*)cq, (bf16_t*)rows_t,
-                                                                   block_table_t));
+                                                                   block_table_t, pairing));
     PALM_LAUNCHED();
     return 0;
 }
 
-PALM_API int palm_latent_query(hipStream_t stream, const void* q, int dtype, const void* uk, int w_dtype, const float* cos_t,
-                               const float* sin_t, int n_tokens, int heads, int dim, int rot_dim, int kv_rank, float* qa) {
+// store: null, or the first token's latent in rows `store_stride` elements apart (the latent, then the key part to rotate): its
+// norm and rotation go to rows_cache (and the latent to rows_t) as latent_prep has it.
+PALM_API int palm_latent_query(hipStream_t stream, const void* q, int dtype, int q_stride, const void* uk, int w_dtype, const float* cos_t,
+                               const float* sin_t, int n_tokens, int heads, int dim, int rot_dim, int kv_rank, int pairing, float* qa,
+                               const void* store, int store_stride, const float* kv_norm_w, float eps, const int* positions,
+                               const int* tok_slot, const int* block_table, int max_pages, void* rows_cache, void* rows_t,
+                               const int* block_table_t) {
     PALM_CHECK(n_tokens >= 0 && heads > 0 && dim > 0 && kv_rank > 0 && rot_dim >= 0 && rot_dim % 2 == 0,
                "latent_query: n=%d heads=%d dim=%d rot_dim=%d kv_rank=%d", n_tokens, heads, dim, rot_dim, kv_rank);
     PALM_CHECK(dim <= LQ_MAX_DIM, "latent_query: an unrotated key size of %d exceeds %d", dim, LQ_MAX_DIM);
     PALM_CHECK(rot_dim == 0 || (cos_t && sin_t), "latent_query: a rotation needs its cos and sin rows");
     PALM_CHECK(heads <= 65535, "latent_query: %d heads are more than one launch takes", heads);
+    PALM_CHECK(q_stride >= heads * (dim + rot_dim), "latent_query: rows of %d do not hold %d heads of %d + %d", q_stride, heads, dim, rot_dim);
+    PALM_CHECK(pairing == 0 || pairing == 1, "latent_query: pairing %d is neither halves (0) nor neighbours (1)", pairing);
+    PALM_CHECK(!store || (kv_norm_w && positions && tok_slot && block_table && max_pages > 0 && rows_cache && store_stride >= kv_rank + rot_dim),
+               "latent_query: cache rows need the latents' norm, positions, slots, pages and rows of %d + %d", kv_rank, rot_dim);
+    PALM_CHECK(!rows_t || block_table_t, "latent_query: the transposed copy needs its page table");
     if (n_tokens == 0) return 0;
     dim3 grid((n_tokens + LQ_TILE - 1) / LQ_TILE, heads, (kv_rank + LQ_COLS - 1) / LQ_COLS);
     PALM_DTYPE_SWITCH(dtype, T, {
         PALM_DTYPE_SWITCH(w_dtype, TW, {
-            latent_query_kernel<T, TW><<<grid, LQ_COLS, 0, stream>>>((const T*)q, (const TW*)uk, cos_t, sin_t, n_tokens, heads, dim,
-                                                                        rot_dim, kv_rank, qa);
+            const LatentStore<T> st{(const T*)store, store_stride, kv_norm_w, eps, positions, tok_slot, block_table, max_pages, (T*)rows_cache,
+                                    (bf16_t*)rows_t, block_table_t};
+            latent_query_kernel<T, TW><<<grid, LQ_COLS, 0, stream>>>((const T*)q, q_stride, (const TW*)uk, cos_t, sin_t, n_tokens, heads, dim,
+                                                                        rot_dim, kv_rank, pairing, st, qa);
         });
     });
     PALM_LAUNCHED();
@@ -360,7 +432,8 @@ PALM_API int palm_latent_query(hipStream_t stream, const void* q, int dtype, con
 
 PALM_API int palm_latent_attention(hipStream_t stream, const float* qa, const void* rows_cache, int dtype, const int* block_table,
                                    int max_pages, const int* seq_slot, const int* seq_start, const int* seq_new, const int* cu_new,
-                                   int n_seqs, int max_new, int heads, int kv_rank, int rot_dim, float scale, int window, float* out) {
+                                   int n_seqs, int max_new, int heads, int kv_rank, int rot_dim, float scale, int window,
+                                   const float* sink_scores, float* out) {
     PALM_CHECK(n_seqs >= 0 && max_new >= 0 && heads > 0 && kv_rank > 0 && rot_dim >= 0, "latent_attention: seqs=%d max_new=%d heads=%d kv_rank=%d rot_dim=%d",
                n_seqs, max_new, heads, kv_rank, rot_dim);
     PALM_CHECK(kv_rank <= LA_MAX_RANK && kv_rank + rot_dim <= LA_MAX_DK, "latent_attention: a latent of %d + %d exceeds %d + %d", kv_rank, rot_dim,
@@ -374,7 +447,7 @@ PALM_API int palm_latent_attention(hipStream_t stream, const float* qa, const vo
     dim3 grid(max_new, (heads + hg - 1) / hg, n_seqs);
     const size_t lds = (size_t)hg * (2 * kv_rank + rot_dim) * sizeof(float);
 #define LA_CASE(HGV, ACCV) latent_attention_kernel<T, HGV, ACCV><<<grid, LA_WAVES * WAVE, lds, stream>>>( \
-        qa, (const T*)rows_cache, block_table, max_pages, seq_slot, seq_start, seq_new, cu_new, heads, kv_rank, rot_dim, scale, window, out)
+        qa, (const T*)rows_cache, block_table, max_pages, seq_slot, seq_start, seq_new, cu_new, heads, kv_rank, rot_dim, scale, window, sink_scores, out)
     PALM_DTYPE_SWITCH(dtype, T, {
         if (acc <= 1) LA_CASE(4, 1);
         else if (acc <= 2) LA_CASE(4, 2);

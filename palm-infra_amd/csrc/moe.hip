@@ -5,9 +5,11 @@
 //   few rows (a decode step): nothing is planned on the host, every (token, choice) reads its expert's weights itself
 //     expert_gate_up   mid[t, c, f] = silu(G_e h_t)[f] * (U_e h_t)[f],  e = chosen[t, c]           (32-bit)
 //     expert_down      out[t, :] = sum_c weight[t, c] * D_e mid[t, c, :]                          (32-bit)
-//   An expert's form: gated (silu(G h) * (U h), the gate rows before the up rows), plain with the exact gelu (gelu(U h)), or
-//   capped gated (g sigmoid(slope g) (u + shift) with g = min(G h, limit), u = clamp(U h, -limit, limit)).
-//   Rows that other branches made (up to two) can be added to the weighted sum where it is written.
+//   An expert's form: gated (silu(G h) * (U h), the gate rows before the up rows), plain with the exact gelu (gelu(U h)) or the
+//   squared relu (max(U h, 0)^2), or capped gated (g sigmoid(slope g) (u + shift) with g = min(G h, limit), u = clamp(U h, -limit, limit)).
+//   Rows that other branches made (up to two) can be added to the weighted sum where it is written; so can one more expert of
+//   the same form, with an inner size of its own, that every token goes through with weight one (the shared expert).
+//   The choices are rows [n, top], or rows of a table that each token's id picks (all choices then weigh 1 / top).
 //
 //   route, scored: the scores are sigmoid(logit) or the softmax over all experts; the choice is made by score plus a
 //              correction per expert (or by the score alone); experts lie in
@@ -153,21 +155,44 @@ __global__ __launch_bounds__(WAVE) void moe_route_scored_kernel(const float* __r
     if (lane < top) weight[t * top + lane] = mine / (sum + 1e-20f) * scale;
 }
 
-// grid (blocks of rows of the expert's inner size, top, tokens); a wave computes a gate row and its up row at a time.
+// The choices of a feed-forward whose experts a table chooses by token id: chosen[t] = table[ids[t]], each with weight 1 / top.
+__global__ void moe_route_table_kernel(const int* __restrict__ ids, const int* __restrict__ table, int vocab, int top, int n_pairs,
+                                       int* __restrict__ chosen, float* __restrict__ weight) {
+    const int p = blockIdx.x * blockDim.x + threadIdx.x;
+    if (p >= n_pairs) return;
+    chosen[p] = table[(size_t)min(max(ids[p / top], 0), vocab - 1) * top + p % top];       // (an id outside the table has no rows: the last one's stand in)
+    weight[p] = 1.0f / (float)top;
+}
+
+// Choice c of token t.
+struct Choices {
+    const int* rows;                 // [n, top], or with ids the table [vocab, top]
+    const float* weight;             // [n, top]; null: 1 / top
+    const int* ids;                  // null, or the tokens' ids
+    int vocab, top;
+    __device__ int expert(int t, int c) const { return rows[(size_t)(ids ? min(max(ids[t], 0), vocab - 1) : t) * top + c]; }
+    __device__ float of(int t, int c) const { return weight ? weight[(size_t)t * top + c] : 1.0f / (float)top; }
+};
+
+// grid (blocks of rows of the expert's inner size, top (+ 1 with a shared expert), tokens); a wave computes a gate row and its up
+// row at a time.
 constexpr int MOE_THREADS = 256;
 
 template <typename T, typename TW>
 __global__ __launch_bounds__(MOE_THREADS) void expert_gate_up_kernel(const T* __restrict__ h, const TW* __restrict__ gate_up,
-                                                                     const int* __restrict__ chosen, int top, int width, int ff,
-                                                                     int rows_per_block, int form, ExpertCap cap, float* __restrict__ mid) {
+                                                                     Choices choices, int width, int ff, const TW* __restrict__ shared_up,
+                                                                     int shared_ff, int rows_per_block, int form, ExpertCap cap,
+                                                                     float* __restrict__ mid) {
     extern __shared__ float h_s[];                  // [width]
     const int t = blockIdx.z, c = blockIdx.y;
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, n_waves = MOE_THREADS / WAVE;
     for (int d = threadIdx.x; d < width; d += MOE_THREADS) h_s[d] = to_float(h[(size_t)t * width + d]);
     __syncthreads();
-    const int e = chosen[(size_t)t * top + c];
-    const bool gated = form != EXPERT_GELU;         // else: up rows alone, through the exact gelu
-    const TW* w = gate_up + (size_t)e * (gated ? 2 : 1) * ff * width;
+    const bool gated = expert_is_gated(form);       // else: up rows alone
+    const bool is_shared = c == choices.top;        // (the shared expert runs behind the chosen ones)
+    const TW* w = is_shared ? shared_up : gate_up + (size_t)choices.expert(t, c) * (gated ? 2 : 1) * ff * width;
+    const int row_ff = choices.top * ff + shared_ff;               // inner values of a token: its choices', then the shared expert's
+    if (is_shared) ff = shared_ff;
     const int f_end = min(ff, (int)(blockIdx.x + 1) * rows_per_block);
     // Two rows of the first matrix are under way at a time in both forms: an inner value's gate row and up row, or (plain)
     // the up rows of two inner values, the wave's own and the one n_waves further on.
@@ -199,12 +224,12 @@ __global__ __launch_bounds__(MOE_THREADS) void expert_gate_up_kernel(const T* __
         u = wave_sum(u);
         g = wave_sum(g);
         if (lane == 0) {
-            float* m = mid + ((size_t)t * top + c) * ff;
+            float* m = mid + (size_t)t * row_ff + (is_shared ? row_ff - shared_ff : c * ff);
             if (gated) {
                 m[f] = form == EXPERT_CAPPED ? expert_capped(g, u, cap) : expert_silu_gated(g, u);
             } else {
-                m[f] = expert_gelu(u);
-                if (f2 < f_end) m[f2] = expert_gelu(g);
+                m[f] = expert_plain(form, u);
+                if (f2 < f_end) m[f2] = expert_plain(form, g);
             }
         }
     }
@@ -216,19 +241,20 @@ constexpr int DOWN_CHOICES = 4;
 // `add0`, `add1`: null, or rows [n, width] that other branches made, added to the sum.
 template <typename T, typename TW>
 __global__ __launch_bounds__(MOE_THREADS) void expert_down_kernel(const float* __restrict__ mid, const TW* __restrict__ down,
-                                                                  const int* __restrict__ chosen, const float* __restrict__ weight,
-                                                                  int top, int width, int ff, int rows_per_block,
+                                                                  Choices choices, int width, int ff, const TW* __restrict__ shared_down,
+                                                                  int shared_ff, int rows_per_block,
                                                                   const T* __restrict__ add0, const T* __restrict__ add1,
                                                                   float* __restrict__ out) {
-    extern __shared__ float m_s[];                  // [top][ff]
+    extern __shared__ float m_s[];                  // [top][ff] (, the shared expert's values)
     __shared__ int expert_s[WAVE];
     __shared__ float weight_s[WAVE];
     const int t = blockIdx.y;
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, n_waves = MOE_THREADS / WAVE;
-    for (int i = threadIdx.x; i < top * ff; i += MOE_THREADS) m_s[i] = mid[(size_t)t * top * ff + i];
+    const int top = choices.top, row_ff = top * ff + shared_ff;
+    for (int i = threadIdx.x; i < row_ff; i += MOE_THREADS) m_s[i] = mid[(size_t)t * row_ff + i];
     if (threadIdx.x < top) {
-        expert_s[threadIdx.x] = chosen[(size_t)t * top + threadIdx.x];
-        weight_s[threadIdx.x] = weight[(size_t)t * top + threadIdx.x];
+        expert_s[threadIdx.x] = choices.expert(t, threadIdx.x);
+        weight_s[threadIdx.x] = choices.of(t, threadIdx.x);
     }
     __syncthreads();
     const int r_end = min(width, (int)(blockIdx.x + 1) * rows_per_block);
@@ -263,6 +289,20 @@ __global__ __launch_bounds__(MOE_THREADS) void expert_down_kernel(const float* _
 #pragma unroll
             for (int i = 0; i < DOWN_CHOICES; ++i)
                 if (c0 + i < top) part = fmaf(weight_s[c0 + i], acc[i], part);
+        }
+        if (shared_ff) {
+            const TW* sr = shared_down + (size_t)r * shared_ff;
+            const float* m = m_s + top * ff;
+            if (shared_ff % 8 == 0) {
+                for (int f = lane * 8; f < shared_ff; f += WAVE * 8) {
+                    float wv[8];
+                    load8(sr + f, wv);
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) part = fmaf(wv[j], m[f + j], part);
+                }
+            } else {
+                for (int f = lane; f < shared_ff; f += WAVE) part = fmaf(to_float(sr[f]), m[f], part);
+            }
         }
         float total = wave_sum(part);
         if (lane == 0) {
@@ -339,27 +379,47 @@ PALM_API int palm_add_gated_rows(hipStream_t stream, float* out, const void* y, 
     return 0;
 }
 
-// h [n, width]; gate_up [experts, 2 ff, width] (an expert's gate rows, then its up rows; the gelu form: [experts, ff, width], up
+// chosen int32 [n, top] = table[ids], weight float32 [n, top] = 1 / top.  The table's entries are checked by whoever keeps it.
+PALM_API int palm_moe_route_table(hipStream_t stream, const int* ids, const int* table, int vocab, int n_tokens, int top, int* chosen,
+                                  float* weight) {
+    PALM_CHECK(n_tokens >= 0 && vocab > 0 && top > 0 && (long long)n_tokens * top < (1ll << 30), "moe_route_table: n=%d vocab=%d top=%d", n_tokens,
+               vocab, top);
+    if (n_tokens == 0) return 0;
+    moe_route_table_kernel<<<(n_tokens * top + 255) / 256, 256, 0, stream>>>(ids, table, vocab, top, n_tokens * top, chosen, weight);
+    PALM_LAUNCHED();
+    return 0;
+}
+
+// h [n, width]; gate_up [experts, 2 ff, width] (an expert's gate rows, then its up rows; the plain forms: [experts, ff, width], up
 // rows alone); add0, add1: null or rows [n, width] of h's type; down [experts, width, ff];
-// chosen, weight [n, top]; mid: room for n * top * ff floats; out float32 [n, width].
+// chosen, weight [n, top], or with ids [n] the table [vocab, top] and no weight; shared_up, shared_down: null, or one more expert's
+// matrices, of inner size shared_ff; mid: room for n * (top * ff + shared_ff) floats; out float32 [n, width].
 PALM_API int palm_moe_experts(hipStream_t stream, const void* h, int dtype, const void* gate_up, const void* down, int w_dtype,
                               const int* chosen, const float* weight, int n_tokens, int top, int width, int ff, float* mid,
-                              float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1) {
-    PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_CAPPED, "moe_experts: form %d is neither gated silu (0) nor plain gelu (1) nor capped gated (2)", form);
+                              float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1,
+                              const int* ids, int vocab, const void* shared_up, const void* shared_down, int shared_ff) {
+    PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_RELU_SQUARED, "moe_experts: form %d is neither gated silu (0) nor plain gelu (1) nor capped "
+               "gated (2) nor squared relu (3)", form);
+    PALM_CHECK(ids ? vocab > 0 : weight != nullptr, "moe_experts: choices come with weights, or from a table of %d ids", vocab);
+    PALM_CHECK(shared_ff >= 0 && (shared_ff == 0 || (shared_up && shared_down)), "moe_experts: a shared expert of inner size %d needs its matrices", shared_ff);
     PALM_CHECK(form != EXPERT_CAPPED || limit > 0.f, "moe_experts: the cap %g must be positive", (double)limit);
     PALM_CHECK(n_tokens >= 0 && top > 0 && width > 0 && ff > 0, "moe_experts: n=%d top=%d width=%d ff=%d", n_tokens, top, width, ff);
-    PALM_CHECK(width <= 16384 && (long long)top * ff <= 16384, "moe_experts: width %d / top x ff %d x %d exceed what a block holds", width, top, ff);
+    PALM_CHECK(width <= 16384 && (long long)top * ff + shared_ff <= 16384, "moe_experts: width %d / top x ff %d x %d + %d exceed what a block holds",
+               width, top, ff, shared_ff);
     PALM_CHECK(n_tokens <= 65535 && top <= WAVE, "moe_experts: %d tokens x %d choices are more than one launch takes", n_tokens, top);
     if (n_tokens == 0) return 0;
     // blocks enough to fill the chip, but no fewer than four rows a wave
-    const int up_rows = max(16, (ff + 15) / 16), up_blocks = (ff + up_rows - 1) / up_rows;
+    const int longest = max(ff, shared_ff);
+    const int up_rows = max(16, (longest + 15) / 16), up_blocks = (longest + up_rows - 1) / up_rows;
+    const Choices choices{chosen, weight, ids, vocab, top};
     const int down_rows = max(16, (width + 63) / 64), down_blocks = (width + down_rows - 1) / down_rows;
     PALM_DTYPE_SWITCH(dtype, T, {
         PALM_DTYPE_SWITCH(w_dtype, TW, {
-            expert_gate_up_kernel<T, TW><<<dim3(up_blocks, top, n_tokens), MOE_THREADS, width * sizeof(float), stream>>>(
-                (const T*)h, (const TW*)gate_up, chosen, top, width, ff, up_rows, form, ExpertCap{limit, slope, shift}, mid);
-            expert_down_kernel<T, TW><<<dim3(down_blocks, n_tokens), MOE_THREADS, (size_t)top * ff * sizeof(float), stream>>>(
-                mid, (const TW*)down, chosen, weight, top, width, ff, down_rows, (const T*)add0, (const T*)add1, out);
+            expert_gate_up_kernel<T, TW><<<dim3(up_blocks, top + (shared_ff > 0), n_tokens), MOE_THREADS, width * sizeof(float), stream>>>(
+                (const T*)h, (const TW*)gate_up, choices, width, ff, (const TW*)shared_up, shared_ff, up_rows, form,
+                ExpertCap{limit, slope, shift}, mid);
+            expert_down_kernel<T, TW><<<dim3(down_blocks, n_tokens), MOE_THREADS, ((size_t)top * ff + shared_ff) * sizeof(float), stream>>>(
+                mid, (const TW*)down, choices, width, ff, (const TW*)shared_down, shared_ff, down_rows, (const T*)add0, (const T*)add1, out);
         });
     });
     PALM_LAUNCHED();

@@ -97,7 +97,7 @@ __global__ __launch_bounds__(PLAN_THREADS) void moe_place_kernel(const int* __re
 // grid (tiles, blocks of GT_FEATURES features).  a: the rows [*, k_dim]; row_of_slot: null (the rows lie in slot order) or
 // slot -> pair, the pair's row being pair / top.  w: [experts, n_w_rows, k_dim]; FORM 1 (gated): n_w_rows = 2 n_features, an
 // expert's gate rows first, and the result is silu(gate) * up; FORM 3: the same rows, capped gated; FORM 2: the product through
-// the exact gelu; FORM 0: the product as it is.  out: bfloat16 [slots, n_features].
+// the exact gelu; FORM 4: the product through the squared relu; FORM 0: the product as it is.  out: bfloat16 [slots, n_features].
 template <int FORM>
 __global__ __launch_bounds__(GT_WAVES * WAVE) void moe_grouped_kernel(const bf16_t* __restrict__ a, const int* __restrict__ slot_pair, int top,
                                                                       const bf16_t* __restrict__ w, const int* __restrict__ tile_expert,
@@ -159,6 +159,8 @@ __global__ __launch_bounds__(GT_WAVES * WAVE) void moe_grouped_kernel(const bf16
                     v[i] = FORM == 3 ? expert_capped(acc[ft][tt][i], acc[2 + ft][tt][i], cap) : expert_silu_gated(acc[ft][tt][i], acc[2 + ft][tt][i]);
                 } else if (FORM == 2) {
                     v[i] = expert_gelu(acc[ft][tt][i]);
+                } else if (FORM == 4) {
+                    v[i] = expert_relu_squared(acc[ft][tt][i]);
                 } else {
                     v[i] = acc[ft][tt][i];
                 }
@@ -185,14 +187,15 @@ __global__ void moe_combine_kernel(const bf16_t* __restrict__ y, const int* __re
 
 PALM_API int palm_moe_tile_tokens() { return GT_TOKENS; }
 
-// chosen, weight [n, top]; h bfloat16 [n, width]; gate_up bfloat16 [experts, 2 ff, width] (the gelu form: [experts, ff, width], up
+// chosen, weight [n, top]; h bfloat16 [n, width]; gate_up bfloat16 [experts, 2 ff, width] (the plain forms: [experts, ff, width], up
 // rows alone); add0, add1: null or bfloat16 rows [n, width]; down bfloat16 [experts, width, ff].
 // Room, with max_tiles = ceil(n top / tile) + experts and slots = max_tiles * tile: plan: (2 experts + 1 + max_tiles + slots
 // + n top) ints; mid: slots * ff bfloat16; y: slots * width bfloat16.  out float32 [n, width].
 PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gate_up, const void* down, const int* chosen,
                               const float* weight, int n_tokens, int top, int experts, int width, int ff, int* plan, void* mid, void* y,
                               float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1) {
-    PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_CAPPED, "moe_grouped: form %d is neither gated silu (0) nor plain gelu (1) nor capped gated (2)", form);
+    PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_RELU_SQUARED, "moe_grouped: form %d is neither gated silu (0) nor plain gelu (1) nor capped "
+               "gated (2) nor squared relu (3)", form);
     PALM_CHECK(form != EXPERT_CAPPED || limit > 0.f, "moe_grouped: the cap %g must be positive", (double)limit);
     PALM_CHECK(n_tokens >= 0 && top > 0 && experts > 0 && width > 0 && ff > 0, "moe_grouped: n=%d top=%d experts=%d width=%d ff=%d", n_tokens,
                top, experts, width, ff);
@@ -215,7 +218,8 @@ PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gat
         tile_expert, ff, width, cap, (bf16_t*)mid)
     if (form == EXPERT_GATED_SILU) MOE_UP(1);
     else if (form == EXPERT_GELU) MOE_UP(2);
-    else MOE_UP(3);
+    else if (form == EXPERT_CAPPED) MOE_UP(3);
+    else MOE_UP(4);
 #undef MOE_UP
     moe_grouped_kernel<0><<<dim3(max_tiles, (width + GT_FEATURES - 1) / GT_FEATURES), GT_WAVES * WAVE, 0, stream>>>(
         (const bf16_t*)mid, nullptr, top, (const bf16_t*)down, tile_expert, width, ff, cap, (bf16_t*)y);

@@ -8,6 +8,7 @@ are memory here; the one computation that torch does on the product path is the 
 from __future__ import annotations
 
 from ctypes import c_float, c_int, c_longlong, c_ulonglong, c_void_p
+from dataclasses import dataclass
 
 import torch
 
@@ -17,6 +18,7 @@ from .library import KernelError
 F32, BF16 = torch.float32, torch.bfloat16
 _CODES = {F32: 0, BF16: 1}
 PAGE_TOKENS = 64
+ROTARY_PAIRINGS = {"half_split": 0, "interleaved": 1}
 
 _SIGNATURES = {
     "palm_embed": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_float],
@@ -779,10 +781,11 @@ _MIXER_SIGNATURES = {
                         c_void_p, c_void_p, c_void_p, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                         c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p],
     "palm_latent_prep": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p,
-                         c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p],
-    "palm_latent_query": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+                         c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int],
+    "palm_latent_query": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                          c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
     "palm_latent_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                              c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
+                              c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p],
     "palm_latent_output": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
 }
 _mixers = None
@@ -820,7 +823,8 @@ _FEEDFORWARD_SIGNATURES = {
     "palm_moe_route_scored": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p],
     "palm_add_gated_rows": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int],
     "palm_moe_experts": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                         c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p],
+                         c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int],
+    "palm_moe_route_table": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
     "palm_moe_tile_tokens": [],
     "palm_moe_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
                          c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p],
@@ -1347,53 +1351,89 @@ def delta_head(rows: torch.Tensor, ab: torch.Tensor, conv_w: torch.Tensor, conv_
 
 def latent_prep(down: torch.Tensor, q_rank: int, kv_off: int, kv_rank: int, rot_dim: int, q_norm_w, kv_norm_w, eps: float,
                 cos, sin, rows_cache: torch.Tensor, block_table: torch.Tensor, ctx, write_cache: bool = True,
-                rows_t: torch.Tensor | None = None, table_t: torch.Tensor | None = None) -> torch.Tensor:
+                rows_t: torch.Tensor | None = None, table_t: torch.Tensor | None = None, pairing: str = "half_split") -> torch.Tensor:
     """down [n, >= kv_off + kv_rank + rot_dim]: the query latent at column 0, the key/value latent at ``kv_off`` and the key
     part to rotate behind it.  Returns the normed query latent [n, q_rank]; writes [normed latent | rotated key part] into
     each token's row of ``rows_cache`` [pages, PAGE_TOKENS, kv_rank + rot_dim] and, if given, the normed latent into
     ``rows_t`` (bfloat16 [pages, kv_rank, PAGE_TOKENS], with the page table ``table_t`` of its own)."""
     what = "latent_prep"
-    _dev(what, down, q_norm_w, kv_norm_w, cos, sin, rows_cache, block_table, ctx.positions, ctx.tok_slot, rows_t, table_t)
-    _i32(what, block_table, ctx.positions, ctx.tok_slot, table_t)
-    _need(rows_t is None or (table_t is not None and rows_t.dtype == BF16 and rows_t.dim() == 3 and rows_t.shape[1:] == (kv_rank, PAGE_TOKENS)
-                             and table_t.shape == block_table.shape),
-          f"{what}: the transposed copy is bfloat16 [pages, {kv_rank}, {PAGE_TOKENS}] with a page table like the rows'")
+    _dev(what, down, q_norm_w)
+    _latent_rows(what, down.dtype, kv_rank, rot_dim, kv_norm_w, rows_cache, block_table, ctx, rows_t, table_t, pairing)
     n = down.shape[0]
     _need(down.dim() == 2 and n == ctx.n_tokens, f"{what}: rows {tuple(down.shape)} for {ctx.n_tokens} tokens")
-    _need(q_norm_w.shape == (q_rank,) and q_norm_w.dtype == F32 and kv_norm_w.shape == (kv_rank,) and kv_norm_w.dtype == F32,
-          f"{what}: the norms' weights are float32 [{q_rank}] and [{kv_rank}]")
-    _need(rows_cache.dim() == 3 and rows_cache.shape[1:] == (PAGE_TOKENS, kv_rank + rot_dim) and rows_cache.dtype == down.dtype,
-          f"{what}: the cache {tuple(rows_cache.shape)} {rows_cache.dtype} is not {down.dtype} [pages, {PAGE_TOKENS}, {kv_rank + rot_dim}]")
-    if rot_dim:
-        for tab in (cos, sin):
-            _need(tab is not None and tab.dtype == F32 and tab.shape == (n, rot_dim // 2), f"{what}: rotation rows are float32 [{n}, {rot_dim // 2}]")
-    _need(block_table.dim() == 2, f"{what}: page table {tuple(block_table.shape)} is not [slots, pages]")
+    _need(q_norm_w.shape == (q_rank,) and q_norm_w.dtype == F32, f"{what}: the query norm's weight is float32 [{q_rank}]")
+    _latent_rotation(what, cos, sin, n, rot_dim)
     cq = torch.empty((n, q_rank), dtype=down.dtype, device=down.device)
     library.call(mixers(), "palm_latent_prep", _stream(), _p(down), _code(down, what), down.shape[1], q_rank, kv_off, kv_rank, rot_dim,
                  _p(q_norm_w), _p(kv_norm_w), float(eps), _p(cos), _p(sin), _p(ctx.positions), _p(ctx.tok_slot), _p(block_table),
-                 block_table.shape[1], _p(rows_cache), int(write_cache), _p(cq), n, _p(rows_t), _p(table_t))
+                 block_table.shape[1], _p(rows_cache), int(write_cache), _p(cq), n, _p(rows_t), _p(table_t), ROTARY_PAIRINGS[pairing])
     return cq
 
 
-def latent_query(q: torch.Tensor, uk: torch.Tensor, cos, sin, heads: int, dim: int, rot_dim: int, kv_rank: int) -> torch.Tensor:
-    """q [n, heads * (dim + rot_dim)], uk [heads * dim, kv_rank] -> float32 [n, heads, kv_rank + rot_dim]: each head's plain
-    part taken through its key matrix, its rotated part behind it."""
-    what = "latent_query"
-    _dev(what, q, uk, cos, sin)
-    n = q.shape[0]
-    _need(q.dim() == 2 and q.shape[1] == heads * (dim + rot_dim) and uk.shape == (heads * dim, kv_rank),
-          f"{what}: q {tuple(q.shape)}, key matrix {tuple(uk.shape)} for {heads} heads of {dim} + {rot_dim} and a latent of {kv_rank}")
+def _latent_rotation(what: str, cos, sin, n: int, rot_dim: int) -> None:
     if rot_dim:
+        _dev(what, cos, sin)
         for tab in (cos, sin):
             _need(tab is not None and tab.dtype == F32 and tab.shape == (n, rot_dim // 2), f"{what}: rotation rows are float32 [{n}, {rot_dim // 2}]")
+
+
+def _latent_rows(what: str, dtype, kv_rank: int, rot_dim: int, kv_norm_w, rows_cache, block_table, ctx, rows_t, table_t, pairing: str) -> None:
+    """The checks of whatever writes cache rows of latents."""
+    _dev(what, kv_norm_w, rows_cache, block_table, ctx.positions, ctx.tok_slot, rows_t, table_t)
+    _i32(what, block_table, ctx.positions, ctx.tok_slot, table_t)
+    _need(pairing in ROTARY_PAIRINGS, f"{what}: pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
+    _need(rows_t is None or (table_t is not None and rows_t.dtype == BF16 and rows_t.dim() == 3 and rows_t.shape[1:] == (kv_rank, PAGE_TOKENS)
+                             and table_t.shape == block_table.shape),
+          f"{what}: the transposed copy is bfloat16 [pages, {kv_rank}, {PAGE_TOKENS}] with a page table like the rows'")
+    _need(kv_norm_w.shape == (kv_rank,) and kv_norm_w.dtype == F32, f"{what}: the latent norm's weight is float32 [{kv_rank}]")
+    _need(rows_cache.dim() == 3 and rows_cache.shape[1:] == (PAGE_TOKENS, kv_rank + rot_dim) and rows_cache.dtype == dtype,
+          f"{what}: the cache {tuple(rows_cache.shape)} {rows_cache.dtype} is not {dtype} [pages, {PAGE_TOKENS}, {kv_rank + rot_dim}]")
+    _need(block_table.dim() == 2, f"{what}: page table {tuple(block_table.shape)} is not [slots, pages]")
+
+
+@dataclass
+class LatentStore:
+    """What ``latent_query`` writes to the cache beside its queries: ``src`` [n, >= kv_rank + rot_dim] (a view of wider rows is fine)
+    holds each token's latent and behind it the key part to rotate; the norm's weight and eps, and where the rows go."""
+    src: torch.Tensor
+    norm_w: torch.Tensor
+    eps: float
+    rows_cache: torch.Tensor
+    block_table: torch.Tensor
+    rows_t: torch.Tensor | None = None
+    table_t: torch.Tensor | None = None
+
+
+def latent_query(q: torch.Tensor, uk: torch.Tensor, cos, sin, heads: int, dim: int, rot_dim: int, kv_rank: int,
+                 pairing: str = "half_split", ctx=None, store: LatentStore | None = None) -> torch.Tensor:
+    """q [n, heads * (dim + rot_dim)] (a view of wider rows is fine), uk [heads * dim, kv_rank] -> float32 [n, heads, kv_rank +
+    rot_dim]: each head's plain part taken through its key matrix, its rotated part behind it (``pairing``: dimension i with i +
+    rot_dim/2, or 2i with 2i + 1).  ``store``: the same launch norms and rotates what the step's tokens keep and writes it."""
+    what = "latent_query"
+    _dev(what, uk)
+    n = q.shape[0]
+    _need(q.is_cuda and q.dim() == 2 and q.shape[1] == heads * (dim + rot_dim) and (n == 0 or q.stride(1) == 1) and uk.shape == (heads * dim, kv_rank),
+          f"{what}: q {tuple(q.shape)}, key matrix {tuple(uk.shape)} for {heads} heads of {dim} + {rot_dim} and a latent of {kv_rank}")
+    _need(pairing in ROTARY_PAIRINGS, f"{what}: pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
+    _latent_rotation(what, cos, sin, n, rot_dim)
+    keep = [None, 0, None, 0.0, None, None, None, 0, None, None, None]
+    if store is not None:
+        src = store.src
+        _latent_rows(what, q.dtype, kv_rank, rot_dim, store.norm_w, store.rows_cache, store.block_table, ctx, store.rows_t, store.table_t, pairing)
+        _need(src.is_cuda and src.dtype == q.dtype and src.dim() == 2 and src.shape[0] == n == ctx.n_tokens and src.shape[1] >= kv_rank + rot_dim
+              and (n == 0 or src.stride(1) == 1), f"{what}: latents {tuple(src.shape)} {src.dtype} for {ctx.n_tokens} tokens")
+        keep = [_p(src), src.stride(0), _p(store.norm_w), float(store.eps), _p(ctx.positions), _p(ctx.tok_slot), _p(store.block_table),
+                store.block_table.shape[1], _p(store.rows_cache), _p(store.rows_t), _p(store.table_t)]
     qa = torch.empty((n, heads, kv_rank + rot_dim), dtype=F32, device=q.device)
-    library.call(mixers(), "palm_latent_query", _stream(), _p(q), _code(q, what), _p(uk), _code(uk, what + " key matrix"), _p(cos), _p(sin),
-                 n, heads, dim, rot_dim, kv_rank, _p(qa))
+    library.call(mixers(), "palm_latent_query", _stream(), _p(q), _code(q, what), q.stride(0), _p(uk), _code(uk, what + " key matrix"), _p(cos), _p(sin),
+                 n, heads, dim, rot_dim, kv_rank, ROTARY_PAIRINGS[pairing], _p(qa), *keep)
     return qa
 
 
 _LATENT_MFMA_SIGNATURE = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                          c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p]
+                          c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p]
+_LATENT_DECODE_SIGNATURE = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                            c_float, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p]
 _latent_libs: dict = {}
 LATENT_MFMA_MAX_ROW, LATENT_MFMA_MAX_RANK = 640, 512
 
@@ -1409,6 +1449,7 @@ def latent_attention_lib(kv_rank: int, rot_dim: int):
     if key not in _latent_libs:
         lib = library.load(f"latent_attention_k{key[0]}_v{key[1]}")
         lib.palm_latent_attention_mfma.argtypes, lib.palm_latent_attention_mfma.restype = _LATENT_MFMA_SIGNATURE, c_int
+        lib.palm_latent_attention_decode.argtypes, lib.palm_latent_attention_decode.restype = _LATENT_DECODE_SIGNATURE, c_int
         lib.palm_latent_attention_mfma_sizes.argtypes, lib.palm_latent_attention_mfma_sizes.restype = [c_int], c_int
         if tuple(lib.palm_latent_attention_mfma_sizes(i) for i in range(2)) != (key[0] * 32, key[1] * 16):
             raise KernelError(f"library latent_attention_k{key[0]}_v{key[1]} was built for other sizes")
@@ -1418,10 +1459,10 @@ def latent_attention_lib(kv_rank: int, rot_dim: int):
 
 def latent_attention(qa: torch.Tensor, rows_cache: torch.Tensor, block_table: torch.Tensor, ctx, heads: int, kv_rank: int,
                      rot_dim: int, scale: float, window: int | None, rows_t: torch.Tensor | None = None,
-                     table_t: torch.Tensor | None = None) -> torch.Tensor:
+                     table_t: torch.Tensor | None = None, sink: torch.Tensor | None = None) -> torch.Tensor:
     """Softmax attention of the step's queries (float32 [n, heads, kv_rank + rot_dim]) over the cached rows of their own
     sequences up to their own positions (the last ``window`` of them if set): float32 [n, heads, kv_rank], the weighted sums
-    of the rows' latents.  Prompts (and portions of them) in bfloat16 go to the matrix cores if the caller keeps the
+    of the rows' latents.  ``sink`` float32 [heads]: head h's denominator has one more term exp(sink[h]).  Prompts (and portions of them) in bfloat16 go to the matrix cores if the caller keeps the
     transposed copy of the latents (``rows_t`` [pages, kv_rank, PAGE_TOKENS] with its page table); single tokens, the
     float32 mode and sizes that kernel does not take go to the exact kernel."""
     what = "latent_attention"
@@ -1432,6 +1473,7 @@ def latent_attention(qa: torch.Tensor, rows_cache: torch.Tensor, block_table: to
     _need(rows_cache.dim() == 3 and rows_cache.shape[1:] == (PAGE_TOKENS, kv_rank + rot_dim),
           f"{what}: the cache {tuple(rows_cache.shape)} is not [pages, {PAGE_TOKENS}, {kv_rank + rot_dim}]")
     _need(block_table.dim() == 2, f"{what}: page table {tuple(block_table.shape)} is not [slots, pages]")
+    _latent_sink(what, sink, heads)
     out = torch.empty((n, heads, kv_rank), dtype=F32, device=qa.device)
     if rows_t is not None and not ctx.is_decode and latent_mfma_serves(rows_cache, kv_rank, rot_dim):
         _need(table_t is not None and rows_t.dtype == BF16 and rows_t.dim() == 3 and rows_t.shape[1:] == (kv_rank, PAGE_TOKENS)
@@ -1439,11 +1481,63 @@ def latent_attention(qa: torch.Tensor, rows_cache: torch.Tensor, block_table: to
               "table like the rows'")
         library.call(latent_attention_lib(kv_rank, rot_dim), "palm_latent_attention_mfma", _stream(), _p(qa), _p(rows_cache), _p(rows_t),
                      _p(block_table), _p(table_t), block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new),
-                     ctx.n_seqs, int(ctx.max_new), heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(out), None, None, 0, 0, None)
+                     ctx.n_seqs, int(ctx.max_new), heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(sink), _p(out), None, None, 0, 0, None)
         return out
     library.call(mixers(), "palm_latent_attention", _stream(), _p(qa), _p(rows_cache), _code(rows_cache, what), _p(block_table),
                  block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs, int(ctx.max_new),
-                 heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(out))
+                 heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(sink), _p(out))
+    return out
+
+
+def _latent_sink(what: str, sink, heads: int) -> None:
+    if sink is not None:
+        _dev(what, sink)
+        _need(sink.shape == (heads,) and sink.dtype == F32, f"{what}: learned sink scores are float32 [{heads}], not {sink.dtype} {tuple(sink.shape)}")
+
+
+LATENT_BLOCKS_WANTED = 512         # a decode step's key ranges are cut into slices until about this many blocks run
+LATENT_MAX_SLICES = 256
+
+
+def latent_slices(ctx, heads: int, window: int | None) -> int:
+    """Into how many slices a decode step's key ranges are cut."""
+    keys = min(ctx.max_total, window) if window else ctx.max_total
+    pages = -(-keys // PAGE_TOKENS) + (1 if window else 0)
+    blocks = ctx.n_seqs * -(-heads // 16)
+    return max(1, min(pages, LATENT_MAX_SLICES, LATENT_BLOCKS_WANTED // max(1, blocks)))
+
+
+def latent_decode_serves(rows_cache: torch.Tensor, rows_t, uv: torch.Tensor, ctx, kv_rank: int, rot_dim: int) -> bool:
+    """Whether the matrix cores take a step of single tokens: the transposed copy of the latents at hand, bfloat16 value matrices."""
+    return rows_t is not None and ctx.is_decode and uv.dtype == BF16 and latent_mfma_serves(rows_cache, kv_rank, rot_dim)
+
+
+def latent_attention_decode(qa: torch.Tensor, rows_cache: torch.Tensor, block_table: torch.Tensor, ctx, heads: int, kv_rank: int,
+                            rot_dim: int, scale: float, window: int | None, rows_t: torch.Tensor, table_t: torch.Tensor, uv: torch.Tensor,
+                            gate: torch.Tensor | None, vdim: int, sink: torch.Tensor | None = None, slices: int | None = None) -> torch.Tensor:
+    """``latent_attention`` and ``latent_output`` for a step of single tokens on the matrix cores, the key range of every sequence
+    cut into slices that run side by side: bfloat16 [n, heads * vdim]."""
+    what = "latent_attention_decode"
+    _dev(what, qa, rows_cache, block_table, ctx.seq_slot, ctx.seq_start, rows_t, table_t, uv)
+    _i32(what, block_table, ctx.seq_slot, ctx.seq_start, table_t)
+    n = qa.shape[0]
+    _need(latent_decode_serves(rows_cache, rows_t, uv, ctx, kv_rank, rot_dim), f"{what}: single tokens in bfloat16 with sizes the kernel takes")
+    _need(qa.shape == (n, heads, kv_rank + rot_dim) and qa.dtype == F32 and n == ctx.n_tokens == ctx.n_seqs, f"{what}: queries {tuple(qa.shape)} {qa.dtype}")
+    _need(rows_cache.dim() == 3 and rows_cache.shape[1:] == (PAGE_TOKENS, kv_rank + rot_dim) and rows_t.dtype == BF16 and rows_t.dim() == 3
+          and rows_t.shape[1:] == (kv_rank, PAGE_TOKENS) and block_table.dim() == 2 and table_t.shape == block_table.shape,
+          f"{what}: the cache {tuple(rows_cache.shape)}, its transposed copy {tuple(rows_t.shape)}, page tables {tuple(block_table.shape)}")
+    _need(uv.shape == (heads * vdim, kv_rank), f"{what}: value matrix {tuple(uv.shape)} for {heads} heads of {vdim} over a latent of {kv_rank}")
+    _need(gate is None or (gate.is_cuda and gate.shape == (n, heads) and gate.dtype == BF16 and (n == 0 or gate.stride(1) == 1)),
+          f"{what}: the gate is bfloat16 [{n}, {heads}] with contiguous rows")
+    _latent_sink(what, sink, heads)
+    slices = latent_slices(ctx, heads, window) if slices is None else int(slices)
+    work_ml = torch.empty((n * heads * slices * 2,), dtype=F32, device=qa.device)
+    work = torch.empty((n * heads * slices * kv_rank,), dtype=F32, device=qa.device)
+    out = torch.empty((n, heads * vdim), dtype=BF16, device=qa.device)
+    library.call(latent_attention_lib(kv_rank, rot_dim), "palm_latent_attention_decode", _stream(), _p(qa), _p(rows_cache), _p(rows_t),
+                 _p(block_table), _p(table_t), block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), n, heads, kv_rank, rot_dim,
+                 float(scale), int(window or 0), _p(sink), slices, _p(work_ml), _p(work), _p(uv), _p(gate),
+                 gate.stride(0) if gate is not None else 0, vdim, _p(out))
     return out
 
 
@@ -1455,7 +1549,7 @@ def latent_fused_serves(qa: torch.Tensor, rows_cache: torch.Tensor, rows_t, uv: 
 
 def latent_attention_fused(qa: torch.Tensor, rows_cache: torch.Tensor, block_table: torch.Tensor, ctx, heads: int, kv_rank: int,
                            rot_dim: int, scale: float, window: int | None, rows_t: torch.Tensor, table_t: torch.Tensor, uv: torch.Tensor,
-                           gate: torch.Tensor | None, vdim: int) -> torch.Tensor:
+                           gate: torch.Tensor | None, vdim: int, sink: torch.Tensor | None = None) -> torch.Tensor:
     """``latent_attention`` on the matrix cores and ``latent_output`` in one kernel: bfloat16 [n, heads * vdim]."""
     what = "latent_attention_fused"
     _dev(what, qa, rows_cache, block_table, ctx.seq_slot, ctx.seq_start, ctx.seq_new, ctx.cu_new, rows_t, table_t, uv)
@@ -1469,10 +1563,11 @@ def latent_attention_fused(qa: torch.Tensor, rows_cache: torch.Tensor, block_tab
     _need(uv.shape == (heads * vdim, kv_rank), f"{what}: value matrix {tuple(uv.shape)} for {heads} heads of {vdim} over a latent of {kv_rank}")
     _need(gate is None or (gate.is_cuda and gate.shape == (n, heads) and gate.dtype == BF16 and (n == 0 or gate.stride(1) == 1)),
           f"{what}: the gate is bfloat16 [{n}, {heads}] with contiguous rows")
+    _latent_sink(what, sink, heads)
     out = torch.empty((n, heads * vdim), dtype=BF16, device=qa.device)
     library.call(latent_attention_lib(kv_rank, rot_dim), "palm_latent_attention_mfma", _stream(), _p(qa), _p(rows_cache), _p(rows_t),
                  _p(block_table), _p(table_t), block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new),
-                 ctx.n_seqs, int(ctx.max_new), heads, kv_rank, rot_dim, float(scale), int(window or 0), None, _p(uv), _p(gate),
+                 ctx.n_seqs, int(ctx.max_new), heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(sink), None, _p(uv), _p(gate),
                  gate.stride(0) if gate is not None else 0, vdim, _p(out))
     return out
 
@@ -1508,13 +1603,15 @@ def moe_route(logits: torch.Tensor, top: int):
     return chosen, weight
 
 
-EXPERT_FORMS = {"gated_silu": 0, "gelu": 1, "capped_gated": 2}
+EXPERT_FORMS = {"gated_silu": 0, "gelu": 1, "capped_gated": 2, "relu_squared": 3}
+PLAIN_EXPERTS = {"gelu": "gelu_erf", "relu_squared": "relu_squared"}          # forms without a gate, and their activation's name
+MOE_ROW_VALUES = 16384             # inner values of a token's experts together that the kernels for few rows hold
 NO_CAP = (1.0, 1.0, 0.0)           # limit, slope, shift: what the other forms pass and do not read
 
 
 def expert_rows(form: str) -> int:
     """Rows of an expert's first matrix for each inner value: gated experts have a gate row and an up row."""
-    return 1 if form == "gelu" else 2
+    return 1 if form in PLAIN_EXPERTS else 2
 
 
 def _addends(what: str, add, h):
@@ -1585,23 +1682,49 @@ def activation(z: torch.Tensor, kind: str) -> torch.Tensor:
     return out
 
 
-def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, ff: int,
-                form: str = "gated_silu", cap=NO_CAP, add=()) -> torch.Tensor:
+def moe_route_table(ids: torch.Tensor, table: torch.Tensor):
+    """ids int32 [n], table int32 [vocab, top] -> (chosen int32 [n, top], weight float32 [n, top]): every token's row of the table,
+    and 1 / top for each choice.  (An id outside the table takes its nearest row: such a token's logits are no numbers anyway.)"""
+    _dev("moe_route_table", ids, table)
+    _i32("moe_route_table", ids, table)
+    _need(ids.dim() == 1 and table.dim() == 2, f"moe_route_table: ids {tuple(ids.shape)}, table {tuple(table.shape)}")
+    n, top = ids.shape[0], table.shape[1]
+    chosen = torch.empty((n, top), dtype=torch.int32, device=ids.device)
+    weight = torch.empty((n, top), dtype=F32, device=ids.device)
+    library.call(feedforward(), "palm_moe_route_table", _stream(), _p(ids), _p(table), table.shape[0], n, top, _p(chosen), _p(weight))
+    return chosen, weight
+
+
+def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor | None, ff: int,
+                form: str = "gated_silu", cap=NO_CAP, add=(), ids: torch.Tensor | None = None, shared=None) -> torch.Tensor:
     """Every row through its chosen experts, nothing planned on the host: h [n, width]; gate_up [experts * 2 ff, width] (an
-    expert's gate rows, then its up rows; ``form`` "gelu": [experts * ff, width], up rows alone, through the exact gelu; ``form``
+    expert's gate rows, then its up rows; ``form`` "gelu" and "relu_squared": [experts * ff, width], up rows alone; ``form``
     "capped_gated": gate and up rows, capped as ``cap`` = (limit, slope, shift) says); down [experts * width, ff].  Returns float32
-    [n, width], the weighted sum plus the rows ``add`` (up to two [n, width] of h's type that other branches made)."""
+    [n, width], the weighted sum plus the rows ``add`` (up to two [n, width] of h's type that other branches made).  ``ids`` int32
+    [n]: ``chosen`` is a table [vocab, top] of which each row takes the row of its token's id, and every choice weighs 1 / top
+    (``weight`` None).  ``shared`` (first matrix, down): one more expert of the same form, for every row, with weight one."""
     what = "moe_experts"
-    _dev(what, h, gate_up, down, chosen, weight)
-    _i32(what, chosen)
+    _dev(what, h, gate_up, down, chosen, weight, ids)
+    _i32(what, chosen, ids)
     n, width = h.shape
     top = chosen.shape[1]
     _expert_shapes(what, h, gate_up, down, ff, form)
-    _need(chosen.shape == (n, top) and weight.shape == (n, top) and weight.dtype == F32, f"{what}: choices {tuple(chosen.shape)}, weights {tuple(weight.shape)}")
-    mid = torch.empty((n, top, ff), dtype=F32, device=h.device)
+    if ids is None:
+        _need(chosen.shape == (n, top) and weight is not None and weight.shape == (n, top) and weight.dtype == F32,
+              f"{what}: choices {tuple(chosen.shape)}, weights {None if weight is None else tuple(weight.shape)}")
+    else:
+        _need(chosen.dim() == 2 and weight is None and ids.shape == (n,), f"{what}: a table of choices {tuple(chosen.shape)} with ids {tuple(ids.shape)} and no weights")
+    shared_up, shared_down = shared if shared is not None else (None, None)
+    shared_ff = shared_down.shape[1] if shared is not None else 0
+    if shared is not None:
+        _dev(what, shared_up, shared_down)
+        _need(shared_up.shape == (expert_rows(form) * shared_ff, width) and shared_down.shape == (width, shared_ff) and shared_up.dtype == gate_up.dtype
+              and shared_down.dtype == gate_up.dtype, f"{what}: the shared expert's matrices {tuple(shared_up.shape)}, {tuple(shared_down.shape)}")
+    mid = torch.empty((n, top * ff + shared_ff), dtype=F32, device=h.device)
     out = torch.empty((n, width), dtype=F32, device=h.device)
     library.call(feedforward(), "palm_moe_experts", _stream(), _p(h), _code(h, what), _p(gate_up), _p(down), _code(gate_up, what + " weights"),
-                 _p(chosen), _p(weight), n, top, width, ff, _p(mid), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h))
+                 _p(chosen), _p(weight), n, top, width, ff, _p(mid), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h),
+                 _p(ids), chosen.shape[0] if ids is not None else 0, _p(shared_up), _p(shared_down), shared_ff)
     return out
 
 
@@ -1660,9 +1783,6 @@ def scatter_add(out: torch.Tensor, y: torch.Tensor, rows: torch.Tensor, weight: 
 
 SINK_NORMS = {None: 0, "projection": 1, "head": 2, "head_unit": 2}       # (head_unit: per head, without a weight)
 SINK_BLOCKS_WANTED = 1024         # a decode step's key ranges are cut into slices until about this many blocks run
-
-
-ROTARY_PAIRINGS = {"half_split": 0, "interleaved": 1}
 
 
 def sink_qkv_store(rows: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, bias, norm: str | None, q_w, k_w, eps: float,

@@ -1,6 +1,6 @@
 """The arrangement of a layer's parts around the residual stream.
 
-``pre_norm``: x += mixer(norm(x)); x += feed_forward(norm(x)) (models/qwen3.py:254-287).  The residual
+``pre_norm``: x += mixer(norm(x)); x += feed_forward(norm(x)) (models/qwen3.py:254-287); a layer may have no feed-forward.  The residual
 stream x is float32.  A branch's output is never added by a kernel of its own: it goes into a
 ``ResidualSink`` (parts/residual.py), and either the norm that reads x next adds it in the pass in which it
 norms (the sum is made in 32-bit and written back to x), or the branch's last product does both.  So the
@@ -47,23 +47,29 @@ class PreNormBlock:
     def __init__(self, spec, builder):
         self.mixer_norm = builder.build(spec.parts["mixer_norm"])
         self.mixer = builder.build(spec.parts["mixer"])
-        self.feed_forward_norm = builder.build(spec.parts["feed_forward_norm"])
-        self.feed_forward = builder.build(spec.parts["feed_forward"])
+        self.feed_forward = builder.build(spec.parts["feed_forward"]) if "feed_forward" in spec.parts else None
+        self.feed_forward_norm = builder.build(spec.parts["feed_forward_norm"]) if self.feed_forward is not None else None
 
     @property
     def capturable(self) -> bool:
-        return all(getattr(p, "capturable", False) for p in (self.mixer_norm, self.mixer, self.feed_forward_norm,
-                                                              self.feed_forward))
+        parts = [self.mixer_norm, self.mixer] + ([self.feed_forward_norm, self.feed_forward] if self.feed_forward is not None else [])
+        return all(getattr(p, "capturable", False) for p in parts)
 
     @staticmethod
     def cache_needs(spec):
         return cache_needs(spec.parts["mixer"])
+
+    @staticmethod
+    def cache_needs_beside_shared(spec):
+        return cache_needs_beside_shared(spec.parts["mixer"])
 
     @property
     def entry_norm(self):
         return self.mixer_norm
 
     def forward(self, x, h, ctx, sink):
+        if self.feed_forward is None:
+            return run_branch(self.mixer, h, ctx, sink)
         h = run_branch(self.mixer, h, ctx, ResidualSink(x, self.feed_forward_norm))
         return run_branch(self.feed_forward, h, ctx, sink)
 

@@ -31,7 +31,12 @@ then hold gate rows before up rows, expert by expert), with ``limit`` and for th
 "softmax": the scores are the softmax over all experts' logits; ``group_score`` "largest": a group ranks by its largest score;
 ``shared_gate`` false: the shared expert's output is added as it is.  ``input`` "shared": the shared expert's first product and
 the router's are columns of wider products that the block makes for all its branches (``forward_rows``); rows that another
-branch of the block made can be added where the experts' weighted sum is written (``addend``)."""
+branch of the block made can be added where the experts' weighted sum is written (``addend``).
+
+``routed_table``: no router: the integer tensor ``table`` [vocab, top] gives every token id its experts (the entries of a row
+differ), and each weighs 1 / top.  Plain experts (``form`` "relu_squared": down(max(up(h), 0)^2), or "gelu").  With ``shared_size`` one more
+expert of the same form and of that inner size runs for every token and is added; in a step of few rows it runs in the
+experts' own kernels."""
 from __future__ import annotations
 
 import numpy as np
@@ -113,7 +118,7 @@ class DenseFeedForward:
 
 class RoutedExperts:
     """The experts of a routed feed-forward and how a step's rows go through them, whatever chose them.  ``form``:
-    "gated_silu" (an expert's first matrix holds its gate rows, then its up rows), "gelu" (up rows alone), or "capped_gated"
+    "gated_silu" (an expert's first matrix holds its gate rows, then its up rows), "gelu" or "relu_squared" (up rows alone), or "capped_gated"
     (gate rows and up rows, capped as ``cap`` = (limit, slope, shift) says)."""
     DIRECT_ROWS = 128            # as many rows as a recorded step holds at most
 
@@ -133,7 +138,7 @@ class RoutedExperts:
         if self.form == "gated_silu":
             return self.expert_first[e].gated(xs)
         z = self.expert_first[e](xs)
-        return ops.capped_gate(z, *self.cap) if self.form == "capped_gated" else ops.activation(z, "gelu_erf")
+        return ops.capped_gate(z, *self.cap) if self.form == "capped_gated" else ops.activation(z, ops.PLAIN_EXPERTS[self.form])
 
     def run_experts(self, h, chosen, weight, add=()):
         """float32 [n, hidden]: sum_c weight[t, c] * expert chosen[t, c] of h[t], plus the rows ``add`` (up to two)."""
@@ -253,3 +258,46 @@ class RoutedScoredFeedForward(RoutedExperts):
         if self.shared_gate:
             ops.add_gated_rows(out, y, logits, self.experts)
         return out
+
+
+@register_part("feed_forward", "routed_table")
+class RoutedTableFeedForward(RoutedExperts):
+    capturable = True
+    SHARED_DIRECT_ROWS = 16      # as many rows share the shared expert's weights well enough when each reads them for itself
+
+    def __init__(self, spec, builder):
+        p = spec.params
+        W, E = int(p["hidden_size"]), int(p["num_experts"])
+        self.top = int(p["top"])
+        form = str(p.get("form", "relu_squared"))
+        if form not in ops.PLAIN_EXPERTS:
+            raise ValueError(f"routed feed-forward: form {form!r} is not one of {sorted(ops.PLAIN_EXPERTS)}")
+        self.table = builder.tensor(spec, "table")
+        if self.table.shape != (int(p["vocab_size"]), self.top) or not 1 <= self.top <= E:
+            raise ValueError(f"routed feed-forward: the table {tuple(self.table.shape)} is not [{p['vocab_size']}, {self.top}] over {E} experts")
+        # the kernels take the entries as they are
+        low, high = int(self.table.min()), int(self.table.max())
+        if low < 0 or high >= E:
+            raise ValueError(f"routed feed-forward: the table names expert {low if low < 0 else high}; there are {E}")
+        self._set_experts(builder.tensor(spec, "up"), builder.tensor(spec, "down"), E, int(p["intermediate_size"]), W, form)
+        self.shared = None
+        if p.get("shared_size"):
+            self.shared = (Linear(builder.tensor(spec, "shared_up")), Linear(builder.tensor(spec, "shared_down")))
+            shapes = tuple(tuple(s.weight.shape) for s in self.shared)
+            if shapes != ((int(p["shared_size"]), W), (W, int(p["shared_size"]))):
+                raise ValueError(f"routed feed-forward: the shared expert's weights {shapes} do not fit inner size {p['shared_size']} over hidden {W}")
+            self.shared_fits = (all(s.weight.dtype == self.first.dtype for s in self.shared)
+                                and self.top * self.inter + int(p["shared_size"]) <= ops.MOE_ROW_VALUES)
+
+    def forward(self, h, ctx):
+        h = as_tensor(h)
+        direct = self.shared is not None and h.shape[0] <= self.SHARED_DIRECT_ROWS and self.shared_fits
+        add = []
+        if self.shared is not None and not direct:
+            up, down = self.shared
+            add.append(down(ops.activation(up(h), ops.PLAIN_EXPERTS[self.form])))
+        if h.shape[0] <= self.DIRECT_ROWS:
+            return ops.moe_experts(h, self.first, self.down_all, self.table, None, self.inter, self.form, add=add, ids=ctx.token_ids,
+                                   shared=tuple(s.weight for s in self.shared) if direct else None)
+        chosen, weight = ops.moe_route_table(ctx.token_ids, self.table)
+        return self.run_experts(h, chosen, weight, add)

@@ -21,6 +21,7 @@ import torch
 
 from ..config.spec import ModelSpec, TensorRef
 from ..kernels import ops
+from .random_init import random_integers
 from .random_numbers import tensor_key
 from .safetensors_io import ModelFiles
 
@@ -165,9 +166,11 @@ def random_weights(spec: ModelSpec, seed: int, mode: torch.dtype, device) -> Wei
         dst = torch.zeros(ref.shape, dtype=dt, device=device)
         row = 0
         for name, shape, how in ref.pieces():
-            if ref.role != "integer":
+            part = dst[row:row + shape[0]] if shape else dst
+            if ref.role == "integer":
+                part.copy_(_taken(random_integers(ref.init, tensor_key(seed, name), how.shape if how is not None else shape), how))
+            else:
                 _, mean, std = ref.init
-                part = dst[row:row + shape[0]] if shape else dst
                 if how is None and dt == torch.bfloat16:
                     ops.random_fill(part, tensor_key(seed, name), mean, std)
                 else:

@@ -15,10 +15,18 @@ from pathlib import Path
 import torch
 
 from ..config.registry import config_from_dict, config_source
-from .random_numbers import normal, tensor_key
+from .random_numbers import distinct_rows, normal, tensor_key
 from .safetensors_io import write_safetensors
 
 _STORE = {"bfloat16": torch.bfloat16, "float32": torch.float32, "float16": torch.float16}
+
+
+def random_integers(init: tuple, key: int, shape) -> torch.Tensor:
+    """An integer table [rows, count] as its description says: ("distinct", n) fills every row with different integers below n,
+    anything else with zeros."""
+    if init[0] != "distinct":
+        return torch.zeros(shape, dtype=torch.int32)
+    return torch.from_numpy(distinct_rows(key, int(shape[0]), int(shape[1]), int(init[1])))
 
 
 def random_tensors(spec, seed: int, dtype: str = "bfloat16") -> dict[str, torch.Tensor]:
@@ -30,7 +38,7 @@ def random_tensors(spec, seed: int, dtype: str = "bfloat16") -> dict[str, torch.
             if name in out:
                 continue
             if ref.role == "integer":
-                out[name] = torch.zeros(shape, dtype=torch.int32)
+                out[name] = random_integers(ref.init, tensor_key(seed, name), shape)
                 continue
             _, mean, std = ref.init
             count = 1

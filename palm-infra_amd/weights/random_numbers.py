@@ -86,6 +86,23 @@ def standard_normal(key: int, first: int, count: int) -> np.ndarray:
     return (r * c).astype(np.float32)
 
 
+def distinct_rows(key: int, rows: int, count: int, n: int) -> np.ndarray:
+    """int32 [rows, count]: every row holds ``count`` different integers of 0 .. n - 1, a function of (key, row) alone (draw c
+    takes one of the n - c numbers that the row does not hold yet)."""
+    if not 1 <= count <= n:
+        raise ValueError(f"{count} different integers of {n}")
+    with np.errstate(over="ignore"):
+        i = np.arange(1, rows * count + 1, dtype=np.uint64)
+        draws = (_mix64(np.uint64(key) + i * _GOLDEN) >> np.uint64(33)).reshape(rows, count)
+    out = np.empty((rows, count), dtype=np.int64)
+    for c in range(count):
+        k = (draws[:, c] % np.uint64(n - c)).astype(np.int64)
+        for held in np.sort(out[:, :c], axis=1).T:               # the k-th number that is not held, counted past those below it
+            k += k >= held
+        out[:, c] = k
+    return out.astype(np.int32)
+
+
 def normal(key: int, count: int, mean: float, std: float, chunk: int = 1 << 18) -> np.ndarray:
     """``count`` float32 values ``z * std + mean`` (a rounded product, then a rounded sum).  Made in pieces that stay
     in the processor's caches (some ten million values a second)."""
