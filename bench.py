@@ -368,6 +368,23 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
             if f and "palm_moe_experts" not in out:
                 amount = 2.0 * f["router"]["top"] * 3 * f["expert"]["ff"] * raw["width"]
                 out["palm_moe_experts"], out["palm_moe_grouped"] = (None, None, batch * amount, hbm), (tokens * amount, mfma, None, None)
+    elif raw.get("architecture") == "Nirotar":
+        for layer in raw["layers"]:
+            m, f = layer["mixer"], layer.get("mlp")
+            w = m["mask"]["size"] if m.get("mask") else max(tokens, context + 1)
+            seen = sum(min(p + 1, w) for p in range(tokens))
+            if layer["type"] == "attention":
+                out["palm_sink_attention_mfma"] = (2.0 * m["heads"] * (m["dim"] + m["vdim"]) * seen, mfma, None, None)
+                out["palm_sink_attention"] = (None, None, 2.0 * batch * min(context, w) * m["kv_heads"] * (m["dim"] + m["vdim"]), hbm)
+            else:
+                row = m["kv_rank"] + m["rot_dim"]
+                out["palm_latent_attention_mfma"] = (2.0 * m["heads"] * ((row + m["kv_rank"]) * seen + tokens * m["kv_rank"] * m["vdim"]), mfma, None, None)
+                # a decode step reads the rows of the sequences and (it applies them) the value matrices once
+                out["palm_latent_attention_decode"] = (None, None, 2.0 * (batch * min(context, w) * row + m["heads"] * m["vdim"] * m["kv_rank"]), hbm)
+            if f:                                                          # plain experts: two matrices each; a decode step's launch has the shared one too
+                amount = 2.0 * f["router"]["top"] * 2 * f["expert"]["ff"] * raw["width"]
+                shared = 2.0 * 2 * f["shared"]["ff"] * raw["width"] if f.get("shared") else 0.0
+                out["palm_moe_experts"], out["palm_moe_grouped"] = (None, None, batch * amount + shared, hbm), (tokens * amount, mfma, None, None)
     elif "layers" in raw:
         for layer in raw["layers"]:
             m = layer["mixer"]
@@ -391,6 +408,7 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
                 row = m["kv_rank"] + m["rot_dim"]
                 flops = 2.0 * m["heads"] * (row + m["kv_rank"]) * seen
                 out["palm_latent_attention"] = (flops, mfma, 2.0 * batch * min(context, w) * row, hbm)
+                out["palm_latent_attention_decode"] = (None, None, 2.0 * (batch * min(context, w) * row + m["heads"] * m["vdim"] * m["kv_rank"]), hbm)
                 # the prompt kernel also applies the value matrices
                 out["palm_latent_attention_mfma"] = (flops + 2.0 * tokens * m["heads"] * m["kv_rank"] * m["vdim"], mfma, None, None)
             elif layer["type"] == "parallel" and "palm_sink_attention" not in out:
@@ -512,7 +530,18 @@ def _vovalix_bench(args, record) -> dict:
     return record["sizes"]["vovalix-2048"]["vovalix"]
 
 
-DESIGNS = {"vovalix": ("Vovalix presets beside Biguzen and Pazilorn presets of equal width and depth", _vovalix_bench),
+def _nirotar_bench(args, record) -> dict:
+    """The Nirotar presets beside the Biguzen and the Pazilorn presets of the same width and depth (the closest designs here:
+    Biguzen has the same windowed attention with learned sinks and plain experts with a shared one, Pazilorn the attention over
+    compressed rows)."""
+    for width in ("2048", "4096"):
+        record["sizes"][f"nirotar-{width}"] = {
+            name: design_points(preset_dict(f"{name}-{width}"), args, PREFILL_TOKENS, BATCH, CONTEXT) for name in ("nirotar", "biguzen", "pazilorn")}
+    return record["sizes"]["nirotar-2048"]["nirotar"]
+
+
+DESIGNS = {"nirotar": ("Nirotar presets beside Biguzen and Pazilorn presets of equal width and depth", _nirotar_bench),
+           "vovalix": ("Vovalix presets beside Biguzen and Pazilorn presets of equal width and depth", _vovalix_bench),
            "biguzen": ("Biguzen presets beside Matalix presets of equal width and depth", _biguzen_bench),
            "matalix": ("Matalix presets beside Sebesun presets of equal width and depth", _matalix_bench),
            "sebesun": ("Sebesun presets beside Qwen3 models of equal width and depth", _sebesun_bench),
