@@ -27,6 +27,7 @@
 //
 // Blocks are numbered so that the 32 blocks that run on one die at a time (blocks go to the eight dies in turn)
 // work on neighbouring tiles: each die's L2 then holds few weight and activation tiles for many blocks.
+#include "lds_stage.h"
 #include "mfma.h"
 
 #ifdef PALM_TILE_STANDALONE
@@ -44,16 +45,6 @@ constexpr int LDS_BYTES = 160 * 1024;
 constexpr int TILE_WAVES = 8;
 constexpr int TILE_THREADS = TILE_WAVES * WAVE;
 constexpr int DIES = 8;
-
-__device__ __forceinline__ void row_chunk_into_lds(const void* from, uint32_t lds_base) {
-    asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" : : "v"(from), "s"(lds_base) : "m0", "memory");
-}
-// s_waitcnt vmcnt(N): loads come back in order, so "all but the N youngest" is a stage's rows with the later stages'
-// still on their way.  (vmcnt is six bits: the low four in bits 0..3, the high two in bits 14..15.)
-template <int N> __device__ __forceinline__ void all_but_the_youngest_have_arrived() {
-    static_assert(N >= 0 && N < 64, "vmcnt has six bits");
-    __builtin_amdgcn_s_waitcnt(0x0F70 | (N & 15) | ((N >> 4) << 14));
-}
 
 template <int TOK, int FEAT, int WAVES_F, typename TC>
 __global__ __launch_bounds__(TILE_THREADS) void linear_tile_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,

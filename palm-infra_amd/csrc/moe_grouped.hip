@@ -1,19 +1,21 @@
 // Routed experts for many rows (a prompt), planned on the device: the (token, choice) pairs are grouped by expert, and two
 // grouped products on the matrix cores run all experts' rows in one launch each.
 //
-//   plan      count the pairs of every expert; pad every expert's run of pairs to whole tiles of GT_TOKENS rows and lay the
+//   plan      count the pairs of every expert; pad every expert's run of pairs to whole tiles of rows and lay the
 //             runs one after the other; place every pair in its run in the order of the pairs (token, then choice), so that
 //             nothing depends on the order in which threads arrive; the slots that pad a run hold -1
 //   grouped   for every tile (its expert comes from the plan): mid = silu(G_e x) * (U_e x) for the tile's rows x, then
 //             y = D_e mid.  The weights are the first operand of the matrix instruction, so that a lane ends with four
-//             neighbouring features of one row; a wave owns 32 features x 64 rows and reads its fragments from memory itself
-//             (a weight fragment feeds four products, a row fragment two or four)
+//             neighbouring features of one row.  Sizes in whole cache lines with enough rows an expert: blocks of 128 rows x 256
+//             features through a ring of stages in LDS (moe_tile_kernel).  Otherwise a wave owns 32 features x 64 rows and reads its
+//             fragments from memory itself (a weight fragment feeds four products, a row fragment two or four)
 //   combine   out[t] = sum_c weight[t, c] * y[place of pair (t, c)], in the order of c, 32-bit, plus up to two rows that other
 //             branches made
 #include "mfma.h"
 #include "expert_form.h"
+#include "lds_stage.h"
 
-constexpr int GT_TOKENS = 64;                     // rows of a tile
+constexpr int GT_TOKENS = 64;                     // rows of a tile whose fragments come from memory
 constexpr int GT_RUNS = GT_TOKENS / 16;           // runs of 16 rows: what one matrix instruction takes
 constexpr int GT_WAVES = 4;
 constexpr int GT_FEATURES = 32 * GT_WAVES;        // features of a block's tile
@@ -45,13 +47,13 @@ __global__ __launch_bounds__(PLAN_THREADS) void moe_count_kernel(const int* __re
 
 // One block: starts[e] = first slot of expert e's run (runs padded to whole tiles), starts[experts] = slots in all;
 // tile_expert[i] = the expert of tile i, -1 beyond the last tile.
-__global__ __launch_bounds__(PLAN_THREADS) void moe_runs_kernel(const int* __restrict__ counts, int experts, int max_tiles,
+__global__ __launch_bounds__(PLAN_THREADS) void moe_runs_kernel(const int* __restrict__ counts, int experts, int max_tiles, int tile,
                                                                 int* __restrict__ starts, int* __restrict__ tile_expert) {
     if (threadIdx.x == 0) {
         int at = 0;
         for (int e = 0; e < experts; ++e) {
             starts[e] = at;
-            at += (counts[e] + GT_TOKENS - 1) / GT_TOKENS * GT_TOKENS;
+            at += (counts[e] + tile - 1) / tile * tile;
         }
         starts[experts] = at;
     }
@@ -59,7 +61,7 @@ __global__ __launch_bounds__(PLAN_THREADS) void moe_runs_kernel(const int* __res
     for (int i = threadIdx.x; i < max_tiles; i += PLAN_THREADS) tile_expert[i] = -1;
     __syncthreads();
     for (int e = threadIdx.x; e < experts; e += PLAN_THREADS)
-        for (int i = starts[e] / GT_TOKENS; i < starts[e + 1] / GT_TOKENS; ++i) tile_expert[i] = e;
+        for (int i = starts[e] / tile; i < starts[e + 1] / tile; ++i) tile_expert[i] = e;
 }
 
 // One block per expert: its pairs into its run, in the order of the pairs.  slot_pair[slot] = pair (or -1), pair_slot[pair] = slot.
@@ -172,6 +174,140 @@ __global__ __launch_bounds__(GT_WAVES * WAVE) void moe_grouped_kernel(const bf16
         }
 }
 
+// The same products with both operands crossing LDS.  A block of eight waves owns TILE_ROWS slots x TILE_W_ROWS rows of an
+// expert's matrix and walks over K in stages of 64 (a row of a stage is one cache line of 128 bytes), the stages in a ring
+// that global_load_lds fills; a row's eight 16-byte chunks are permuted by the row's number so that an operand's reads spread
+// over the banks (the lane that fills a place fetches the chunk that belongs there).  MFMA 32x32x16: 32 weight rows x 32 slots, a wave
+// owns 64 weight rows x 64 slots.  Gated forms: of every 64 weight rows of a tile the first 32 are gate rows and the others
+// their up rows.  FORM as above.  The tiles of an expert that lies in the plan follow each other, features innermost, and each
+// die gets a run of neighbouring tiles.
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+constexpr int TILE_ROWS = 128, TILE_W_ROWS = 256, TILE_K = 64, TILE_WAVES = 8, TILE_WAVES_F = 4;
+constexpr int TILE_LINE = TILE_K * 2, TILE_CHUNKS = TILE_LINE / 16, TILE_RING = 3;
+constexpr int TILE_STAGE = (TILE_ROWS + TILE_W_ROWS) * TILE_LINE;
+constexpr int TILE_LOADS = TILE_STAGE / 1024 / TILE_WAVES;            // instructions a wave and stage
+constexpr int TILE_DIES = 8;
+
+template <int FORM>
+__global__ __launch_bounds__(TILE_WAVES * WAVE) void moe_tile_kernel(const bf16_t* __restrict__ a, const int* __restrict__ slot_pair, int top,
+                                                                     const bf16_t* __restrict__ w, const int* __restrict__ tile_expert,
+                                                                     int max_tiles, int feature_tiles, int n_features, int k_dim,
+                                                                     ExpertCap cap, bf16_t* __restrict__ out) {
+    constexpr bool GATED = FORM == 1 || FORM == 3;
+    constexpr int TILE_FEATURES = GATED ? TILE_W_ROWS / 2 : TILE_W_ROWS;
+    __shared__ __attribute__((aligned(1024))) char lds[TILE_RING * TILE_STAGE];
+    const int total = max_tiles * feature_tiles, per_die = (total + TILE_DIES - 1) / TILE_DIES;
+    const int pid = (blockIdx.x % TILE_DIES) * per_die + blockIdx.x / TILE_DIES;
+    if (pid >= total) return;
+    const int tile = pid / feature_tiles, f0 = pid % feature_tiles * TILE_FEATURES;
+    const int e = tile_expert[tile];
+    if (e < 0) return;
+    const int lane = threadIdx.x % WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+    const int wave_f = wave % TILE_WAVES_F, wave_t = wave / TILE_WAVES_F;
+    const bf16_t* we = w + (size_t)e * (GATED ? 2 : 1) * n_features * k_dim;
+
+    // the rows this lane brings in: instruction q of this wave fills the stage's rows (q * 8 + wave) * 8 .. + 7, weights first
+    const char* src[TILE_LOADS];
+#pragma unroll
+    for (int q = 0; q < TILE_LOADS; ++q) {
+        const int R = (q * TILE_WAVES + wave) * 8 + lane / TILE_CHUNKS;
+        const int chunk = (lane % TILE_CHUNKS) ^ ((R >> 1) & (TILE_CHUNKS - 1));
+        const bf16_t* row;
+        if (R < TILE_W_ROWS) {
+            const int f = GATED ? f0 + R / 64 * 32 + R % 32 : f0 + R;
+            row = we + ((size_t)min(f, n_features - 1) + (GATED && R / 32 % 2 ? n_features : 0)) * k_dim;
+        } else {
+            const int slot = tile * TILE_ROWS + R - TILE_W_ROWS;
+            // a slot that pads the run reads row 0; nobody reads its result
+            row = a + (size_t)(slot_pair ? max(slot_pair[slot], 0) / top : slot) * k_dim;
+        }
+        src[q] = reinterpret_cast<const char*>(row) + chunk * 16;
+    }
+    const uint32_t lds0 = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)lds);
+    auto bring = [&](int kt, int place) {
+#pragma unroll
+        for (int q = 0; q < TILE_LOADS; ++q)
+            row_chunk_into_lds(src[q] + (size_t)kt * TILE_LINE, lds0 + place * TILE_STAGE + (q * TILE_WAVES + wave) * 1024);
+    };
+    int w_off[2], x_off[2], cs[TILE_K / 16];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        w_off[i] = (wave_f * 64 + i * 32 + lane % 32) * TILE_LINE;
+        x_off[i] = (TILE_W_ROWS + wave_t * 64 + i * 32 + lane % 32) * TILE_LINE;
+    }
+#pragma unroll
+    for (int s = 0; s < TILE_K / 16; ++s) cs[s] = ((2 * s + lane / 32) ^ ((lane >> 1) & (TILE_CHUNKS - 1))) * 16;
+    f32x16 acc[2][2];
+#pragma unroll
+    for (int f = 0; f < 2; ++f)
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int v = 0; v < 16; ++v) acc[f][t][v] = 0.f;
+
+    const int stages = k_dim / TILE_K;
+    constexpr int AHEAD = TILE_RING - 1;
+#pragma unroll
+    for (int i = 0; i < AHEAD; ++i)
+        if (i < stages) bring(i, i);
+    int place = 0;
+    for (int kt = 0; kt < stages; ++kt) {
+        if (kt + AHEAD <= stages) all_but_the_youngest_have_arrived<(AHEAD - 1) * TILE_LOADS>();
+        else all_but_the_youngest_have_arrived<0>();
+        __syncthreads();                                       // every wave's share of the stage; and everyone is done with the one before
+        if (kt + AHEAD < stages) bring(kt + AHEAD, place == 0 ? TILE_RING - 1 : place - 1);
+        const char* stage = lds + place * TILE_STAGE;
+        bf16x8 wf[2][2], xf[2][2];
+        auto read_operands = [&](int s) {
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                wf[s & 1][i] = *reinterpret_cast<const bf16x8*>(stage + w_off[i] + cs[s]);
+                xf[s & 1][i] = *reinterpret_cast<const bf16x8*>(stage + x_off[i] + cs[s]);
+            }
+        };
+        read_operands(0);
+#pragma unroll
+        for (int s = 0; s < TILE_K / 16; ++s) {
+            if (s + 1 < TILE_K / 16) read_operands(s + 1);
+#pragma unroll
+            for (int f = 0; f < 2; ++f)
+#pragma unroll
+                for (int t = 0; t < 2; ++t)
+                    acc[f][t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[s & 1][f], xf[s & 1][t], acc[f][t], 0, 0, 0);
+            if (s + 1 < TILE_K / 16) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);      // one matrix instruction
+                    __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);      // one LDS read
+                }
+            }
+        }
+        place = place + 1 == TILE_RING ? 0 : place + 1;
+    }
+
+    // element v of a result tile: slot lane % 32, weight row 8 (v / 4) + 4 (lane / 32) + v % 4
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        const size_t slot = (size_t)tile * TILE_ROWS + wave_t * 64 + t * 32 + lane % 32;
+#pragma unroll
+        for (int f = 0; f < (GATED ? 1 : 2); ++f)
+#pragma unroll
+            for (int q4 = 0; q4 < 4; ++q4) {
+                const int feat = f0 + (GATED ? wave_f * 32 : wave_f * 64 + f * 32) + 8 * q4 + 4 * (lane / 32);
+                if (feat >= n_features) continue;              // n_features is a multiple of four
+                bf16_t v[4];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float z = acc[f][t][4 * q4 + i];
+                    v[i] = f32_to_bf16(FORM == 1 ? expert_silu_gated(z, acc[1][t][4 * q4 + i]) : FORM == 3 ? expert_capped(z, acc[1][t][4 * q4 + i], cap)
+                                       : FORM == 2 ? expert_gelu(z) : FORM == 4 ? expert_relu_squared(z) : z);
+                }
+                *reinterpret_cast<uint2*>(out + slot * n_features + feat) = make_uint2((uint32_t)v[0].bits | ((uint32_t)v[1].bits << 16),
+                                                                                       (uint32_t)v[2].bits | ((uint32_t)v[3].bits << 16));
+            }
+    }
+}
+
 // One block per token.
 __global__ void moe_combine_kernel(const bf16_t* __restrict__ y, const int* __restrict__ pair_slot, const float* __restrict__ weight, int top,
                                    int width, const bf16_t* __restrict__ add0, const bf16_t* __restrict__ add1, float* __restrict__ out) {
@@ -185,11 +321,15 @@ __global__ void moe_combine_kernel(const bf16_t* __restrict__ y, const int* __re
     }
 }
 
-PALM_API int palm_moe_tile_tokens() { return GT_TOKENS; }
+// Rows of a tile: the kernel whose operands cross LDS takes sizes in whole lines and pays from some 40 rows an expert on.
+static int tile_of(long long n_pairs, int experts, int width, int ff) {
+    return width % TILE_K == 0 && ff % TILE_K == 0 && n_pairs >= 40ll * experts ? TILE_ROWS : GT_TOKENS;
+}
+PALM_API int palm_moe_tile_tokens(int n_pairs, int experts, int width, int ff) { return tile_of(n_pairs, experts, width, ff); }
 
 // chosen, weight [n, top]; h bfloat16 [n, width]; gate_up bfloat16 [experts, 2 ff, width] (the plain forms: [experts, ff, width], up
 // rows alone); add0, add1: null or bfloat16 rows [n, width]; down bfloat16 [experts, width, ff].
-// Room, with max_tiles = ceil(n top / tile) + experts and slots = max_tiles * tile: plan: (2 experts + 1 + max_tiles + slots
+// Room, with tile = palm_moe_tile_tokens(n top, experts, width, ff), max_tiles = ceil(n top / tile) + experts and slots = max_tiles * tile: plan: (2 experts + 1 + max_tiles + slots
 // + n top) ints; mid: slots * ff bfloat16; y: slots * width bfloat16.  out float32 [n, width].
 PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gate_up, const void* down, const int* chosen,
                               const float* weight, int n_tokens, int top, int experts, int width, int ff, int* plan, void* mid, void* y,
@@ -203,16 +343,35 @@ PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gat
     if (n_tokens == 0) return 0;
     const long long n_pairs = (long long)n_tokens * top;
     PALM_CHECK(n_pairs < (1ll << 30), "moe_grouped: %lld pairs are more than one launch takes", n_pairs);
-    const int max_tiles = (int)((n_pairs + GT_TOKENS - 1) / GT_TOKENS) + experts;
+    const int tile = tile_of(n_pairs, experts, width, ff);
+    const int max_tiles = (int)((n_pairs + tile - 1) / tile) + experts;
     int* counts = plan;
     int* starts = counts + experts;
     int* tile_expert = starts + experts + 1;
     int* slot_pair = tile_expert + max_tiles;
-    int* pair_slot = slot_pair + (size_t)max_tiles * GT_TOKENS;
+    int* pair_slot = slot_pair + (size_t)max_tiles * tile;
     moe_count_kernel<<<experts, PLAN_THREADS, 0, stream>>>(chosen, (int)n_pairs, counts);
-    moe_runs_kernel<<<1, PLAN_THREADS, 0, stream>>>(counts, experts, max_tiles, starts, tile_expert);
+    moe_runs_kernel<<<1, PLAN_THREADS, 0, stream>>>(counts, experts, max_tiles, tile, starts, tile_expert);
     moe_place_kernel<<<experts, PLAN_THREADS, 0, stream>>>(chosen, (int)n_pairs, starts, slot_pair, pair_slot);
     const ExpertCap cap{limit, slope, shift};
+    if (tile == TILE_ROWS) {
+        auto blocks = [&](int feature_tiles) { return dim3((max_tiles * feature_tiles + TILE_DIES - 1) / TILE_DIES * TILE_DIES); };
+        const int up_features = expert_is_gated(form) ? TILE_W_ROWS / 2 : TILE_W_ROWS;
+        const int up_tiles = (ff + up_features - 1) / up_features, down_tiles = (width + TILE_W_ROWS - 1) / TILE_W_ROWS;
+        PALM_CHECK((long long)max_tiles * max(up_tiles, down_tiles) < (1ll << 30), "moe_grouped: %d tiles of rows are more than one launch takes", max_tiles);
+#define MOE_TILE_UP(FORM) moe_tile_kernel<FORM><<<blocks(up_tiles), TILE_WAVES * WAVE, 0, stream>>>((const bf16_t*)h, slot_pair, top, \
+            (const bf16_t*)gate_up, tile_expert, max_tiles, up_tiles, ff, width, cap, (bf16_t*)mid)
+        if (form == EXPERT_GATED_SILU) MOE_TILE_UP(1);
+        else if (form == EXPERT_GELU) MOE_TILE_UP(2);
+        else if (form == EXPERT_CAPPED) MOE_TILE_UP(3);
+        else MOE_TILE_UP(4);
+#undef MOE_TILE_UP
+        moe_tile_kernel<0><<<blocks(down_tiles), TILE_WAVES * WAVE, 0, stream>>>((const bf16_t*)mid, nullptr, top, (const bf16_t*)down, tile_expert,
+                                                                                 max_tiles, down_tiles, width, ff, cap, (bf16_t*)y);
+        moe_combine_kernel<<<n_tokens, 256, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, (const bf16_t*)add0, (const bf16_t*)add1, out);
+        PALM_LAUNCHED();
+        return 0;
+    }
     const dim3 up_grid(max_tiles, (ff + GT_FEATURES - 1) / GT_FEATURES);
 #define MOE_UP(FORM) moe_grouped_kernel<FORM><<<up_grid, GT_WAVES * WAVE, 0, stream>>>((const bf16_t*)h, slot_pair, top, (const bf16_t*)gate_up, \
         tile_expert, ff, width, cap, (bf16_t*)mid)

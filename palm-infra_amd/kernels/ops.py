@@ -825,7 +825,7 @@ _FEEDFORWARD_SIGNATURES = {
     "palm_moe_experts": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                          c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int],
     "palm_moe_route_table": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
-    "palm_moe_tile_tokens": [],
+    "palm_moe_tile_tokens": [c_int, c_int, c_int, c_int],
     "palm_moe_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
                          c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p],
     "palm_gather_rows": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
@@ -1747,7 +1747,7 @@ def moe_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chos
     experts = _expert_shapes(what, h, gate_up, down, ff, form)
     _need(down.dtype == BF16, f"{what}: bfloat16 weights")
     _need(chosen.shape == (n, top) and weight.shape == (n, top) and weight.dtype == F32, f"{what}: choices {tuple(chosen.shape)}, weights {tuple(weight.shape)}")
-    tile = feedforward().palm_moe_tile_tokens()
+    tile = feedforward().palm_moe_tile_tokens(n * top, experts, width, ff)
     max_tiles = (n * top + tile - 1) // tile + experts
     slots = max_tiles * tile
     plan = torch.empty((2 * experts + 1 + max_tiles + slots + n * top,), dtype=torch.int32, device=h.device)
