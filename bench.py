@@ -330,6 +330,12 @@ def other_sizes(name: str, args, sampler) -> dict:
 # and one decode step (launched one by one under the kernel recorder), and for the mixers' kernels the fraction of the
 # peak that binds them.
 
+def _experts_in_use(batch: int, f: dict) -> float:
+    """How many experts a step of ``batch`` rows reads, its choices being even: E (1 - (1 - top / E)^batch)."""
+    E, top = f["router"]["experts"], f["router"]["top"]
+    return E * (1.0 - (1.0 - top / E) ** batch)
+
+
 def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
     """entry point -> (prefill work, prefill peak, decode work, decode peak) for one launch, by the sizes of the first
     layer of each kind: flops against the matrix cores (attention for prompts) or the 32-bit vector units (the
@@ -349,8 +355,8 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
                 per = m["heads"] * m["dim"] * (m["vdim"] + 1)          # two multiply-adds for every element of the memory and token
                 out["palm_mlstm"] = (4.0 * tokens * per, vec, 2.0 * 4 * batch * per, hbm)
             f = layer.get("mlp")
-            if f and f["kind"] == "moe" and "palm_moe_experts" not in out:                 # plain experts: two matrices each
-                out["palm_moe_experts"] = (None, None, 2.0 * batch * f["router"]["top"] * 2 * f["expert"]["ff"] * raw["width"], hbm)
+            if f and f["kind"] == "moe" and "palm_moe_few" not in out:                 # plain experts: two matrices each
+                out["palm_moe_few"] = (None, None, 2.0 * _experts_in_use(batch, f) * 2 * f["expert"]["ff"] * raw["width"], hbm)
                 out["palm_moe_grouped"] = (2.0 * tokens * f["router"]["top"] * 2 * f["expert"]["ff"] * raw["width"], mfma, None, None)
     elif raw.get("architecture") == "Vovalix":
         for layer in raw["layers"]:
@@ -365,9 +371,9 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
                 out["palm_gla"] = (4.0 * tokens * per, vec, 2.0 * 4 * batch * per, hbm)
             elif layer["type"] == "delta":                              # four
                 out["palm_delta_head"] = (8.0 * tokens * per, vec, 2.0 * 4 * batch * per, hbm)
-            if f and "palm_moe_experts" not in out:
+            if f and "palm_moe_few" not in out:
                 amount = 2.0 * f["router"]["top"] * 3 * f["expert"]["ff"] * raw["width"]
-                out["palm_moe_experts"], out["palm_moe_grouped"] = (None, None, batch * amount, hbm), (tokens * amount, mfma, None, None)
+                out["palm_moe_few"], out["palm_moe_grouped"] = (None, None, _experts_in_use(batch, f) / f["router"]["top"] * amount, hbm), (tokens * amount, mfma, None, None)
     elif raw.get("architecture") == "Nirotar":
         for layer in raw["layers"]:
             m, f = layer["mixer"], layer.get("mlp")
@@ -384,7 +390,7 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
             if f:                                                          # plain experts: two matrices each; a decode step's launch has the shared one too
                 amount = 2.0 * f["router"]["top"] * 2 * f["expert"]["ff"] * raw["width"]
                 shared = 2.0 * 2 * f["shared"]["ff"] * raw["width"] if f.get("shared") else 0.0
-                out["palm_moe_experts"], out["palm_moe_grouped"] = (None, None, batch * amount + shared, hbm), (tokens * amount, mfma, None, None)
+                out["palm_moe_few"], out["palm_moe_grouped"] = (None, None, _experts_in_use(batch, f) * 2.0 * 2 * f["expert"]["ff"] * raw["width"] + shared, hbm), (tokens * amount, mfma, None, None)
     elif "layers" in raw:
         for layer in raw["layers"]:
             m = layer["mixer"]
@@ -419,9 +425,9 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
                 out["palm_sink_attention"] = (None, None, 2.0 * batch * min(context, w) * a["kv_heads"] * (a["dim"] + a["vdim"]), hbm)
                 per = r["heads"] * r["dim"] * r["vdim"]
                 out["palm_retention"] = (4.0 * tokens * per, vec, 2.0 * 4 * batch * per, hbm)
-            if layer.get("mlp") and layer["mlp"].get("kind") == "moe" and "palm_moe_experts" not in out:
+            if layer.get("mlp") and layer["mlp"].get("kind") == "moe" and "palm_moe_few" not in out:
                 f = layer["mlp"]
-                out["palm_moe_experts"] = (None, None, 2.0 * batch * f["router"]["top"] * 3 * f["expert"]["ff"] * raw["width"], hbm)
+                out["palm_moe_few"] = (None, None, 2.0 * _experts_in_use(batch, f) * 3 * f["expert"]["ff"] * raw["width"], hbm)
                 out["palm_moe_grouped"] = (2.0 * tokens * f["router"]["top"] * 3 * f["expert"]["ff"] * raw["width"], mfma, None, None)
     else:
         nh, nkv, hd = raw["num_attention_heads"], raw["num_key_value_heads"], raw["head_dim"]

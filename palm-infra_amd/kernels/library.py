@@ -62,7 +62,7 @@ DIFF_ATTENTION_SOURCES = ["attention_diff_mfma.hip"]
 LATENT_ATTENTION_SOURCES = ["latent_attention_mfma.hip"]
 MIXER_SOURCES = ["stream.hip", "mamba.hip", "attention_diff.hip", "residual_scaled.hip", "delta_rule.hip",
                  "latent_attention.hip"]
-FEEDFORWARD_SOURCES = ["moe.hip", "moe_grouped.hip", "activation.hip"]
+FEEDFORWARD_SOURCES = ["moe.hip", "moe_few.hip", "moe_grouped.hip", "activation.hip"]
 STREAMS_SOURCES = ["streams.hip"]
 MLSTM_SOURCES = ["mlstm.hip"]
 RECURRENT_SOURCES = ["retention.hip"]
@@ -74,7 +74,7 @@ BRANCH_SOURCES = ["branch_scaled.hip"]
 HEADERS = ["common.h", "mfma.h", "linear_thin.h", "linear_wide.h", "attention_api.h"]
 # headers of a few sources only: a change of one rebuilds the libraries of the sources that include it
 OWN_HEADERS = {"retention.hip": ["linear_recurrence.h"], "gla.hip": ["linear_recurrence.h"], "delta_rule.hip": ["delta_rule.h"],
-               "delta_head.hip": ["delta_rule.h", "conv_state.h"], "mamba.hip": ["conv_state.h"], "moe.hip": ["expert_form.h"],
+               "delta_head.hip": ["delta_rule.h", "conv_state.h"], "mamba.hip": ["conv_state.h"], "moe.hip": ["expert_form.h"], "moe_few.hip": ["expert_form.h"],
                "moe_grouped.hip": ["expert_form.h", "lds_stage.h"], "linear_tile.hip": ["lds_stage.h"], "branch_scaled.hip": ["expert_form.h"]}
 
 

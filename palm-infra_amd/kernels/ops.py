@@ -824,6 +824,9 @@ _FEEDFORWARD_SIGNATURES = {
     "palm_add_gated_rows": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int],
     "palm_moe_experts": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                          c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int],
+    "palm_moe_few": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
+                     c_void_p, c_int, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
+    "palm_moe_few_planes": [c_int],
     "palm_moe_route_table": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
     "palm_moe_tile_tokens": [c_int, c_int, c_int, c_int],
     "palm_moe_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
@@ -1704,11 +1707,51 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chos
     [n]: ``chosen`` is a table [vocab, top] of which each row takes the row of its token's id, and every choice weighs 1 / top
     (``weight`` None).  ``shared`` (first matrix, down): one more expert of the same form, for every row, with weight one."""
     what = "moe_experts"
+    n, width = h.shape
+    top = chosen.shape[1]
+    shared_up, shared_down, shared_ff = _few_rows(what, h, gate_up, down, chosen, weight, ff, form, ids, shared)[1:]
+    mid = torch.empty((n, top * ff + shared_ff), dtype=F32, device=h.device)
+    out = torch.empty((n, width), dtype=F32, device=h.device)
+    library.call(feedforward(), "palm_moe_experts", _stream(), _p(h), _code(h, what), _p(gate_up), _p(down), _code(gate_up, what + " weights"),
+                 _p(chosen), _p(weight), n, top, width, ff, _p(mid), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h),
+                 _p(ids), chosen.shape[0] if ids is not None else 0, _p(shared_up), _p(shared_down), shared_ff)
+    return out
+
+
+FEW_ROWS, FEW_EXPERTS, FEW_PAIRS = 128, 512, 4096
+
+
+def moe_few_serves(h: torch.Tensor, gate_up: torch.Tensor, ff: int, experts: int, top: int, shared=None) -> bool:
+    """Whether the matrix cores take a step of few rows: bfloat16 rows and matrices, sizes in multiples of eight."""
+    return (h.dtype == BF16 and gate_up.dtype == BF16 and h.shape[0] <= FEW_ROWS and h.shape[0] * top <= FEW_PAIRS and experts <= FEW_EXPERTS
+            and h.shape[1] % 8 == 0 and ff % 8 == 0 and (shared is None or (shared[1].shape[1] % 8 == 0 and shared[0].dtype == BF16)))
+
+
+def moe_few(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor | None, ff: int,
+            form: str = "gated_silu", cap=NO_CAP, add=(), ids: torch.Tensor | None = None, shared=None, planes_ok: bool = False) -> torch.Tensor:
+    """``moe_experts`` on the matrix cores (its arguments): every expert in use is read once for all its rows.  Returns float32
+    [n, width], or with ``planes_ok`` possibly planes [P, n, width] for a reader that adds them."""
+    what = "moe_few"
+    n, width = h.shape
+    top = chosen.shape[1]
+    experts, shared_up, shared_down, shared_ff = _few_rows(what, h, gate_up, down, chosen, weight, ff, form, ids, shared)
+    _need(moe_few_serves(h, gate_up, ff, experts, top, shared), f"{what}: at most {FEW_ROWS} bfloat16 rows, bfloat16 weights, sizes in multiples of eight")
+    planes = feedforward().palm_moe_few_planes(width) if planes_ok else 1
+    mid = torch.empty((n, top * ff + shared_ff), dtype=BF16, device=h.device)
+    out = torch.empty((planes, n, width), dtype=F32, device=h.device)
+    library.call(feedforward(), "palm_moe_few", _stream(), _p(h), _p(gate_up), _p(down), _p(chosen), _p(weight), _p(ids),
+                 chosen.shape[0] if ids is not None else 0, n, top, experts, width, ff, _p(shared_up), _p(shared_down), shared_ff,
+                 EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h), _p(mid), planes, _p(out))
+    return out if planes > 1 else out[0]
+
+
+def _few_rows(what: str, h, gate_up, down, chosen, weight, ff: int, form: str, ids, shared):
+    """The checks of both kernels for few rows: (experts, the shared expert's matrices and inner size)."""
     _dev(what, h, gate_up, down, chosen, weight, ids)
     _i32(what, chosen, ids)
     n, width = h.shape
     top = chosen.shape[1]
-    _expert_shapes(what, h, gate_up, down, ff, form)
+    experts = _expert_shapes(what, h, gate_up, down, ff, form)
     if ids is None:
         _need(chosen.shape == (n, top) and weight is not None and weight.shape == (n, top) and weight.dtype == F32,
               f"{what}: choices {tuple(chosen.shape)}, weights {None if weight is None else tuple(weight.shape)}")
@@ -1720,12 +1763,7 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chos
         _dev(what, shared_up, shared_down)
         _need(shared_up.shape == (expert_rows(form) * shared_ff, width) and shared_down.shape == (width, shared_ff) and shared_up.dtype == gate_up.dtype
               and shared_down.dtype == gate_up.dtype, f"{what}: the shared expert's matrices {tuple(shared_up.shape)}, {tuple(shared_down.shape)}")
-    mid = torch.empty((n, top * ff + shared_ff), dtype=F32, device=h.device)
-    out = torch.empty((n, width), dtype=F32, device=h.device)
-    library.call(feedforward(), "palm_moe_experts", _stream(), _p(h), _code(h, what), _p(gate_up), _p(down), _code(gate_up, what + " weights"),
-                 _p(chosen), _p(weight), n, top, width, ff, _p(mid), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h),
-                 _p(ids), chosen.shape[0] if ids is not None else 0, _p(shared_up), _p(shared_down), shared_ff)
-    return out
+    return experts, shared_up, shared_down, shared_ff
 
 
 def moe_grouped_serves(h: torch.Tensor, gate_up: torch.Tensor, ff: int) -> bool:

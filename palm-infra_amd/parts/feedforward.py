@@ -140,11 +140,19 @@ class RoutedExperts:
         z = self.expert_first[e](xs)
         return ops.capped_gate(z, *self.cap) if self.form == "capped_gated" else ops.activation(z, ops.PLAIN_EXPERTS[self.form])
 
+    def run_few(self, h, chosen, weight, add=(), ids=None, shared=None, planes_ok=False):
+        """``run_experts`` for at most DIRECT_ROWS rows, planned nowhere: the matrix cores, or the kernels that each (row, choice)
+        reads its expert in.  ``ids``, ``shared``: see ``ops.moe_experts``; ``planes_ok``: float32 planes may come back."""
+        args = (h, self.first, self.down_all, chosen, weight, self.inter, self.form, self.cap, add, ids, shared)
+        if ops.moe_few_serves(h, self.first, self.inter, self.experts, chosen.shape[1], shared):
+            return ops.moe_few(*args, planes_ok=planes_ok)
+        return ops.moe_experts(*args)
+
     def run_experts(self, h, chosen, weight, add=()):
         """float32 [n, hidden]: sum_c weight[t, c] * expert chosen[t, c] of h[t], plus the rows ``add`` (up to two)."""
         top = chosen.shape[1]
         if h.shape[0] <= self.DIRECT_ROWS:
-            return ops.moe_experts(h, self.first, self.down_all, chosen, weight, self.inter, self.form, self.cap, add)
+            return self.run_few(h, chosen, weight, add)
         if ops.moe_grouped_serves(h, self.first, self.inter):
             return ops.moe_grouped(h, self.first, self.down_all, chosen, weight, self.inter, self.form, self.cap, add)
         # group the (token, choice) pairs by expert; within an expert in the order of the tokens
@@ -263,6 +271,7 @@ class RoutedScoredFeedForward(RoutedExperts):
 @register_part("feed_forward", "routed_table")
 class RoutedTableFeedForward(RoutedExperts):
     capturable = True
+    takes_sink = True            # (for planes of partial sums, which the norm that reads the stream next adds)
     SHARED_DIRECT_ROWS = 16      # as many rows share the shared expert's weights well enough when each reads them for itself
 
     def __init__(self, spec, builder):
@@ -289,15 +298,21 @@ class RoutedTableFeedForward(RoutedExperts):
             self.shared_fits = (all(s.weight.dtype == self.first.dtype for s in self.shared)
                                 and self.top * self.inter + int(p["shared_size"]) <= ops.MOE_ROW_VALUES)
 
-    def forward(self, h, ctx):
+    def forward(self, h, ctx, sink=None):
         h = as_tensor(h)
-        direct = self.shared is not None and h.shape[0] <= self.SHARED_DIRECT_ROWS and self.shared_fits
+        out = self._run(h, ctx, sink is not None and sink.takes_planes)
+        return out if sink is None else sink.finish(out)
+
+    def _run(self, h, ctx, planes_ok):
+        n, shared = h.shape[0], tuple(s.weight for s in self.shared) if self.shared is not None else None
+        # in a step of few rows the shared expert rides in the experts' own kernels
+        rides = shared is not None and n <= self.DIRECT_ROWS and (
+            ops.moe_few_serves(h, self.first, self.inter, self.experts, self.top, shared) or (n <= self.SHARED_DIRECT_ROWS and self.shared_fits))
         add = []
-        if self.shared is not None and not direct:
+        if shared is not None and not rides:
             up, down = self.shared
             add.append(down(ops.activation(up(h), ops.PLAIN_EXPERTS[self.form])))
-        if h.shape[0] <= self.DIRECT_ROWS:
-            return ops.moe_experts(h, self.first, self.down_all, self.table, None, self.inter, self.form, add=add, ids=ctx.token_ids,
-                                   shared=tuple(s.weight for s in self.shared) if direct else None)
+        if n <= self.DIRECT_ROWS:
+            return self.run_few(h, self.table, None, add, ids=ctx.token_ids, shared=shared if rides else None, planes_ok=planes_ok)
         chosen, weight = ops.moe_route_table(ctx.token_ids, self.table)
         return self.run_experts(h, chosen, weight, add)

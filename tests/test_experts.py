@@ -66,3 +66,36 @@ def test_grouped_products(form, E, top, W, F, n, uneven):
     y = torch.randn(n, W).to(torch.bfloat16)
     more = ops.moe_grouped(*args, F, form, CAP if form == "capped_gated" else ops.NO_CAP, add=[y.cuda()])
     assert torch.allclose(more - got, y.cuda().float(), atol=1e-4)
+
+
+@gpu
+@pytest.mark.parametrize("form", ["gated_silu", "gelu", "capped_gated", "relu_squared"])
+@pytest.mark.parametrize("E,top,W,F,shared", [(4, 2, 64, 64, 40), (3, 1, 72, 24, None), (33, 4, 320, 264, 264), (5, 5, 8, 8, 16), (512, 3, 48, 16, None), (6, 2, 2056, 520, 1032)])
+def test_few_rows(form, E, top, W, F, shared):
+    """One row, a decode batch's rows, and as many as a recorded step holds: both kernels for few rows, with a shared expert and
+    with planes of partial sums."""
+    from palm_infra_amd.kernels import ops
+    cap = CAP if form == "capped_gated" else ops.NO_CAP
+    for n, uneven in ((1, False), (8, False), (17, True), (40, False), (70, True), (128, True), (128, False)):
+        h, up, down, chosen, weight = case(form, E, top, W, F, n, uneven, E + F + n, torch.bfloat16)
+        want = plain_mixture(form, h, up, down, chosen, weight, F)
+        extra = None
+        if shared:
+            per = (2 if form in ("gated_silu", "capped_gated") else 1) * shared
+            extra = ((torch.randn(per, W) * W ** -0.5).to(torch.bfloat16), (torch.randn(W, shared) * shared ** -0.5).to(torch.bfloat16))
+            want += plain_expert(form, h.double() @ extra[0].double().T, shared) @ extra[1].double().T
+            extra = tuple(t.cuda() for t in extra)
+        args = [t.cuda() for t in (h, up, down, chosen, weight)]
+        tol = 0.02 * float(want.abs().max())
+        got = ops.moe_few(*args, F, form, cap, shared=extra)
+        assert float((got.cpu().double() - want).abs().max()) <= tol, (n, uneven)
+        again = ops.moe_few(*args, F, form, cap, shared=extra)
+        assert torch.equal(got, again)
+        planes = ops.moe_few(*args, F, form, cap, shared=extra, planes_ok=True)
+        planes = planes if planes.dim() == 2 else planes.sum(0)
+        assert torch.allclose(planes, got, atol=1e-4 * float(want.abs().max()), rtol=1e-4)
+        exact = ops.moe_experts(*args, F, form, cap, shared=extra)
+        assert float((exact.cpu().double() - want).abs().max()) <= tol, (n, uneven)
+        y = [torch.randn(n, W).to(torch.bfloat16).cuda() for _ in range(2)]
+        more = ops.moe_few(*args, F, form, cap, add=y, shared=extra)
+        assert torch.allclose(more, got + y[0].float() + y[1].float(), atol=1e-3, rtol=1e-4)
