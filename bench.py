@@ -456,7 +456,7 @@ def design_points(raw: dict, args, tokens: int, batch: int, context: int) -> dic
     slot = engine.open()
     with rec:
         engine.step([StepEntry(slot, random_ids(tokens, vocab, 77), [tokens - 1])])
-        engine.step([StepEntry(s, [1], [0]) for s in slots])
+        engine.step([StepEntry(s, [t], [0]) for s, t in zip(slots, random_ids(batch, vocab, 78))])
         torch.cuda.synchronize()
     engine.close(slot)
     roofs = _mixer_rooflines(raw, tokens, batch, context)

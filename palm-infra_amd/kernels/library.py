@@ -75,7 +75,8 @@ HEADERS = ["common.h", "mfma.h", "linear_thin.h", "linear_wide.h", "attention_ap
 # headers of a few sources only: a change of one rebuilds the libraries of the sources that include it
 OWN_HEADERS = {"retention.hip": ["linear_recurrence.h"], "gla.hip": ["linear_recurrence.h"], "delta_rule.hip": ["delta_rule.h"],
                "delta_head.hip": ["delta_rule.h", "conv_state.h"], "mamba.hip": ["conv_state.h"], "moe.hip": ["expert_form.h"], "moe_few.hip": ["expert_form.h"],
-               "moe_grouped.hip": ["expert_form.h", "lds_stage.h"], "linear_tile.hip": ["lds_stage.h"], "branch_scaled.hip": ["expert_form.h"]}
+               "moe_grouped.hip": ["expert_form.h", "lds_stage.h"], "linear_tile.hip": ["lds_stage.h"], "attention_sink_mfma.hip": ["lds_stage.h"],
+               "branch_scaled.hip": ["expert_form.h"]}
 
 
 class KernelBuildError(RuntimeError):
