@@ -13,10 +13,13 @@
 //                      of latent_attention_mfma.hip, the latent into a bfloat16 copy with the positions innermost)
 //   latent_query       q rows -> [a_h | rotated q_rot,h] per head, 32-bit; where the queries come straight from the layer's
 //                      input (no query latent to be normed first) the same launch writes the positions' cache rows
+//                      (latent_query_mfma: the same on the matrix cores in bfloat16, from the key matrices' transposes)
+//   latent_turn        the queries as they are with their rotated parts turned, and the cache rows, for prompts whose keys and
+//                      values are expanded; latent_gather: the latents and key parts of whole sequences in plain rows for that
 //   latent_attention   softmax over the visible rows (causal, optional window, optionally one more term exp(sink_h) in the
 //                      denominator), o_lat,h = sum_j p_j c_j, 32-bit
 //   latent_output      head h: sigmoid(gate_h) * U_v,h o_lat,h
-#include "common.h"
+#include "mfma.h"
 
 constexpr int LAT_THREADS = 256;
 
@@ -182,6 +185,113 @@ __global__ __launch_bounds__(LQ_COLS) void latent_query_kernel(
 #pragma unroll
     for (int ti = 0; ti < LQ_TILE; ++ti)
         if (ti < tt) qa[((size_t)(t0 + ti) * heads + h) * dk + r] = acc[ti];
+}
+
+// The same queries on the matrix cores, bfloat16: a wave makes 16 latent columns of one head for 16 CT tokens; uk_t [heads, kv_rank,
+// dim] holds the key matrices' transposes, so that both operands are runs along the key size.  The first columns' blocks also
+// rotate, and share out the cache rows as above.
+constexpr int LQM_WAVES = 4;
+
+__device__ inline bf16x8 lat_row8(const bf16_t* row, int col, int dim) {
+    const bf16x8 v = load_bf16x8(row + min(col, dim - 8));
+    return col < dim ? v : zero_bf16x8();
+}
+
+template <int CT>
+__global__ __launch_bounds__(LQM_WAVES * WAVE) void latent_query_mfma_kernel(
+    const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ uk_t, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+    int n_tokens, int heads, int dim, int rot_dim, int kv_rank, int neighbours, LatentStore<bf16_t> st, float* __restrict__ qa) {
+    const int t0 = blockIdx.x * 16 * CT, h = blockIdx.y, tt = min(16 * CT, n_tokens - t0);
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, r = lane % 16, g = lane / 16;
+    const int hd = dim + rot_dim, dk = kv_rank + rot_dim, half = rot_dim / 2;
+    if (blockIdx.z == 0) {
+        for (int idx = threadIdx.x; idx < tt * half; idx += LQM_WAVES * WAVE) {
+            const int i = idx % half;
+            const size_t row = t0 + idx / half;
+            const bf16_t* qr = q + row * q_stride + (size_t)h * hd + dim;
+            const float c = cos_t[row * half + i], s = sin_t[row * half + i];
+            const int i0 = pair_first(i, neighbours), i1 = pair_second(i, half, neighbours);
+            const float a = to_float(qr[i0]), b = to_float(qr[i1]);
+            float* o = qa + (row * heads + h) * dk + kv_rank;
+            o[i0] = a * c - b * s;
+            o[i1] = b * c + a * s;
+        }
+        if (st.src)
+            for (int ti = h * LQM_WAVES + wave; ti < tt; ti += heads * LQM_WAVES)
+                latent_store_row(st, (size_t)(t0 + ti), kv_rank, rot_dim, cos_t, sin_t, neighbours, lane);
+    }
+    const int r0 = (blockIdx.z * LQM_WAVES + wave) * 16;
+    if (r0 >= kv_rank) return;
+    const bf16_t* wr = uk_t + ((size_t)h * kv_rank + min(r0 + r, kv_rank - 1)) * dim;
+    const bf16_t* xr[CT];
+    f32x4 acc[CT];
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+        xr[ct] = q + (size_t)(t0 + min(16 * ct + r, tt - 1)) * q_stride + (size_t)h * hd;
+        acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll 4
+    for (int k = 0; k < dim; k += 32) {
+        const bf16x8 wf = lat_row8(wr, k + 8 * g, dim);
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct) acc[ct] = mfma_16x16x32(wf, lat_row8(xr[ct], k + 8 * g, dim), acc[ct]);
+    }
+    // lane (r, g) holds latent columns r0 + 4 g + i of token r
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+        const int t = 16 * ct + r, d = r0 + 4 * g;
+        if (t < tt && d < kv_rank)                               // kv_rank is a multiple of four
+            *reinterpret_cast<float4*>(qa + ((size_t)(t0 + t) * heads + h) * dk + d) = make_float4(acc[ct][0], acc[ct][1], acc[ct][2], acc[ct][3]);
+    }
+}
+
+// One block per token: out [n, heads, dim + rot_dim], every head's plain part as it is and its rotated part turned; the last wave
+// writes the token's cache row.
+template <typename T>
+__global__ __launch_bounds__(LAT_THREADS) void latent_turn_kernel(const T* __restrict__ q, int q_stride, const float* __restrict__ cos_t,
+                                                                  const float* __restrict__ sin_t, int heads, int dim, int rot_dim, int kv_rank,
+                                                                  int neighbours, LatentStore<T> st, T* __restrict__ out) {
+    const size_t row = blockIdx.x;
+    const int hd = dim + rot_dim, half = rot_dim / 2;
+    const T* qr = q + row * q_stride;
+    T* o = out + row * heads * hd;
+    constexpr int VEC = 16 / sizeof(T);                          // dim and rot_dim are multiples of eight
+    for (int idx = threadIdx.x; idx < heads * (dim / VEC); idx += LAT_THREADS) {
+        const int at = idx / (dim / VEC) * hd + idx % (dim / VEC) * VEC;
+        *reinterpret_cast<uint4*>(o + at) = *reinterpret_cast<const uint4*>(qr + at);
+    }
+    for (int idx = threadIdx.x; idx < heads * half; idx += LAT_THREADS) {
+        const int base = idx / half * hd + dim, i = idx % half;
+        const float c = cos_t[row * half + i], s = sin_t[row * half + i];
+        const int i0 = base + pair_first(i, neighbours), i1 = base + pair_second(i, half, neighbours);
+        const float a = to_float(qr[i0]), b = to_float(qr[i1]);
+        o[i0] = from_float<T>(a * c - b * s);
+        o[i1] = from_float<T>(b * c + a * s);
+    }
+    const int wave = threadIdx.x / WAVE;
+    if (st.src && wave == LAT_THREADS / WAVE - 1)
+        latent_store_row(st, row, kv_rank, rot_dim, cos_t, sin_t, neighbours, threadIdx.x % WAVE);
+}
+
+// One block per gathered page: the 64 cache rows of page page_of[i] of sequence seq_of[i], its latents to c [*, kv_rank] and its key
+// parts to k2 [*, rot_dim]; zero where a row lies beyond the sequence's last.
+template <typename T>
+__global__ __launch_bounds__(LAT_THREADS) void latent_gather_kernel(const T* __restrict__ rows_cache, const int* __restrict__ block_table,
+                                                                    int max_pages, const int* __restrict__ seq_slot, const int* __restrict__ seq_start,
+                                                                    const int* __restrict__ seq_new, const int* __restrict__ seq_of,
+                                                                    const int* __restrict__ page_of, int kv_rank, int rot_dim,
+                                                                    T* __restrict__ c, T* __restrict__ k2) {
+    const int b = seq_of[blockIdx.x], pg = page_of[blockIdx.x];
+    const int dk = kv_rank + rot_dim, last = seq_start[b] + seq_new[b] - 1 - pg * PAGE_TOKENS;
+    const T* from = rows_cache + (size_t)block_table[(size_t)seq_slot[b] * max_pages + pg] * PAGE_TOKENS * dk;
+    constexpr int VEC = 16 / sizeof(T);                          // the sizes are multiples of eight
+    const size_t row0 = (size_t)blockIdx.x * PAGE_TOKENS;
+    for (int idx = threadIdx.x; idx < PAGE_TOKENS * (dk / VEC); idx += LAT_THREADS) {
+        const int j = idx / (dk / VEC), d = idx % (dk / VEC) * VEC;
+        const uint4 v = j <= last ? *reinterpret_cast<const uint4*>(from + (size_t)j * dk + d) : make_uint4(0, 0, 0, 0);
+        T* to = d < kv_rank ? c + (row0 + j) * kv_rank + d : k2 + (row0 + j) * rot_dim + d - kv_rank;
+        *reinterpret_cast<uint4*>(to) = v;
+    }
 }
 
 // One block of LA_WAVES waves per (query, group of HG heads).  A wave takes every LA_WAVES-th page of the key range;
@@ -426,6 +536,70 @@ PALM_API int palm_latent_query(hipStream_t stream, const void* q, int dtype, int
                                                                         rot_dim, kv_rank, pairing, st, qa);
         });
     });
+    PALM_LAUNCHED();
+    return 0;
+}
+
+// uk_t bfloat16 [heads, kv_rank, dim]; q's rows, a head's columns and the sizes in steps of eight; else as palm_latent_query.
+PALM_API int palm_latent_query_mfma(hipStream_t stream, const void* q, int q_stride, const void* uk_t, const float* cos_t, const float* sin_t,
+                                    int n_tokens, int heads, int dim, int rot_dim, int kv_rank, int pairing, float* qa, const void* store,
+                                    int store_stride, const float* kv_norm_w, float eps, const int* positions, const int* tok_slot,
+                                    const int* block_table, int max_pages, void* rows_cache, void* rows_t, const int* block_table_t) {
+    PALM_CHECK(n_tokens >= 0 && heads > 0 && heads <= 65535 && dim > 0 && kv_rank > 0 && rot_dim >= 0 && rot_dim % 2 == 0,
+               "latent_query_mfma: n=%d heads=%d dim=%d rot_dim=%d kv_rank=%d", n_tokens, heads, dim, rot_dim, kv_rank);
+    PALM_CHECK(dim % 8 == 0 && rot_dim % 8 == 0 && kv_rank % 8 == 0 && q_stride % 8 == 0 && (uintptr_t)q % 16 == 0, "latent_query_mfma: sizes %d, %d, "
+               "%d and rows of %d in steps of eight", dim, rot_dim, kv_rank, q_stride);
+    PALM_CHECK(rot_dim == 0 || (cos_t && sin_t), "latent_query_mfma: a rotation needs its cos and sin rows");
+    PALM_CHECK(q_stride >= heads * (dim + rot_dim), "latent_query_mfma: rows of %d do not hold %d heads of %d + %d", q_stride, heads, dim, rot_dim);
+    PALM_CHECK(pairing == 0 || pairing == 1, "latent_query_mfma: pairing %d is neither halves (0) nor neighbours (1)", pairing);
+    PALM_CHECK(!store || (kv_norm_w && positions && tok_slot && block_table && max_pages > 0 && rows_cache && store_stride >= kv_rank + rot_dim),
+               "latent_query_mfma: cache rows need the latents' norm, positions, slots, pages and rows of %d + %d", kv_rank, rot_dim);
+    PALM_CHECK(!rows_t || block_table_t, "latent_query_mfma: the transposed copy needs its page table");
+    if (n_tokens == 0) return 0;
+    const LatentStore<bf16_t> st{(const bf16_t*)store, store_stride, kv_norm_w, eps, positions, tok_slot, block_table, max_pages, (bf16_t*)rows_cache,
+                                 (bf16_t*)rows_t, block_table_t};
+    const int runs = (kv_rank + 16 * LQM_WAVES - 1) / (16 * LQM_WAVES);
+#define LQM_LAUNCH(CT) latent_query_mfma_kernel<CT><<<dim3((n_tokens + 16 * CT - 1) / (16 * CT), heads, runs), LQM_WAVES * WAVE, 0, stream>>>( \
+        (const bf16_t*)q, q_stride, (const bf16_t*)uk_t, cos_t, sin_t, n_tokens, heads, dim, rot_dim, kv_rank, pairing, st, qa)
+    if (n_tokens <= 16) LQM_LAUNCH(1); else LQM_LAUNCH(4);
+#undef LQM_LAUNCH
+    PALM_LAUNCHED();
+    return 0;
+}
+
+// out [n, heads, dim + rot_dim] of q's type; store and what follows as in palm_latent_query.
+PALM_API int palm_latent_turn(hipStream_t stream, const void* q, int dtype, int q_stride, const float* cos_t, const float* sin_t, int n_tokens,
+                              int heads, int dim, int rot_dim, int kv_rank, int pairing, void* out, const void* store, int store_stride,
+                              const float* kv_norm_w, float eps, const int* positions, const int* tok_slot, const int* block_table, int max_pages,
+                              void* rows_cache, void* rows_t, const int* block_table_t) {
+    PALM_CHECK(n_tokens >= 0 && heads > 0 && dim > 0 && dim % 8 == 0 && rot_dim >= 0 && rot_dim % 8 == 0 && q_stride % 8 == 0 && (uintptr_t)q % 16 == 0,
+               "latent_turn: n=%d heads=%d of %d + %d in rows of %d (steps of eight)", n_tokens, heads, dim, rot_dim, q_stride);
+    PALM_CHECK(rot_dim == 0 || (cos_t && sin_t), "latent_turn: a rotation needs its cos and sin rows");
+    PALM_CHECK(q_stride >= heads * (dim + rot_dim), "latent_turn: rows of %d do not hold %d heads of %d + %d", q_stride, heads, dim, rot_dim);
+    PALM_CHECK(pairing == 0 || pairing == 1, "latent_turn: pairing %d is neither halves (0) nor neighbours (1)", pairing);
+    PALM_CHECK(!store || (kv_norm_w && positions && tok_slot && block_table && max_pages > 0 && rows_cache && kv_rank > 0 && store_stride >= kv_rank + rot_dim),
+               "latent_turn: cache rows need the latents' norm, positions, slots, pages and rows of %d + %d", kv_rank, rot_dim);
+    PALM_CHECK(!rows_t || block_table_t, "latent_turn: the transposed copy needs its page table");
+    if (n_tokens == 0) return 0;
+    PALM_DTYPE_SWITCH(dtype, T, {
+        const LatentStore<T> st{(const T*)store, store_stride, kv_norm_w, eps, positions, tok_slot, block_table, max_pages, (T*)rows_cache,
+                                (bf16_t*)rows_t, block_table_t};
+        latent_turn_kernel<T><<<n_tokens, LAT_THREADS, 0, stream>>>((const T*)q, q_stride, cos_t, sin_t, heads, dim, rot_dim, kv_rank, pairing, st,
+                                                                    (T*)out);
+    });
+    PALM_LAUNCHED();
+    return 0;
+}
+
+// n_pages gathered pages: c [64 n_pages, kv_rank], k2 [64 n_pages, rot_dim].
+PALM_API int palm_latent_gather(hipStream_t stream, const void* rows_cache, int dtype, const int* block_table, int max_pages, const int* seq_slot,
+                                const int* seq_start, const int* seq_new, const int* seq_of, const int* page_of, int n_pages, int kv_rank,
+                                int rot_dim, void* c, void* k2) {
+    PALM_CHECK(n_pages >= 0 && max_pages > 0 && kv_rank > 0 && kv_rank % 8 == 0 && rot_dim >= 0 && rot_dim % 8 == 0,
+               "latent_gather: %d pages (tables of %d) of rows %d + %d in steps of eight", n_pages, max_pages, kv_rank, rot_dim);
+    if (n_pages == 0) return 0;
+    PALM_DTYPE_SWITCH(dtype, T, latent_gather_kernel<T><<<n_pages, LAT_THREADS, 0, stream>>>(
+        (const T*)rows_cache, block_table, max_pages, seq_slot, seq_start, seq_new, seq_of, page_of, kv_rank, rot_dim, (T*)c, (T*)k2));
     PALM_LAUNCHED();
     return 0;
 }

@@ -407,7 +407,8 @@ __global__ __launch_bounds__(LM_WAVES * WAVE) void latent_merge_output_kernel(
     const float* __restrict__ sink_scores, const bf16_t* __restrict__ uv, const bf16_t* __restrict__ gate, int gate_stride, int vdim,
     bf16_t* __restrict__ out) {
     __shared__ float w_s[LM_MAX_SLICES];
-    __shared__ float o_s[VT * 16];
+    __shared__ __attribute__((aligned(16))) float part_s[LM_WAVES][VT * 16];
+    __shared__ __attribute__((aligned(16))) float o_s[VT * 16];
     const int h = blockIdx.x, j0 = blockIdx.y * LM_ROWS;
     const size_t b = blockIdx.z;
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
@@ -426,11 +427,23 @@ __global__ __launch_bounds__(LM_WAVES * WAVE) void latent_merge_output_kernel(
     __syncthreads();
     const float inv = 1.0f / l;
     const float* wk = work + (b * heads + h) * n_slices * kv_rank;
+    // a wave takes every fourth slice, a lane four neighbouring columns; what a slice without pages left unwritten counts as nothing
+    for (int d = 4 * lane; d < kv_rank; d += 4 * WAVE) {
+        float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 4
+        for (int s = wave; s < n_slices; s += LM_WAVES) {
+            const float4 v = *reinterpret_cast<const float4*>(wk + (size_t)s * kv_rank + d);
+            const float f = w_s[s];
+            o.x = fmaf(f != 0.f ? v.x : 0.f, f, o.x); o.y = fmaf(f != 0.f ? v.y : 0.f, f, o.y);
+            o.z = fmaf(f != 0.f ? v.z : 0.f, f, o.z); o.w = fmaf(f != 0.f ? v.w : 0.f, f, o.w);
+        }
+        *reinterpret_cast<float4*>(&part_s[wave][d]) = o;
+    }
+    __syncthreads();
     for (int d = threadIdx.x; d < kv_rank; d += LM_WAVES * WAVE) {
         float o = 0.f;
-#pragma unroll 4
-        for (int s = 0; s < n_slices; ++s)
-            if (w_s[s] != 0.f) o = fmaf(wk[(size_t)s * kv_rank + d], w_s[s], o);   // (what a slice without pages left unwritten counts as nothing)
+#pragma unroll
+        for (int w = 0; w < LM_WAVES; ++w) o += part_s[w][d];
         o_s[d] = o * inv;
     }
     __syncthreads();

@@ -784,6 +784,12 @@ _MIXER_SIGNATURES = {
                          c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int],
     "palm_latent_query": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                           c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
+    "palm_latent_query_mfma": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
+                               c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
+    "palm_latent_turn": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
+                         c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
+    "palm_latent_gather": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                           c_void_p, c_void_p],
     "palm_latent_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                               c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p],
     "palm_latent_output": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
@@ -1407,11 +1413,20 @@ class LatentStore:
     table_t: torch.Tensor | None = None
 
 
+def latent_key_transposes(uk: torch.Tensor, heads: int, dim: int, kv_rank: int) -> torch.Tensor | None:
+    """The key matrices [heads * dim, kv_rank] as [heads, kv_rank, dim], which is how the matrix cores read them for the queries
+    (bfloat16, sizes in steps of eight; else None)."""
+    if uk.dtype != BF16 or dim % 8 or kv_rank % 8:
+        return None
+    return uk.view(heads, dim, kv_rank).transpose(1, 2).contiguous()
+
+
 def latent_query(q: torch.Tensor, uk: torch.Tensor, cos, sin, heads: int, dim: int, rot_dim: int, kv_rank: int,
-                 pairing: str = "half_split", ctx=None, store: LatentStore | None = None) -> torch.Tensor:
+                 pairing: str = "half_split", ctx=None, store: LatentStore | None = None, uk_t: torch.Tensor | None = None) -> torch.Tensor:
     """q [n, heads * (dim + rot_dim)] (a view of wider rows is fine), uk [heads * dim, kv_rank] -> float32 [n, heads, kv_rank +
     rot_dim]: each head's plain part taken through its key matrix, its rotated part behind it (``pairing``: dimension i with i +
-    rot_dim/2, or 2i with 2i + 1).  ``store``: the same launch norms and rotates what the step's tokens keep and writes it."""
+    rot_dim/2, or 2i with 2i + 1).  ``store``: the same launch norms and rotates what the step's tokens keep and writes it.
+    ``uk_t``: the key matrices' transposes (``latent_key_transposes``): bfloat16 queries then go to the matrix cores."""
     what = "latent_query"
     _dev(what, uk)
     n = q.shape[0]
@@ -1419,18 +1434,114 @@ def latent_query(q: torch.Tensor, uk: torch.Tensor, cos, sin, heads: int, dim: i
           f"{what}: q {tuple(q.shape)}, key matrix {tuple(uk.shape)} for {heads} heads of {dim} + {rot_dim} and a latent of {kv_rank}")
     _need(pairing in ROTARY_PAIRINGS, f"{what}: pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
     _latent_rotation(what, cos, sin, n, rot_dim)
-    keep = [None, 0, None, 0.0, None, None, None, 0, None, None, None]
-    if store is not None:
-        src = store.src
-        _latent_rows(what, q.dtype, kv_rank, rot_dim, store.norm_w, store.rows_cache, store.block_table, ctx, store.rows_t, store.table_t, pairing)
-        _need(src.is_cuda and src.dtype == q.dtype and src.dim() == 2 and src.shape[0] == n == ctx.n_tokens and src.shape[1] >= kv_rank + rot_dim
-              and (n == 0 or src.stride(1) == 1), f"{what}: latents {tuple(src.shape)} {src.dtype} for {ctx.n_tokens} tokens")
-        keep = [_p(src), src.stride(0), _p(store.norm_w), float(store.eps), _p(ctx.positions), _p(ctx.tok_slot), _p(store.block_table),
-                store.block_table.shape[1], _p(store.rows_cache), _p(store.rows_t), _p(store.table_t)]
+    keep = _latent_store(what, store, q, kv_rank, rot_dim, ctx, pairing)
     qa = torch.empty((n, heads, kv_rank + rot_dim), dtype=F32, device=q.device)
+    if uk_t is not None and q.dtype == BF16 and rot_dim % 8 == 0 and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0:
+        _dev(what, uk_t)
+        _need(uk_t.shape == (heads, kv_rank, dim) and uk_t.dtype == BF16, f"{what}: transposed key matrices {tuple(uk_t.shape)} {uk_t.dtype}")
+        library.call(mixers(), "palm_latent_query_mfma", _stream(), _p(q), q.stride(0), _p(uk_t), _p(cos), _p(sin), n, heads, dim, rot_dim, kv_rank,
+                     ROTARY_PAIRINGS[pairing], _p(qa), *keep)
+        return qa
     library.call(mixers(), "palm_latent_query", _stream(), _p(q), _code(q, what), q.stride(0), _p(uk), _code(uk, what + " key matrix"), _p(cos), _p(sin),
                  n, heads, dim, rot_dim, kv_rank, ROTARY_PAIRINGS[pairing], _p(qa), *keep)
     return qa
+
+
+def _latent_store(what: str, store: LatentStore | None, q: torch.Tensor, kv_rank: int, rot_dim: int, ctx, pairing: str) -> list:
+    """The entry points' arguments for the cache rows that are written beside the queries q (none without ``store``)."""
+    if store is None:
+        return [None, 0, None, 0.0, None, None, None, 0, None, None, None]
+    src, n = store.src, q.shape[0]
+    _latent_rows(what, q.dtype, kv_rank, rot_dim, store.norm_w, store.rows_cache, store.block_table, ctx, store.rows_t, store.table_t, pairing)
+    _need(src.is_cuda and src.dtype == q.dtype and src.dim() == 2 and src.shape[0] == n == ctx.n_tokens and src.shape[1] >= kv_rank + rot_dim
+          and (n == 0 or src.stride(1) == 1), f"{what}: latents {tuple(src.shape)} {src.dtype} for {ctx.n_tokens} tokens")
+    return [_p(src), src.stride(0), _p(store.norm_w), float(store.eps), _p(ctx.positions), _p(ctx.tok_slot), _p(store.block_table),
+            store.block_table.shape[1], _p(store.rows_cache), _p(store.rows_t), _p(store.table_t)]
+
+
+# A long prompt's keys and values are expanded: two library products make every visible position's keys and values of all heads,
+# and the prompt kernel of attention with a sink runs over them.  A score then takes key_dim + rot_dim products instead of
+# kv_rank + rot_dim and a weighted sum value_dim instead of kv_rank; the expansion is what it costs.
+LATENT_EXPAND_TOKENS = 192         # new tokens of a step from which on it is considered (such steps are never recorded)
+LATENT_EXPAND_BYTES = 4 << 30      # the expanded keys and values of a step at most
+
+
+def latent_expand_plan(ctx, window: int | None):
+    """(positions to expand, in whole pages; new x visible positions over the step's sequences): what every sequence's new tokens
+    see, from the host's copy of the step."""
+    pages, pairs = 0, 0.0
+    for start, new in zip(ctx.host["starts"], ctx.host["counts"]):
+        if new <= 0:
+            continue
+        low = max(0, start - window + 1) if window else 0
+        pages += (start + new - 1) // PAGE_TOKENS - low // PAGE_TOKENS + 1
+        pairs += new * (min(start + new / 2.0, window) if window else start + new / 2.0)
+    return pages * PAGE_TOKENS, pairs
+
+
+def latent_expanded_serves(q: torch.Tensor, rows_cache: torch.Tensor, uk: torch.Tensor, uv: torch.Tensor, ctx, heads: int, dim: int, rot_dim: int,
+                           kv_rank: int, vdim: int, window: int | None) -> bool:
+    """Whether a prompt's keys and values are expanded: bfloat16, sizes in steps of eight that the prompt kernel of attention
+    with a sink takes, and enough new tokens for the positions that they see."""
+    if ctx.is_decode or ctx.n_tokens < LATENT_EXPAND_TOKENS or q.dtype != BF16 or rows_cache.dtype != BF16 or uk.dtype != BF16 or uv.dtype != BF16:
+        return False
+    if dim % 8 or rot_dim % 8 or kv_rank % 8 or vdim % 8 or dim + rot_dim > 256 or vdim > 256 or q.stride(0) % 8 or q.data_ptr() % 16:
+        return False
+    positions, pairs = latent_expand_plan(ctx, window)
+    saved = 2 * kv_rank + rot_dim - (dim + rot_dim + vdim)
+    # (a multiply-add of the library's products takes about a quarter of the time that one of the attention takes)
+    return (pairs * saved > 0.25 * positions * kv_rank * (dim + vdim)
+            and 2 * positions * (heads * (dim + vdim) + kv_rank + rot_dim) <= LATENT_EXPAND_BYTES and positions * vdim < 1 << 31)
+
+
+def latent_attention_expanded(q: torch.Tensor, uk: torch.Tensor, uv: torch.Tensor, cos, sin, heads: int, dim: int, rot_dim: int, kv_rank: int,
+                              vdim: int, pairing: str, ctx, store: LatentStore | None, rows_cache: torch.Tensor, block_table: torch.Tensor,
+                              scale: float, window: int | None, sink: torch.Tensor | None, gate: torch.Tensor | None) -> torch.Tensor:
+    """Attention of a prompt's queries q [n, heads * (dim + rot_dim)] (not rotated yet; a view of wider rows is fine) with keys and
+    values made from the cached rows for every position that they see; ``store`` (what the step's tokens keep) is written first.
+    bfloat16 [n, heads * vdim]."""
+    what = "latent_attention_expanded"
+    _dev(what, uk, uv, rows_cache, block_table, ctx.seq_slot, ctx.seq_start, ctx.seq_new, ctx.cu_new)
+    _i32(what, block_table, ctx.seq_slot, ctx.seq_start, ctx.seq_new, ctx.cu_new)
+    n = q.shape[0]
+    _need(latent_expanded_serves(q, rows_cache, uk, uv, ctx, heads, dim, rot_dim, kv_rank, vdim, window), f"{what}: a long prompt in bfloat16 with "
+          "sizes the kernels take")
+    _need(q.is_cuda and q.shape == (ctx.n_tokens, heads * (dim + rot_dim)) and q.stride(1) == 1, f"{what}: queries {tuple(q.shape)}")
+    _need(uk.shape == (heads * dim, kv_rank) and uv.shape == (heads * vdim, kv_rank), f"{what}: matrices {tuple(uk.shape)}, {tuple(uv.shape)}")
+    _need(rows_cache.dim() == 3 and rows_cache.shape[1:] == (PAGE_TOKENS, kv_rank + rot_dim) and block_table.dim() == 2,
+          f"{what}: the cache {tuple(rows_cache.shape)}, page table {tuple(block_table.shape)}")
+    _need(gate is None or (gate.is_cuda and gate.shape == (n, heads) and gate.dtype == BF16 and gate.stride(1) == 1),
+          f"{what}: the gate is bfloat16 [{n}, {heads}] with contiguous rows")
+    _latent_sink(what, sink, heads)
+    _latent_rotation(what, cos, sin, n, rot_dim)
+    key = ("latent_pages", window)
+    if key not in ctx.memo:                     # which pages of which sequence are gathered, and where a sequence's page 0 would lie
+        seq_of, page_of, page0 = [], [], []
+        for b, (start, new) in enumerate(zip(ctx.host["starts"], ctx.host["counts"])):
+            first = max(0, start - window + 1) // PAGE_TOKENS if window else 0
+            last = (start + new - 1) // PAGE_TOKENS if new > 0 else first - 1
+            page0.append(len(seq_of) - first)
+            seq_of += [b] * (last - first + 1)
+            page_of += range(first, last + 1)
+        flat = torch.tensor(page0 + seq_of + page_of, dtype=torch.int32).to(q.device)
+        B, N = len(page0), len(seq_of)
+        ctx.memo[key] = (flat[:B], flat[B:B + N], flat[B + N:], N)
+    page0, seq_of, page_of, n_pages = ctx.memo[key]
+    positions = n_pages * PAGE_TOKENS
+    turned = torch.empty((n, heads, dim + rot_dim), dtype=BF16, device=q.device)
+    library.call(mixers(), "palm_latent_turn", _stream(), _p(q), _CODES[BF16], q.stride(0), _p(cos), _p(sin), n, heads, dim, rot_dim, kv_rank,
+                 ROTARY_PAIRINGS[pairing], _p(turned), *_latent_store(what, store, q, kv_rank, rot_dim, ctx, pairing))
+    c = torch.empty((positions, kv_rank), dtype=BF16, device=q.device)
+    k2 = torch.empty((positions, rot_dim), dtype=BF16, device=q.device)
+    library.call(mixers(), "palm_latent_gather", _stream(), _p(rows_cache), _CODES[BF16], _p(block_table), block_table.shape[1], _p(ctx.seq_slot),
+                 _p(ctx.seq_start), _p(ctx.seq_new), _p(seq_of), _p(page_of), n_pages, kv_rank, rot_dim, _p(c), _p(k2))
+    keys = linear_library(c, uk)                 # [positions, heads * dim]
+    values = linear_library(uv, c)               # [heads * vdim, positions]: positions innermost, as the kernel reads values
+    out = torch.empty((n, heads * vdim), dtype=BF16, device=q.device)
+    library.call(sink_attention_mfma_lib(dim + rot_dim, vdim), "palm_sink_attention_rows_mfma", _stream(), _p(turned), _p(keys), _p(k2) if rot_dim else None,
+                 _p(values), dim, positions, _p(page0), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs, int(ctx.max_new), heads,
+                 dim + rot_dim, vdim, float(scale), int(window or 0), _p(sink), _p(gate), gate.stride(0) if gate is not None else 0, _p(out))
+    return out
 
 
 _LATENT_MFMA_SIGNATURE = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
@@ -1952,6 +2063,8 @@ def _sink_slopes(what: str, slopes, heads: int, window, chunked: bool) -> None:
 
 _SINK_MFMA_SIGNATURE = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
                         c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_void_p]
+_SINK_ROWS_SIGNATURE = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                        c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_int, c_void_p]
 _sink_mfma_libs: dict = {}
 
 
@@ -1967,6 +2080,7 @@ def sink_attention_mfma_lib(dim: int, vdim: int):
     if lib is None:
         lib = library.load(f"sink_attention_k{key[0]}_v{key[1]}")
         lib.palm_sink_attention_mfma.argtypes, lib.palm_sink_attention_mfma.restype = _SINK_MFMA_SIGNATURE, c_int
+        lib.palm_sink_attention_rows_mfma.argtypes, lib.palm_sink_attention_rows_mfma.restype = _SINK_ROWS_SIGNATURE, c_int
         _sink_mfma_libs[key] = lib
     return lib
 

@@ -12,7 +12,8 @@ are a_h . c_j + q_rot . r_j, the weighted sum is taken over the rows c_j, and U_
 the same rows.  The rotation's angles and the scores, weights and sums are 32-bit.  In the bfloat16 mode the cache keeps the
 latents a second time with the positions innermost, which is how the kernels on the matrix cores read them (prompts, and
 single tokens with their key range in slices); the float32 mode and sizes those do not take go through the exact kernel, which
-reads the rows alone.
+reads the rows alone.  A long prompt is the exception: there the keys and values of every visible position are expanded by two
+products (a score then takes key_dim + rot_dim multiply-adds instead of kv_rank + rot_dim), where that pays.
 
 Options: without ``q_rank`` the joined product makes the queries themselves (q = W_q h, no latent, no norm; tensor ``down``: q
 | latent and key part | gates).  ``sink`` "learned": head h's softmax has one more term exp(sink_h) in its denominator (tensor
@@ -73,6 +74,7 @@ class LatentAttention:
         if self.position is not None and self.position.rotary_dim != self.dr:
             raise ValueError("latent attention: the rotation covers the whole rotated part")
         self.pairing = self.position.pairing if self.position is not None else "half_split"
+        self.uk_t = ops.latent_key_transposes(self.uk, self.nh, self.dk, self.kv_rank)
         self.dtype = builder.dtype
 
     @staticmethod
@@ -110,12 +112,16 @@ class LatentAttention:
         if self.q_rank:
             cq = ops.latent_prep(down, self.q_rank, self.kv_off, self.kv_rank, self.dr, self.q_norm_w, self.kv_norm_w, self.eps, cos, sin,
                                  view.data, view.table_dev, ctx, write_cache=lc.writes, rows_t=rows_t, table_t=table_t, pairing=self.pairing)
-            qa = ops.latent_query(self.uq(cq), self.uk, cos, sin, *sizes, pairing=self.pairing)
+            q, store = self.uq(cq), None
         else:
             store = None if not lc.writes else ops.LatentStore(down[:, self.kv_off:self.gate_off], self.kv_norm_w, self.eps, view.data,
                                                               view.table_dev, rows_t, table_t)
-            qa = ops.latent_query(down[:, :self.kv_off], self.uk, cos, sin, *sizes, pairing=self.pairing, ctx=ctx, store=store)
+            q = down[:, :self.kv_off]
         gate = down[:, self.gate_off:] if self.gated else None
+        if ops.latent_expanded_serves(q, view.data, self.uk, self.uv, ctx, *sizes, self.dv, self.window):
+            return self.out(ops.latent_attention_expanded(q, self.uk, self.uv, cos, sin, *sizes, self.dv, self.pairing, ctx, store, view.data,
+                                                          view.table_dev, self.scale, self.window, self.sink, gate))
+        qa = ops.latent_query(q, self.uk, cos, sin, *sizes, pairing=self.pairing, ctx=ctx, store=store, uk_t=self.uk_t)
         attend = (qa, view.data, view.table_dev, ctx, self.nh, self.kv_rank, self.dr, self.scale, self.window)
         # on the matrix cores the value matrices and the gates ride in the attention's own launches
         if ops.latent_decode_serves(view.data, rows_t, self.uv, ctx, self.kv_rank, self.dr):

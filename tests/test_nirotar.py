@@ -458,8 +458,81 @@ def test_latent_attention_far_keys_page_borders_window_edges_and_sinks(dtype, he
 
 
 @gpu
+@pytest.mark.parametrize("heads,d,dr,dv,R,window", [(3, 16, 8, 24, 64, None), (5, 64, 32, 128, 256, None), (2, 32, 16, 40, 96, 70), (1, 128, 64, 128, 512, None), (4, 24, 8, 72, 136, 64)])
+def test_latent_attention_with_expanded_keys_and_values(heads, d, dr, dv, R, window):
+    """A prompt's portions of three sequences (one from its start, two further on) over cached rows in scrambled pages, NaN wherever
+    a page belongs to nobody; the queries come unrotated as columns of a wider product.  For chosen queries one position's key
+    stands out: the first ones, a page's borders, a window's edges, the query's own.  One head's sink outweighs every key."""
+    from palm_infra_amd.kernels import ops
+    g = torch.Generator().manual_seed(R + d)
+    bf, dk, scale = torch.bfloat16, R + dr, 0.4
+    lens, counts = [330, 100, 290], [150, 100, 70]
+    starts = [ln - c for ln, c in zip(lens, counts)]
+    n = sum(counts)
+    sinks = torch.randn(heads, generator=g)
+    if heads > 1:
+        sinks[heads - 1] = 90.0
+    uk, uv = (torch.randn(heads * d, R, generator=g) * R ** -0.5).to(bf), (torch.randn(heads * dv, R, generator=g) * R ** -0.5).to(bf)
+    rot = {"dims": dr, "base": 40.0}
+    q = torch.randn(n, heads * (d + dr) + 24, generator=g) * 0.3
+    rows = [(torch.randn(ln, dk, generator=g) * 0.5).to(bf) for ln in lens]
+    w = window or 10 ** 9
+    at = 0
+    for b, (s, c) in enumerate(zip(starts, counts)):
+        for i in range(0, c, 9):
+            pos = s + i
+            key = [0, 1, pos // 64 * 64 - 1, pos // 64 * 64, max(0, pos - w + 1), pos - w, pos][i // 9 % 7]
+            if 0 <= key <= pos:
+                r = rows[b][key].double()
+                for h in range(heads):                              # the query points along that position's unrotated key
+                    k = uk[h * d:(h + 1) * d].double() @ r[:R]
+                    q[at + i, h * (d + dr):h * (d + dr) + d] = (k / k.norm() ** 2 * 30.0 / scale).float()
+        at += c
+    q = q.to(bf)
+    pages_of = [[7, 6, 5, 4, 3, 2], [9, 12], [8, 10, 0, 13, 11]]
+    cache = torch.full((16, 64, dk), float("nan"), dtype=bf)
+    table = torch.full((4, 8), 15, dtype=torch.int32)
+    for b in range(3):
+        table[b + 1, :len(pages_of[b])] = torch.tensor(pages_of[b], dtype=torch.int32)
+        for j in range(lens[b]):
+            if window is None or j // 64 >= max(0, starts[b] - window + 1) // 64:              # (pages that no query sees may be gone)
+                cache[pages_of[b][j // 64], j % 64] = rows[b][j]
+    ctx = _step_context(starts, counts, slots=[1, 2, 3])
+    ang = ctx.positions.cpu().double()[:, None] * P.frequencies(rot)
+    cos, sin = torch.cos(ang).float().cuda(), torch.sin(ang).float().cuda()
+    gate = torch.randn(n, heads + 5, generator=g).to(bf)
+    want, at = [], 0
+    for b, (s, c) in enumerate(zip(starts, counts)):
+        r = rows[b].double()
+        qs = torch.zeros(lens[b], heads, d + dr, dtype=P.F64)
+        qs[s:] = q[at:at + c, :heads * (d + dr)].double().reshape(c, heads, d + dr)
+        qt = P.rotate_pairs(qs[..., d:], rot)
+        kp, v = (r[:, :R] @ uk.double().T).reshape(-1, heads, d), (r[:, :R] @ uv.double().T).reshape(-1, heads, dv)
+        scores = torch.stack([(qs[:, h, :d] @ kp[:, h].T + qt[:, h] @ r[:, R:].T) * scale for h in range(heads)])
+        p = P.sink_softmax_heads(scores, sinks.double(), window)
+        want.append(torch.stack([p[h] @ v[:, h] for h in range(heads)], 1)[s:])
+        at += c
+    want = torch.cat(want)
+    qc = q.cuda()[:, :heads * (d + dr)]
+    serves = ops.latent_expanded_serves(qc, cache.cuda(), uk.cuda(), uv.cuda(), ctx, heads, d, dr, R, dv, window)
+    assert serves or R < 100                                          # (a small latent: it may not pay, which the next line overrides)
+    plan, ops.latent_expand_plan = ops.latent_expand_plan, lambda ctx, window: (64, 1e12)
+    try:
+        args = (qc, uk.cuda(), uv.cuda(), cos, sin, heads, d, dr, R, dv, "interleaved", ctx, None, cache.cuda(), table.cuda(), scale, window, sinks.cuda())
+        got = ops.latent_attention_expanded(*args, None).double().cpu().reshape(n, heads, dv)
+        assert torch.isfinite(got).all()
+        assert torch.allclose(got, want, atol=4e-2, rtol=4e-2), float((got - want).abs().max())
+        gated = ops.latent_attention_expanded(*args, gate.cuda()[:, 5:]).double().cpu().reshape(n, heads, dv)
+        assert torch.allclose(gated, want * torch.sigmoid(gate.double()[:, 5:, None]), atol=4e-2, rtol=4e-2)
+    finally:
+        ops.latent_expand_plan = plan
+    if heads > 1:
+        assert float(want[:, heads - 1].abs().max()) < 1e-2
+
+
+@gpu
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,d,dr,R", [(3, 12, 6, 24), (1, 40, 2, 70), (20, 16, 8, 130)])
+@pytest.mark.parametrize("H,d,dr,R", [(3, 12, 6, 24), (1, 40, 2, 70), (20, 16, 8, 136), (3, 72, 24, 56)])
 def test_direct_queries_through_the_key_matrix_and_cache_rows_in_one_launch(dtype, H, d, dr, R):
     """Queries as columns of a wider product, neighbouring pairs turned, the latent normed and written to its page and to the
     transposed copy's page; a part that reads another's rows writes none."""
@@ -469,6 +542,7 @@ def test_direct_queries_through_the_key_matrix_and_cache_rows_in_one_launch(dtyp
     g = torch.Generator().manual_seed(R)
     n, q_size = 11, H * (d + dr)
     ctx = _step_context([60, 0], [8, 3], slots=[0, 1])
+    assert (ops.latent_key_transposes(torch.zeros(H * d, R, dtype=td), H, d, R) is not None) == (dtype == "bfloat16" and d % 8 == R % 8 == 0)
     down = torch.randn(n, q_size + R + dr, generator=g).to(td)
     wk = 1 + 0.2 * torch.randn(R, generator=g)
     uk = (torch.randn(H * d, R, generator=g) * 0.3).to(td)
@@ -494,8 +568,11 @@ def test_direct_queries_through_the_key_matrix_and_cache_rows_in_one_launch(dtyp
         cache = torch.zeros((4, 64, R + dr), dtype=td, device="cuda")
         turned = torch.zeros((4, R, 64), dtype=torch.bfloat16, device="cuda")
         store = ops.LatentStore(dc[:, q_size:], wk.cuda(), 1e-5, cache, table, turned, table_t) if writes else None
-        qa = ops.latent_query(dc[:, :q_size], uk.cuda(), cos, sin, H, d, dr, R, pairing="interleaved", ctx=ctx, store=store).double().cpu()
+        qa = ops.latent_query(dc[:, :q_size], uk.cuda(), cos, sin, H, d, dr, R, pairing="interleaved", ctx=ctx, store=store,
+                              uk_t=ops.latent_key_transposes(uk.cuda(), H, d, R)).double().cpu()
         assert torch.allclose(qa, want_qa, **tol)
+        plain = ops.latent_query(dc[:, :q_size], uk.cuda(), cos, sin, H, d, dr, R, pairing="interleaved").double().cpu()
+        assert torch.allclose(plain, want_qa, **tol)
         where = [(1, 60 + i - 64) if 60 + i >= 64 else (2, 60 + i) for i in range(8)] + [(0, i) for i in range(3)]
         where_t = [(3, 60 + i - 64) if 60 + i >= 64 else (1, 60 + i) for i in range(8)] + [(2, i) for i in range(3)]
         if not writes:
