@@ -2,8 +2,8 @@
 // matrices read once, whatever the number of rows that chose it; nothing is planned on the host and no launch of its own plans.
 //
 //   up     a block per (expert, run of matrix rows): the block finds the rows that chose its expert (none: it is done), and
-//          each wave streams 16 rows of the expert's first matrix (gated forms: 16 gate rows and their 16 up rows) past them, 16
-//          rows of activations a column tile; mid[t, c, f] = act(..) in bfloat16, t's choices one after the other, the shared
+//          two waves, half the inner size each, stream 16 rows of the expert's first matrix (gated forms: 16 gate rows and their
+//          16 up rows) past them, 16 rows of activations a column tile, and add their sums through LDS; mid[t, c, f] = act(..) in bfloat16, t's choices one after the other, the shared
 //          expert's values behind them
 //   down   a block per (16 output features, plane): all (row, choice) pairs are sorted by expert in LDS; pieces of 256 inner
 //          values of the experts in use are dealt to the planes' waves in turn; a piece's products go, weighted, into the wave's
@@ -15,7 +15,7 @@
 #include "expert_form.h"
 
 constexpr int FEW_ROWS = 128;                     // rows of a step at most
-constexpr int FEW_UP_WAVES = 4;
+constexpr int FEW_UP_WAVES = 4;                   // runs of 16 matrix rows a block, two waves each
 constexpr int FEW_DOWN_WAVES = 8;
 constexpr int FEW_PIECE = 256;                    // inner values of a piece
 constexpr int FEW_STEPS = 8;                      // reads of 32 values of every matrix row under way together
@@ -77,7 +77,7 @@ __device__ inline void few_products(const bf16_t* const (&wr)[MATS], const bf16_
 template <bool GATED, int CT>
 __device__ inline void few_up_tile(const bf16_t* __restrict__ h, const bf16_t* __restrict__ w, const int* list, int c0, int m, bool is_shared,
                                    const FewChoices& ch, int width, int ff, int my_ff, int row_ff, int f0, int r, int g, int form,
-                                   const ExpertCap& cap, bf16_t* __restrict__ mid) {
+                                   const ExpertCap& cap, int part, f32x4* exchange, bf16_t* __restrict__ mid) {
     const bf16_t* xr[CT];
     const bf16_t* wr[GATED ? 2 : 1];
 #pragma unroll
@@ -92,7 +92,26 @@ __device__ inline void few_up_tile(const bf16_t* __restrict__ h, const bf16_t* _
     for (int i = 0; i < (GATED ? 2 : 1); ++i)
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) acc[i][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
-    few_products<GATED ? 2 : 1, CT>(wr, xr, 0, width, g, acc);
+    const int middle = (width / 2 + 31) / 32 * 32;
+    if (part == 0) few_products<GATED ? 2 : 1, CT>(wr, xr, 0, min(middle, width), g, acc);
+    else if (middle < width) few_products<GATED ? 2 : 1, CT>(wr, xr, middle, width, g, acc);
+    __syncthreads();                                                  // (whoever still reads the exchange is done)
+    if (part == 1) {
+#pragma unroll
+        for (int i = 0; i < (GATED ? 2 : 1); ++i)
+#pragma unroll
+            for (int ct = 0; ct < CT; ++ct) exchange[(i * CT + ct) * WAVE + 16 * g + r] = acc[i][ct];
+    }
+    __syncthreads();
+    if (part == 1) return;
+#pragma unroll
+    for (int i = 0; i < (GATED ? 2 : 1); ++i)
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct) {
+            const f32x4 other = exchange[(i * CT + ct) * WAVE + 16 * g + r];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) acc[i][ct][k] += other[k];
+        }
     // lane (r, g) holds inner values f0 + 4 g + i of column r
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
@@ -111,11 +130,12 @@ __device__ inline void few_up_tile(const bf16_t* __restrict__ h, const bf16_t* _
 }
 
 template <bool GATED>
-__global__ __launch_bounds__(FEW_UP_WAVES * WAVE) void moe_few_up_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ up, FewChoices ch,
+__global__ __launch_bounds__(2 * FEW_UP_WAVES * WAVE) void moe_few_up_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ up, FewChoices ch,
                                                                          int experts, int width, int ff, const bf16_t* __restrict__ shared_up,
                                                                          int shared_ff, int form, ExpertCap cap, bf16_t* __restrict__ mid) {
     __shared__ int list_s[FEW_MAX_PAIRS];
     __shared__ int count_s;
+    __shared__ f32x4 exchange_s[FEW_UP_WAVES][(GATED ? 2 : 1) * 4 * WAVE];
     const int e = blockIdx.x;
     const bool is_shared = e == experts;
     const int my_ff = is_shared ? shared_ff : ff, row_ff = ch.top * ff + shared_ff;
@@ -132,13 +152,13 @@ __global__ __launch_bounds__(FEW_UP_WAVES * WAVE) void moe_few_up_kernel(const b
     }
     __syncthreads();
     const int m = count_s;
-    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
-    const int r = lane % 16, g = lane / 16, f0 = block_f + 16 * wave;
-    if (m == 0 || f0 >= my_ff) return;
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE % FEW_UP_WAVES, part = threadIdx.x / WAVE / FEW_UP_WAVES;
+    const int r = lane % 16, g = lane / 16, f0 = block_f + 16 * wave;   // (rows beyond the matrix: its last one again, not kept)
+    if (m == 0) return;
     const bf16_t* w = is_shared ? shared_up : up + (size_t)e * (GATED ? 2 : 1) * ff * width;
     for (int c0 = 0; c0 < m;) {
         const int left = m - c0;
-#define FEW_UP(CT) { few_up_tile<GATED, CT>(h, w, list_s, c0, m, is_shared, ch, width, ff, my_ff, row_ff, f0, r, g, form, cap, mid); c0 += 16 * CT; }
+#define FEW_UP(CT) { few_up_tile<GATED, CT>(h, w, list_s, c0, m, is_shared, ch, width, ff, my_ff, row_ff, f0, r, g, form, cap, part, exchange_s[wave], mid); c0 += 16 * CT; }
         if (left > 32) FEW_UP(4) else if (left > 16) FEW_UP(2) else FEW_UP(1)
 #undef FEW_UP
     }
@@ -287,7 +307,7 @@ PALM_API int palm_moe_few(hipStream_t stream, const void* h, const void* up, con
     const int longest = max(ff, shared_ff), runs = (longest + 16 * FEW_UP_WAVES - 1) / (16 * FEW_UP_WAVES);
     PALM_CHECK(runs <= 65535, "moe_few: an inner size of %d is more than one launch takes", longest);
     const dim3 grid(experts + (shared_ff > 0), runs);
-#define FEW_LAUNCH(GATED) moe_few_up_kernel<GATED><<<grid, FEW_UP_WAVES * WAVE, 0, stream>>>((const bf16_t*)h, (const bf16_t*)up, ch, experts, width, ff, \
+#define FEW_LAUNCH(GATED) moe_few_up_kernel<GATED><<<grid, 2 * FEW_UP_WAVES * WAVE, 0, stream>>>((const bf16_t*)h, (const bf16_t*)up, ch, experts, width, ff, \
         (const bf16_t*)shared_up, shared_ff, form, cap, (bf16_t*)mid)
     if (expert_is_gated(form)) FEW_LAUNCH(true); else FEW_LAUNCH(false);
 #undef FEW_LAUNCH

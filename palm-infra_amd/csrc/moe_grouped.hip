@@ -2,8 +2,8 @@
 // grouped products on the matrix cores run all experts' rows in one launch each.
 //
 //   plan      count the pairs of every expert; pad every expert's run of pairs to whole tiles of rows and lay the
-//             runs one after the other; place every pair in its run in the order of the pairs (token, then choice), so that
-//             nothing depends on the order in which threads arrive; the slots that pad a run hold -1
+//             runs one after the other; place every pair in its run, in no particular order (a slot is a column of the
+//             products by itself: no result depends on where in its run a pair lies); the slots that pad a run hold -1
 //   grouped   for every tile (its expert comes from the plan): mid = silu(G_e x) * (U_e x) for the tile's rows x, then
 //             y = D_e mid.  The weights are the first operand of the matrix instruction, so that a lane ends with four
 //             neighbouring features of one row.  Sizes in whole cache lines with enough rows an expert: blocks of 128 rows x 256
@@ -19,7 +19,8 @@ constexpr int GT_TOKENS = 64;                     // rows of a tile whose fragme
 constexpr int GT_RUNS = GT_TOKENS / 16;           // runs of 16 rows: what one matrix instruction takes
 constexpr int GT_WAVES = 4;
 constexpr int GT_FEATURES = 32 * GT_WAVES;        // features of a block's tile
-constexpr int PLAN_THREADS = 256;
+constexpr int PLAN_THREADS = 1024;
+constexpr int PLAN_MAX_EXPERTS = 512;
 
 __device__ inline bf16x8 grouped_row8(const bf16_t* row, int col, int dim) {
     // eight values of a row from column `col`; columns beyond `dim` are zero (dim is a multiple of eight); the read itself
@@ -28,72 +29,60 @@ __device__ inline bf16x8 grouped_row8(const bf16_t* row, int col, int dim) {
     return col < dim ? v : zero_bf16x8();
 }
 
-// One block per expert: counts[e] = pairs that chose e.
-__global__ __launch_bounds__(PLAN_THREADS) void moe_count_kernel(const int* __restrict__ chosen, int n_pairs, int* __restrict__ counts) {
-    __shared__ int part[PLAN_THREADS / WAVE];
-    const int e = blockIdx.x;
-    int mine = 0;
-    for (int p = threadIdx.x; p < n_pairs; p += PLAN_THREADS) mine += chosen[p] == e;
-#pragma unroll
-    for (int off = WAVE / 2; off > 0; off >>= 1) mine += __shfl_xor(mine, off, WAVE);
-    if (threadIdx.x % WAVE == 0) part[threadIdx.x / WAVE] = mine;
+// One block.  starts[e] = first slot of expert e's run (runs padded to whole tiles); tile_expert[i] = the expert of tile i, -1 beyond
+// the last tile; slot_pair[slot] = pair (-1 where a run is padded), pair_slot[pair] = slot.  The choices are rows [n, top], or with
+// ids the rows of a table [vocab, top] that the tokens' ids pick.
+__global__ __launch_bounds__(PLAN_THREADS) void moe_plan_kernel(const int* __restrict__ chosen, const int* __restrict__ ids, int vocab, int top,
+                                                                int n_pairs, int experts, int max_tiles, int tile,
+                                                                int* __restrict__ tile_expert, int* __restrict__ slot_pair,
+                                                                int* __restrict__ pair_slot) {
+    __shared__ int start_s[PLAN_MAX_EXPERTS + 1], cursor_s[PLAN_MAX_EXPERTS];
+    const int lane = threadIdx.x % WAVE;
+    auto choice = [&](int p) { return ids ? chosen[(size_t)min(max(ids[p / top], 0), vocab - 1) * top + p % top] : chosen[p]; };
+    for (int e = threadIdx.x; e < experts; e += PLAN_THREADS) cursor_s[e] = 0;
     __syncthreads();
-    if (threadIdx.x == 0) {
-        int total = 0;
-        for (int w = 0; w < PLAN_THREADS / WAVE; ++w) total += part[w];
-        counts[e] = total;
-    }
-}
-
-// One block: starts[e] = first slot of expert e's run (runs padded to whole tiles), starts[experts] = slots in all;
-// tile_expert[i] = the expert of tile i, -1 beyond the last tile.
-__global__ __launch_bounds__(PLAN_THREADS) void moe_runs_kernel(const int* __restrict__ counts, int experts, int max_tiles, int tile,
-                                                                int* __restrict__ starts, int* __restrict__ tile_expert) {
-    if (threadIdx.x == 0) {
-        int at = 0;
-        for (int e = 0; e < experts; ++e) {
-            starts[e] = at;
-            at += (counts[e] + tile - 1) / tile * tile;
+    for (int p = threadIdx.x; p < n_pairs; p += PLAN_THREADS) atomicAdd(&cursor_s[choice(p)], 1);
+    __syncthreads();
+    if (threadIdx.x < WAVE) {
+        constexpr int PER = PLAN_MAX_EXPERTS / WAVE;
+        int padded[PER], mine = 0;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const int e = lane * PER + i;
+            padded[i] = e < experts ? (cursor_s[e] + tile - 1) / tile * tile : 0;
+            mine += padded[i];
         }
-        starts[experts] = at;
+        int up_to = mine;                                             // the sum over the lanes up to this one
+#pragma unroll
+        for (int off = 1; off < WAVE; off <<= 1) {
+            const int other = __shfl_up(up_to, off, WAVE);
+            if (lane >= off) up_to += other;
+        }
+        int at = up_to - mine;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const int e = lane * PER + i;
+            if (e < experts) start_s[e] = at;
+            at += padded[i];
+        }
+        if (lane == WAVE - 1) start_s[experts] = up_to;
     }
     __syncthreads();
     for (int i = threadIdx.x; i < max_tiles; i += PLAN_THREADS) tile_expert[i] = -1;
+    // the slots that pad each run
+    for (int e = threadIdx.x / WAVE; e < experts; e += PLAN_THREADS / WAVE)
+        for (int s = start_s[e] + cursor_s[e] + lane; s < start_s[e + 1]; s += WAVE) slot_pair[s] = -1;
     __syncthreads();
-    for (int e = threadIdx.x; e < experts; e += PLAN_THREADS)
-        for (int i = starts[e] / tile; i < starts[e + 1] / tile; ++i) tile_expert[i] = e;
-}
-
-// One block per expert: its pairs into its run, in the order of the pairs.  slot_pair[slot] = pair (or -1), pair_slot[pair] = slot.
-__global__ __launch_bounds__(PLAN_THREADS) void moe_place_kernel(const int* __restrict__ chosen, int n_pairs, const int* __restrict__ starts,
-                                                                 int* __restrict__ slot_pair, int* __restrict__ pair_slot) {
-    __shared__ int wave_count[PLAN_THREADS / WAVE];
-    __shared__ int base_s;
-    const int e = blockIdx.x, lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
-    if (threadIdx.x == 0) base_s = starts[e];
-    __syncthreads();
-    for (int p0 = 0; p0 < n_pairs; p0 += PLAN_THREADS) {
-        const int p = p0 + threadIdx.x;
-        const bool mine = p < n_pairs && chosen[p] == e;
-        const unsigned long long votes = __ballot(mine);
-        const int before = __popcll(votes & ((1ull << lane) - 1ull));
-        if (lane == 0) wave_count[wave] = __popcll(votes);
-        __syncthreads();
-        int base = base_s;
-        for (int w = 0; w < wave; ++w) base += wave_count[w];
-        if (mine) {
-            slot_pair[base + before] = p;
-            pair_slot[p] = base + before;
-        }
-        __syncthreads();
-        if (threadIdx.x == 0) {
-            int total = 0;
-            for (int w = 0; w < PLAN_THREADS / WAVE; ++w) total += wave_count[w];
-            base_s += total;
-        }
-        __syncthreads();
+    for (int e = threadIdx.x; e < experts; e += PLAN_THREADS) {
+        for (int i = start_s[e] / tile; i < start_s[e + 1] / tile; ++i) tile_expert[i] = e;
+        cursor_s[e] = start_s[e];
     }
-    for (int s = base_s + threadIdx.x; s < starts[e + 1]; s += PLAN_THREADS) slot_pair[s] = -1;
+    __syncthreads();
+    for (int p = threadIdx.x; p < n_pairs; p += PLAN_THREADS) {
+        const int slot = atomicAdd(&cursor_s[choice(p)], 1);
+        slot_pair[slot] = p;
+        pair_slot[p] = slot;
+    }
 }
 
 // grid (tiles, blocks of GT_FEATURES features).  a: the rows [*, k_dim]; row_of_slot: null (the rows lie in slot order) or
@@ -308,16 +297,26 @@ __global__ __launch_bounds__(TILE_WAVES * WAVE) void moe_tile_kernel(const bf16_
     }
 }
 
-// One block per token.
+// One block per token; eight neighbouring columns a thread (width is a multiple of eight).  weight: null, or [n, top] (null: 1 / top).
 __global__ void moe_combine_kernel(const bf16_t* __restrict__ y, const int* __restrict__ pair_slot, const float* __restrict__ weight, int top,
                                    int width, const bf16_t* __restrict__ add0, const bf16_t* __restrict__ add1, float* __restrict__ out) {
     const size_t t = blockIdx.x;
-    for (int d = threadIdx.x; d < width; d += blockDim.x) {
-        float total = 0.f;
-        for (int c = 0; c < top; ++c) total = fmaf(weight[t * top + c], to_float(y[(size_t)pair_slot[t * top + c] * width + d]), total);
-        if (add0) total += to_float(add0[t * width + d]);
-        if (add1) total += to_float(add1[t * width + d]);
-        out[t * width + d] = total;
+    for (int d = threadIdx.x * 8; d < width; d += blockDim.x * 8) {
+        float total[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) total[i] = 0.f;
+        auto add = [&](const bf16_t* row, float f) {
+            const bf16x8 v = load_bf16x8(row + d);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) total[i] = fmaf(f, (float)v[i], total[i]);
+        };
+#pragma unroll 4
+        for (int c = 0; c < top; ++c)
+            add(y + (size_t)pair_slot[t * top + c] * width, weight ? weight[t * top + c] : 1.0f / (float)top);
+        if (add0) add(add0 + t * width, 1.0f);
+        if (add1) add(add1 + t * width, 1.0f);
+        *reinterpret_cast<float4*>(out + t * width + d) = make_float4(total[0], total[1], total[2], total[3]);
+        *reinterpret_cast<float4*>(out + t * width + d + 4) = make_float4(total[4], total[5], total[6], total[7]);
     }
 }
 
@@ -329,11 +328,15 @@ PALM_API int palm_moe_tile_tokens(int n_pairs, int experts, int width, int ff) {
 
 // chosen, weight [n, top]; h bfloat16 [n, width]; gate_up bfloat16 [experts, 2 ff, width] (the plain forms: [experts, ff, width], up
 // rows alone); add0, add1: null or bfloat16 rows [n, width]; down bfloat16 [experts, width, ff].
-// Room, with tile = palm_moe_tile_tokens(n top, experts, width, ff), max_tiles = ceil(n top / tile) + experts and slots = max_tiles * tile: plan: (2 experts + 1 + max_tiles + slots
+// With ids [n] chosen is a table [vocab, top] of which every token takes its id's row, and weight may be null (1 / top).
+// Room, with tile = palm_moe_tile_tokens(n top, experts, width, ff), max_tiles = ceil(n top / tile) + experts and slots = max_tiles * tile: plan: (max_tiles + slots
 // + n top) ints; mid: slots * ff bfloat16; y: slots * width bfloat16.  out float32 [n, width].
 PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gate_up, const void* down, const int* chosen,
                               const float* weight, int n_tokens, int top, int experts, int width, int ff, int* plan, void* mid, void* y,
-                              float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1) {
+                              float* out, int form, float limit, float slope, float shift, const void* add0, const void* add1,
+                              const int* ids, int vocab) {
+    PALM_CHECK(ids ? vocab > 0 : weight != nullptr, "moe_grouped: choices come with weights, or from a table of %d ids", vocab);
+    PALM_CHECK(experts <= PLAN_MAX_EXPERTS, "moe_grouped: %d experts exceed %d", experts, PLAN_MAX_EXPERTS);
     PALM_CHECK(form >= EXPERT_GATED_SILU && form <= EXPERT_RELU_SQUARED, "moe_grouped: form %d is neither gated silu (0) nor plain gelu (1) nor capped "
                "gated (2) nor squared relu (3)", form);
     PALM_CHECK(form != EXPERT_CAPPED || limit > 0.f, "moe_grouped: the cap %g must be positive", (double)limit);
@@ -345,14 +348,11 @@ PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gat
     PALM_CHECK(n_pairs < (1ll << 30), "moe_grouped: %lld pairs are more than one launch takes", n_pairs);
     const int tile = tile_of(n_pairs, experts, width, ff);
     const int max_tiles = (int)((n_pairs + tile - 1) / tile) + experts;
-    int* counts = plan;
-    int* starts = counts + experts;
-    int* tile_expert = starts + experts + 1;
+    int* tile_expert = plan;
     int* slot_pair = tile_expert + max_tiles;
     int* pair_slot = slot_pair + (size_t)max_tiles * tile;
-    moe_count_kernel<<<experts, PLAN_THREADS, 0, stream>>>(chosen, (int)n_pairs, counts);
-    moe_runs_kernel<<<1, PLAN_THREADS, 0, stream>>>(counts, experts, max_tiles, tile, starts, tile_expert);
-    moe_place_kernel<<<experts, PLAN_THREADS, 0, stream>>>(chosen, (int)n_pairs, starts, slot_pair, pair_slot);
+    moe_plan_kernel<<<1, PLAN_THREADS, 0, stream>>>(chosen, ids, vocab, top, (int)n_pairs, experts, max_tiles, tile, tile_expert, slot_pair, pair_slot);
+    const int combine_threads = width >= 2048 ? 256 : 128;
     const ExpertCap cap{limit, slope, shift};
     if (tile == TILE_ROWS) {
         auto blocks = [&](int feature_tiles) { return dim3((max_tiles * feature_tiles + TILE_DIES - 1) / TILE_DIES * TILE_DIES); };
@@ -368,7 +368,7 @@ PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gat
 #undef MOE_TILE_UP
         moe_tile_kernel<0><<<blocks(down_tiles), TILE_WAVES * WAVE, 0, stream>>>((const bf16_t*)mid, nullptr, top, (const bf16_t*)down, tile_expert,
                                                                                  max_tiles, down_tiles, width, ff, cap, (bf16_t*)y);
-        moe_combine_kernel<<<n_tokens, 256, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, (const bf16_t*)add0, (const bf16_t*)add1, out);
+        moe_combine_kernel<<<n_tokens, combine_threads, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, (const bf16_t*)add0, (const bf16_t*)add1, out);
         PALM_LAUNCHED();
         return 0;
     }
@@ -382,7 +382,7 @@ PALM_API int palm_moe_grouped(hipStream_t stream, const void* h, const void* gat
 #undef MOE_UP
     moe_grouped_kernel<0><<<dim3(max_tiles, (width + GT_FEATURES - 1) / GT_FEATURES), GT_WAVES * WAVE, 0, stream>>>(
         (const bf16_t*)mid, nullptr, top, (const bf16_t*)down, tile_expert, width, ff, cap, (bf16_t*)y);
-    moe_combine_kernel<<<n_tokens, 256, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, (const bf16_t*)add0, (const bf16_t*)add1, out);
+    moe_combine_kernel<<<n_tokens, combine_threads, 0, stream>>>((const bf16_t*)y, pair_slot, weight, top, width, (const bf16_t*)add0, (const bf16_t*)add1, out);
     PALM_LAUNCHED();
     return 0;
 }

@@ -836,7 +836,7 @@ _FEEDFORWARD_SIGNATURES = {
     "palm_moe_route_table": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
     "palm_moe_tile_tokens": [c_int, c_int, c_int, c_int],
     "palm_moe_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
-                         c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p],
+                         c_void_p, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int],
     "palm_gather_rows": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
     "palm_scatter_add": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "palm_activation": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_longlong],
@@ -1820,7 +1820,7 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chos
     what = "moe_experts"
     n, width = h.shape
     top = chosen.shape[1]
-    shared_up, shared_down, shared_ff = _few_rows(what, h, gate_up, down, chosen, weight, ff, form, ids, shared)[1:]
+    shared_up, shared_down, shared_ff = _check_experts(what, h, gate_up, down, chosen, weight, ff, form, ids, shared)[1:]
     mid = torch.empty((n, top * ff + shared_ff), dtype=F32, device=h.device)
     out = torch.empty((n, width), dtype=F32, device=h.device)
     library.call(feedforward(), "palm_moe_experts", _stream(), _p(h), _code(h, what), _p(gate_up), _p(down), _code(gate_up, what + " weights"),
@@ -1845,7 +1845,7 @@ def moe_few(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: 
     what = "moe_few"
     n, width = h.shape
     top = chosen.shape[1]
-    experts, shared_up, shared_down, shared_ff = _few_rows(what, h, gate_up, down, chosen, weight, ff, form, ids, shared)
+    experts, shared_up, shared_down, shared_ff = _check_experts(what, h, gate_up, down, chosen, weight, ff, form, ids, shared)
     _need(moe_few_serves(h, gate_up, ff, experts, top, shared), f"{what}: at most {FEW_ROWS} bfloat16 rows, bfloat16 weights, sizes in multiples of eight")
     planes = feedforward().palm_moe_few_planes(width) if planes_ok else 1
     mid = torch.empty((n, top * ff + shared_ff), dtype=BF16, device=h.device)
@@ -1856,8 +1856,8 @@ def moe_few(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: 
     return out if planes > 1 else out[0]
 
 
-def _few_rows(what: str, h, gate_up, down, chosen, weight, ff: int, form: str, ids, shared):
-    """The checks of both kernels for few rows: (experts, the shared expert's matrices and inner size)."""
+def _check_experts(what: str, h, gate_up, down, chosen, weight, ff: int, form: str, ids, shared):
+    """The checks that the experts' kernels share: (experts, the shared expert's matrices and inner size)."""
     _dev(what, h, gate_up, down, chosen, weight, ids)
     _i32(what, chosen, ids)
     n, width = h.shape
@@ -1882,29 +1882,26 @@ def moe_grouped_serves(h: torch.Tensor, gate_up: torch.Tensor, ff: int) -> bool:
     return h.dtype == BF16 and gate_up.dtype == BF16 and h.shape[1] % 8 == 0 and ff % 8 == 0
 
 
-def moe_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, ff: int,
-                form: str = "gated_silu", cap=NO_CAP, add=()) -> torch.Tensor:
+def moe_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor | None, ff: int,
+                form: str = "gated_silu", cap=NO_CAP, add=(), ids: torch.Tensor | None = None) -> torch.Tensor:
     """Every row through its chosen experts, for many rows, planned on the device: the (row, choice) pairs grouped by expert,
     two grouped products on the matrix cores, the weighted sum in the order of the choices.  Shapes as ``moe_experts``;
     returns float32 [n, width]."""
     what = "moe_grouped"
-    _dev(what, h, gate_up, down, chosen, weight)
-    _i32(what, chosen)
     n, width = h.shape
     top = chosen.shape[1]
-    _need(moe_grouped_serves(h, gate_up, ff), f"{what}: bfloat16 rows and weights, sizes in multiples of eight")
-    experts = _expert_shapes(what, h, gate_up, down, ff, form)
-    _need(down.dtype == BF16, f"{what}: bfloat16 weights")
-    _need(chosen.shape == (n, top) and weight.shape == (n, top) and weight.dtype == F32, f"{what}: choices {tuple(chosen.shape)}, weights {tuple(weight.shape)}")
+    experts = _check_experts(what, h, gate_up, down, chosen, weight, ff, form, ids, None)[0]
+    _need(moe_grouped_serves(h, gate_up, ff) and down.dtype == BF16, f"{what}: bfloat16 rows and weights, sizes in multiples of eight")
     tile = feedforward().palm_moe_tile_tokens(n * top, experts, width, ff)
     max_tiles = (n * top + tile - 1) // tile + experts
     slots = max_tiles * tile
-    plan = torch.empty((2 * experts + 1 + max_tiles + slots + n * top,), dtype=torch.int32, device=h.device)
+    plan = torch.empty((max_tiles + slots + n * top,), dtype=torch.int32, device=h.device)
     mid = torch.empty((slots, ff), dtype=BF16, device=h.device)
     y = torch.empty((slots, width), dtype=BF16, device=h.device)
     out = torch.empty((n, width), dtype=F32, device=h.device)
     library.call(feedforward(), "palm_moe_grouped", _stream(), _p(h), _p(gate_up), _p(down), _p(chosen), _p(weight), n, top, experts, width, ff,
-                 _p(plan), _p(mid), _p(y), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h))
+                 _p(plan), _p(mid), _p(y), _p(out), EXPERT_FORMS[form], *(float(c) for c in cap), *_addends(what, add, h), _p(ids),
+                 chosen.shape[0] if ids is not None else 0)
     return out
 
 

@@ -314,5 +314,7 @@ class RoutedTableFeedForward(RoutedExperts):
             add.append(down(ops.activation(up(h), ops.PLAIN_EXPERTS[self.form])))
         if n <= self.DIRECT_ROWS:
             return self.run_few(h, self.table, None, add, ids=ctx.token_ids, shared=shared if rides else None, planes_ok=planes_ok)
+        if ops.moe_grouped_serves(h, self.first, self.inter):
+            return ops.moe_grouped(h, self.first, self.down_all, self.table, None, self.inter, self.form, self.cap, add, ids=ctx.token_ids)
         chosen, weight = ops.moe_route_table(ctx.token_ids, self.table)
         return self.run_experts(h, chosen, weight, add)
