@@ -1,13 +1,15 @@
 // Routed experts for few rows (a decode step's batch) in bfloat16 on the matrix cores.  Every expert that somebody chose has its
 // matrices read once, whatever the number of rows that chose it; nothing is planned on the host and no launch of its own plans.
 //
-//   up     a block per (expert, run of matrix rows): the block finds the rows that chose its expert (none: it is done), and
-//          two waves, half the inner size each, stream 16 rows of the expert's first matrix (gated forms: 16 gate rows and their
-//          16 up rows) past them, 16 rows of activations a column tile, and add their sums through LDS; mid[t, c, f] = act(..) in bfloat16, t's choices one after the other, the shared
+//   up     a block per (expert, run of matrix rows): the block finds the rows that chose its expert (none: it is done) and
+//          brings their activations into LDS, and each wave streams 16 rows of the expert's first matrix (gated forms: 16 gate
+//          rows and their 16 up rows) past them, 16 rows of activations a column tile; mid[t, c, f] = act(..) in bfloat16, t's choices one after the other, the shared
 //          expert's values behind them
 //   down   a block per (16 output features, plane): all (row, choice) pairs are sorted by expert in LDS; pieces of 256 inner
 //          values of the experts in use are dealt to the planes' waves in turn; a piece's products go, weighted, into the wave's
 //          own sums [row, 16 features] in LDS, and the waves' sums are added in their order
+//
+// Both kernels are made for up to 16 rows (one column tile) and for more (up to four that share every matrix fragment).
 //
 // A shared expert that every row goes through (weight one, an inner size of its own) runs as one more expert.  Result: float32
 // planes [planes, n, width] for a reader that adds them, the first with the rows of other branches.
@@ -15,10 +17,10 @@
 #include "expert_form.h"
 
 constexpr int FEW_ROWS = 128;                     // rows of a step at most
-constexpr int FEW_UP_WAVES = 4;                   // runs of 16 matrix rows a block, two waves each
+constexpr int FEW_UP_WAVES = 4;
 constexpr int FEW_DOWN_WAVES = 8;
-constexpr int FEW_PIECE = 256;                    // inner values of a piece
 constexpr int FEW_STEPS = 8;                      // reads of 32 values of every matrix row under way together
+constexpr int FEW_PIECE = 32 * FEW_STEPS;         // inner values of a piece
 constexpr int FEW_MAX_EXPERTS = 512;
 constexpr int FEW_MAX_PAIRS = 4096;
 
@@ -38,104 +40,33 @@ __device__ inline bf16x8 few_row8(const bf16_t* row, int col, int dim) {
     return col < dim ? v : zero_bf16x8();
 }
 
-// acc[i][ct] += (16 rows of matrix i) x (16 rows of activations in column tile ct) over k0 .. k1 (in steps of eight): lane (r, g) reads row r of each,
-// the eight values of group g of every step of 32.  wr: this lane's matrix rows; xr: its activation rows.
-template <int MATS, int CT>
-__device__ inline void few_products(const bf16_t* const (&wr)[MATS], const bf16_t* const (&xr)[CT], int k0, int k1, int g,
-                                    f32x4 (&acc)[MATS][CT]) {
-    bf16x8 wf[MATS][FEW_STEPS];
+// acc[ct] += (16 matrix rows) x (16 rows of activations in column tile ct) over one piece k0 .. k1: lane (r, g) reads row r of each, the
+// eight values of group g of every step of 32.  w_row: this lane's matrix row; xr: its activation rows.
+template <int CT>
+__device__ inline void few_piece(const bf16_t* w_row, const bf16_t* const (&xr)[CT], int k0, int k1, int g, f32x4 (&acc)[CT]) {
+    bf16x8 wf[FEW_STEPS];
 #pragma unroll
-    for (int m = 0; m < MATS; ++m)
+    for (int s = 0; s < FEW_STEPS; ++s) wf[s] = few_row8(w_row, k0 + 32 * s + 8 * g, k1);
 #pragma unroll
-        for (int s = 0; s < FEW_STEPS; ++s) wf[m][s] = few_row8(wr[m], k0 + 32 * s + 8 * g, k1);
-    for (int k = k0; k < k1; k += 32 * FEW_STEPS) {
-        bf16x8 next[MATS][FEW_STEPS];
-        const bool more = k + 32 * FEW_STEPS < k1;
-        if (more) {
+    for (int s = 0; s < FEW_STEPS; ++s)
 #pragma unroll
-            for (int m = 0; m < MATS; ++m)
-#pragma unroll
-                for (int s = 0; s < FEW_STEPS; ++s) next[m][s] = few_row8(wr[m], k + 32 * (FEW_STEPS + s) + 8 * g, k1);
-        }
-#pragma unroll
-        for (int s = 0; s < FEW_STEPS; ++s)
-#pragma unroll
-            for (int ct = 0; ct < CT; ++ct) {
-                const bf16x8 xf = few_row8(xr[ct], k + 32 * s + 8 * g, k1);
-#pragma unroll
-                for (int m = 0; m < MATS; ++m) acc[m][ct] = mfma_16x16x32(wf[m][s], xf, acc[m][ct]);
-            }
-        if (more) {
-#pragma unroll
-            for (int m = 0; m < MATS; ++m)
-#pragma unroll
-                for (int s = 0; s < FEW_STEPS; ++s) wf[m][s] = next[m][s];
-        }
-    }
+        for (int ct = 0; ct < CT; ++ct) acc[ct] = mfma_16x16x32(wf[s], few_row8(xr[ct], k0 + 32 * s + 8 * g, k1), acc[ct]);
 }
 
-template <bool GATED, int CT>
-__device__ inline void few_up_tile(const bf16_t* __restrict__ h, const bf16_t* __restrict__ w, const int* list, int c0, int m, bool is_shared,
-                                   const FewChoices& ch, int width, int ff, int my_ff, int row_ff, int f0, int r, int g, int form,
-                                   const ExpertCap& cap, int part, f32x4* exchange, bf16_t* __restrict__ mid) {
-    const bf16_t* xr[CT];
-    const bf16_t* wr[GATED ? 2 : 1];
-#pragma unroll
-    for (int ct = 0; ct < CT; ++ct) {
-        const int p = list[min(c0 + 16 * ct + r, m - 1)];             // (a column beyond the last repeats it and is not kept)
-        xr[ct] = h + (size_t)(is_shared ? p : p / ch.top) * width;
-    }
-    wr[0] = w + (size_t)min(f0 + r, my_ff - 1) * width;
-    if constexpr (GATED) wr[1] = wr[0] + (size_t)my_ff * width;
-    f32x4 acc[GATED ? 2 : 1][CT];
-#pragma unroll
-    for (int i = 0; i < (GATED ? 2 : 1); ++i)
-#pragma unroll
-        for (int ct = 0; ct < CT; ++ct) acc[i][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int middle = (width / 2 + 31) / 32 * 32;
-    if (part == 0) few_products<GATED ? 2 : 1, CT>(wr, xr, 0, min(middle, width), g, acc);
-    else if (middle < width) few_products<GATED ? 2 : 1, CT>(wr, xr, middle, width, g, acc);
-    __syncthreads();                                                  // (whoever still reads the exchange is done)
-    if (part == 1) {
-#pragma unroll
-        for (int i = 0; i < (GATED ? 2 : 1); ++i)
-#pragma unroll
-            for (int ct = 0; ct < CT; ++ct) exchange[(i * CT + ct) * WAVE + 16 * g + r] = acc[i][ct];
-    }
-    __syncthreads();
-    if (part == 1) return;
-#pragma unroll
-    for (int i = 0; i < (GATED ? 2 : 1); ++i)
-#pragma unroll
-        for (int ct = 0; ct < CT; ++ct) {
-            const f32x4 other = exchange[(i * CT + ct) * WAVE + 16 * g + r];
-#pragma unroll
-            for (int k = 0; k < 4; ++k) acc[i][ct][k] += other[k];
-        }
-    // lane (r, g) holds inner values f0 + 4 g + i of column r
-#pragma unroll
-    for (int ct = 0; ct < CT; ++ct) {
-        const int col = c0 + 16 * ct + r, f = f0 + 4 * g;
-        if (col >= m || f >= my_ff) continue;
-        const int p = list[col];
-        bf16_t v[4];
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            if constexpr (GATED) v[i] = f32_to_bf16(form == EXPERT_CAPPED ? expert_capped(acc[0][ct][i], acc[1][ct][i], cap) : expert_silu_gated(acc[0][ct][i], acc[1][ct][i]));
-            else v[i] = f32_to_bf16(expert_plain(form, acc[0][ct][i]));
-        }
-        bf16_t* to = mid + (is_shared ? (size_t)p * row_ff + ch.top * ff : (size_t)(p / ch.top) * row_ff + (size_t)(p % ch.top) * ff) + f;
-        *reinterpret_cast<uint2*>(to) = make_uint2((uint32_t)v[0].bits | ((uint32_t)v[1].bits << 16), (uint32_t)v[2].bits | ((uint32_t)v[3].bits << 16));
-    }
-}
+// Activations for the first products: the columns' rows in LDS, a segment of the inner size at a time.
+// (The matrices come in order through one counter of loads: activations read from memory between them would make every wait for
+// them a wait for the rows asked for ahead.)
+constexpr int few_segment(int max_ct) { return max_ct == 1 ? 2048 : 512; }
+constexpr int FEW_PAD = 8;                         // elements between a segment's end and the next row: rows begin in different banks
 
-template <bool GATED>
-__global__ __launch_bounds__(2 * FEW_UP_WAVES * WAVE) void moe_few_up_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ up, FewChoices ch,
+template <bool GATED, int MAX_CT>
+__global__ __launch_bounds__(FEW_UP_WAVES * WAVE) void moe_few_up_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ up, FewChoices ch,
                                                                          int experts, int width, int ff, const bf16_t* __restrict__ shared_up,
                                                                          int shared_ff, int form, ExpertCap cap, bf16_t* __restrict__ mid) {
+    constexpr int MATS = GATED ? 2 : 1, COLS = 16 * MAX_CT;
+    extern __shared__ __attribute__((aligned(16))) bf16_t x_s[];     // [columns][segment + FEW_PAD]
     __shared__ int list_s[FEW_MAX_PAIRS];
     __shared__ int count_s;
-    __shared__ f32x4 exchange_s[FEW_UP_WAVES][(GATED ? 2 : 1) * 4 * WAVE];
     const int e = blockIdx.x;
     const bool is_shared = e == experts;
     const int my_ff = is_shared ? shared_ff : ff, row_ff = ch.top * ff + shared_ff;
@@ -152,15 +83,76 @@ __global__ __launch_bounds__(2 * FEW_UP_WAVES * WAVE) void moe_few_up_kernel(con
     }
     __syncthreads();
     const int m = count_s;
-    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE % FEW_UP_WAVES, part = threadIdx.x / WAVE / FEW_UP_WAVES;
-    const int r = lane % 16, g = lane / 16, f0 = block_f + 16 * wave;   // (rows beyond the matrix: its last one again, not kept)
     if (m == 0) return;
-    const bf16_t* w = is_shared ? shared_up : up + (size_t)e * (GATED ? 2 : 1) * ff * width;
-    for (int c0 = 0; c0 < m;) {
-        const int left = m - c0;
-#define FEW_UP(CT) { few_up_tile<GATED, CT>(h, w, list_s, c0, m, is_shared, ch, width, ff, my_ff, row_ff, f0, r, g, form, cap, part, exchange_s[wave], mid); c0 += 16 * CT; }
-        if (left > 32) FEW_UP(4) else if (left > 16) FEW_UP(2) else FEW_UP(1)
-#undef FEW_UP
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
+    const int r = lane % 16, g = lane / 16, f0 = block_f + 16 * wave;   // (rows beyond the matrix: its last one again, not kept)
+    const bf16_t* w = is_shared ? shared_up : up + (size_t)e * MATS * ff * width;
+    const bf16_t* wr[MATS];
+    wr[0] = w + (size_t)min(f0 + r, my_ff - 1) * width;
+    if constexpr (GATED) wr[1] = wr[0] + (size_t)my_ff * width;
+    const int segment = min(width, few_segment(MAX_CT)), stride = segment + FEW_PAD;
+    for (int c0 = 0; c0 < m; c0 += COLS) {
+        const int cols = min(COLS, m - c0);
+        f32x4 acc[MATS][MAX_CT];
+#pragma unroll
+        for (int i = 0; i < MATS; ++i)
+#pragma unroll
+            for (int ct = 0; ct < MAX_CT; ++ct) acc[i][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int k0 = 0; k0 < width; k0 += segment) {
+            const int k1 = min(width, k0 + segment), len = k1 - k0;
+            // the first chunk's matrix rows are on their way while the activations go to LDS
+            constexpr int CHUNK = 32 * FEW_STEPS;
+            bf16x8 wf[MATS][FEW_STEPS];
+            auto read = [&](int k, bf16x8 (&to)[MATS][FEW_STEPS]) {
+#pragma unroll
+                for (int i = 0; i < MATS; ++i)
+#pragma unroll
+                    for (int s = 0; s < FEW_STEPS; ++s) to[i][s] = load_bf16x8(wr[i] + min(k + 32 * s + 8 * g, k1 - 8));   // (beyond the end: met by zeros)
+            };
+            read(k0, wf);
+            __syncthreads();                                         // (whoever still reads the segment before is done)
+            for (int i = threadIdx.x; i < cols * (len / 8); i += blockDim.x) {
+                const int col = i / (len / 8), d = i % (len / 8) * 8;
+                const int p = list_s[c0 + col];
+                *reinterpret_cast<uint4*>(x_s + (size_t)col * stride + d) = *reinterpret_cast<const uint4*>(h + (size_t)(is_shared ? p : p / ch.top) * width + k0 + d);
+            }
+            __syncthreads();
+            for (int k = k0; k < k1; k += CHUNK) {
+                bf16x8 next[MATS][FEW_STEPS];
+                read(min(k + CHUNK, k1 - 8), next);                  // (after the last chunk: its end once more, not used)
+#pragma unroll
+                for (int s = 0; s < FEW_STEPS; ++s) {
+                    const int d = k - k0 + 32 * s + 8 * g;
+#pragma unroll
+                    for (int ct = 0; ct < MAX_CT; ++ct) {
+                        if (16 * ct >= cols) continue;               // (the same in every lane)
+                        bf16x8 x = *reinterpret_cast<const bf16x8*>(x_s + (size_t)min(16 * ct + r, cols - 1) * stride + min(d, len - 8));
+                        if (d >= len) x = zero_bf16x8();
+#pragma unroll
+                        for (int i = 0; i < MATS; ++i) acc[i][ct] = mfma_16x16x32(wf[i][s], x, acc[i][ct]);
+                    }
+                }
+#pragma unroll
+                for (int i = 0; i < MATS; ++i)
+#pragma unroll
+                    for (int s = 0; s < FEW_STEPS; ++s) wf[i][s] = next[i][s];
+            }
+        }
+        // lane (r, g) holds inner values f0 + 4 g + i of column r
+#pragma unroll
+        for (int ct = 0; ct < MAX_CT; ++ct) {
+            const int col = 16 * ct + r, f = f0 + 4 * g;
+            if (col >= cols || f >= my_ff) continue;
+            const int p = list_s[c0 + col];
+            bf16_t v[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if constexpr (GATED) v[i] = f32_to_bf16(form == EXPERT_CAPPED ? expert_capped(acc[0][ct][i], acc[1][ct][i], cap) : expert_silu_gated(acc[0][ct][i], acc[1][ct][i]));
+                else v[i] = f32_to_bf16(expert_plain(form, acc[0][ct][i]));
+            }
+            bf16_t* to = mid + (is_shared ? (size_t)p * row_ff + ch.top * ff : (size_t)(p / ch.top) * row_ff + (size_t)(p % ch.top) * ff) + f;
+            *reinterpret_cast<uint2*>(to) = make_uint2((uint32_t)v[0].bits | ((uint32_t)v[1].bits << 16), (uint32_t)v[2].bits | ((uint32_t)v[3].bits << 16));
+        }
     }
 }
 
@@ -178,23 +170,23 @@ __device__ inline void few_down_tile(const bf16_t* __restrict__ mid, const bf16_
         weight[ct] = is_shared ? 1.0f : ch.weight ? ch.weight[p] : 1.0f / (float)ch.top;
         xr[ct] = mid + (size_t)token[ct] * row_ff + (is_shared ? ch.top * ff : (p % ch.top) * ff);
     }
-    const bf16_t* wr[1] = {w_row};
-    f32x4 acc[1][CT];
+    f32x4 acc[CT];
 #pragma unroll
-    for (int ct = 0; ct < CT; ++ct) acc[0][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
-    few_products<1, CT>(wr, xr, k0, k1, g, acc);
+    for (int ct = 0; ct < CT; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
+    few_piece<CT>(w_row, xr, k0, k1, g, acc);
     // lane (r, g) holds features 4 g + i of column r; the columns of a tile are different rows
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
         if (c0 + 16 * ct + r >= m) continue;
         float4* to = reinterpret_cast<float4*>(sums + token[ct] * 16 + 4 * g);
         float4 v = *to;
-        v.x = fmaf(weight[ct], acc[0][ct][0], v.x); v.y = fmaf(weight[ct], acc[0][ct][1], v.y);
-        v.z = fmaf(weight[ct], acc[0][ct][2], v.z); v.w = fmaf(weight[ct], acc[0][ct][3], v.w);
+        v.x = fmaf(weight[ct], acc[ct][0], v.x); v.y = fmaf(weight[ct], acc[ct][1], v.y);
+        v.z = fmaf(weight[ct], acc[ct][2], v.z); v.w = fmaf(weight[ct], acc[ct][3], v.w);
         *to = v;
     }
 }
 
+template <int MAX_CT>
 __global__ __launch_bounds__(FEW_DOWN_WAVES * WAVE) void moe_few_down_kernel(const bf16_t* __restrict__ mid, const bf16_t* __restrict__ down,
                                                                              FewChoices ch, int experts, int width, int ff,
                                                                              const bf16_t* __restrict__ shared_down, int shared_ff,
@@ -260,7 +252,7 @@ __global__ __launch_bounds__(FEW_DOWN_WAVES * WAVE) void moe_few_down_kernel(con
         for (int c0 = 0; c0 < m;) {
             const int left = m - c0;
 #define FEW_DOWN(CT) { few_down_tile<CT>(mid, w_row, sorted + first, c0, m, is_shared, ch, ff, row_ff, k0, k1, r, g, mine); c0 += 16 * CT; }
-            if (left > 32) FEW_DOWN(4) else if (left > 16) FEW_DOWN(2) else FEW_DOWN(1)
+            if constexpr (MAX_CT == 1) FEW_DOWN(1) else if (left > 32) FEW_DOWN(4) else if (left > 16) FEW_DOWN(2) else FEW_DOWN(1)
 #undef FEW_DOWN
         }
     }
@@ -307,14 +299,21 @@ PALM_API int palm_moe_few(hipStream_t stream, const void* h, const void* up, con
     const int longest = max(ff, shared_ff), runs = (longest + 16 * FEW_UP_WAVES - 1) / (16 * FEW_UP_WAVES);
     PALM_CHECK(runs <= 65535, "moe_few: an inner size of %d is more than one launch takes", longest);
     const dim3 grid(experts + (shared_ff > 0), runs);
-#define FEW_LAUNCH(GATED) moe_few_up_kernel<GATED><<<grid, 2 * FEW_UP_WAVES * WAVE, 0, stream>>>((const bf16_t*)h, (const bf16_t*)up, ch, experts, width, ff, \
-        (const bf16_t*)shared_up, shared_ff, form, cap, (bf16_t*)mid)
-    if (expert_is_gated(form)) FEW_LAUNCH(true); else FEW_LAUNCH(false);
+#define FEW_LAUNCH(GATED, MAX_CT) moe_few_up_kernel<GATED, MAX_CT><<<grid, FEW_UP_WAVES * WAVE, \
+        (size_t)min(n_tokens, 16 * MAX_CT) * (min(width, few_segment(MAX_CT)) + FEW_PAD) * sizeof(bf16_t), stream>>>( \
+        (const bf16_t*)h, (const bf16_t*)up, ch, experts, width, ff, (const bf16_t*)shared_up, shared_ff, form, cap, (bf16_t*)mid)
+    if (n_tokens <= 16) {
+        if (expert_is_gated(form)) FEW_LAUNCH(true, 1); else FEW_LAUNCH(false, 1);
+    } else {
+        if (expert_is_gated(form)) FEW_LAUNCH(true, 4); else FEW_LAUNCH(false, 4);
+    }
 #undef FEW_LAUNCH
     const size_t lds = (size_t)FEW_DOWN_WAVES * n_tokens * 16 * sizeof(float) + (size_t)n_tokens * top * sizeof(int);
-    moe_few_down_kernel<<<dim3((width + 15) / 16, planes), FEW_DOWN_WAVES * WAVE, lds, stream>>>(
-        (const bf16_t*)mid, (const bf16_t*)down, ch, experts, width, ff, (const bf16_t*)shared_down, shared_ff, (const bf16_t*)add0,
-        (const bf16_t*)add1, out);
+#define FEW_LAUNCH(MAX_CT) moe_few_down_kernel<MAX_CT><<<dim3((width + 15) / 16, planes), FEW_DOWN_WAVES * WAVE, lds, stream>>>( \
+        (const bf16_t*)mid, (const bf16_t*)down, ch, experts, width, ff, (const bf16_t*)shared_down, shared_ff, (const bf16_t*)add0, \
+        (const bf16_t*)add1, out)
+    if (n_tokens <= 16) FEW_LAUNCH(1); else FEW_LAUNCH(4);
+#undef FEW_LAUNCH
     PALM_LAUNCHED();
     return 0;
 }
