@@ -314,7 +314,7 @@ __global__ __launch_bounds__(LD_WAVES * WAVE) void latent_attention_decode_kerne
         const bf16_t* vp = rows_t + (size_t)pages_t[pg] * kv_rank * PAGE_TOKENS;
         bf16x8 kf[KK];
 #pragma unroll
-        for (int kk = 0; kk < KK; ++kk) kf[kk] = load_row8(kp, kk * 32 + g * 8, dk);
+        for (int kk = 0; kk < KK; ++kk) kf[kk] = load_bf16x8(kp + min(kk * 32 + g * 8, dk - 8));    // (columns beyond the row meet zeros of the query)
         bf16x8 vf[LD_TILES][2];
 #pragma unroll
         for (int i = 0; i < LD_TILES; ++i) {
