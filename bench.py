@@ -385,6 +385,8 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
             else:
                 row = m["kv_rank"] + m["rot_dim"]
                 out["palm_latent_attention_mfma"] = (2.0 * m["heads"] * ((row + m["kv_rank"]) * seen + tokens * m["kv_rank"] * m["vdim"]), mfma, None, None)
+                # (long prompts: keys and values expanded, by the library's products)
+                out["palm_sink_attention_rows_mfma"] = (2.0 * m["heads"] * (m["dim"] + m["rot_dim"] + m["vdim"]) * seen, mfma, None, None)
                 # a decode step reads the rows of the sequences and (it applies them) the value matrices once
                 out["palm_latent_attention_decode"] = (None, None, 2.0 * (batch * min(context, w) * row + m["heads"] * m["vdim"] * m["kv_rank"]), hbm)
             if f:                                                          # plain experts: two matrices each; a decode step's launch has the shared one too
@@ -415,6 +417,7 @@ def _mixer_rooflines(raw: dict, tokens: int, batch: int, context: int) -> dict:
                 flops = 2.0 * m["heads"] * (row + m["kv_rank"]) * seen
                 out["palm_latent_attention"] = (flops, mfma, 2.0 * batch * min(context, w) * row, hbm)
                 out["palm_latent_attention_decode"] = (None, None, 2.0 * (batch * min(context, w) * row + m["heads"] * m["vdim"] * m["kv_rank"]), hbm)
+                out["palm_sink_attention_rows_mfma"] = (2.0 * m["heads"] * (m["dim"] + m["rot_dim"] + m["vdim"]) * seen, mfma, None, None)
                 # the prompt kernel also applies the value matrices
                 out["palm_latent_attention_mfma"] = (flops + 2.0 * tokens * m["heads"] * m["kv_rank"] * m["vdim"], mfma, None, None)
             elif layer["type"] == "parallel" and "palm_sink_attention" not in out:

@@ -653,3 +653,5 @@ PALM_API int palm_latent_output(hipStream_t stream, const float* o_lat, const vo
     PALM_LAUNCHED();
     return 0;
 }
+
+PALM_DEFINE_LAST_ERROR()

@@ -16,16 +16,17 @@ Libraries:
                         value sizes up to 16 V
   ``branches``          branch outputs scaled by a learned vector into the residual stream; the capped feed-forward gate
   ``mixers``            the other mixers beside softmax attention over equal key and value sizes (the selective
-                        scan and its convolution, differential attention, the delta rule, attention over compressed
-                        rows), and the stream of blocks that norm a branch's output; loaded when a model has such a part
+                        scan and its convolution, differential attention, the delta rule), and the stream of blocks that
+                        norm a branch's output; loaded when a model has such a part
+  ``latent``            attention over compressed rows: what lies around it, and the exact kernel
   ``feedforward``       routed experts (routing by softmax or by scores in groups, experts gated or plain) and the
                         activations of plain feed-forwards
   ``gla_d<N>``          gated linear attention (a decay for every key channel and token), compiled for key sizes up to N
   ``delta_head_d<N>``   the delta rule with one decay a head behind short convolutions, compiled for key sizes up to N
   ``streams``           a residual stream in several copies with learned weights between them, and its norms
   ``mlstm``             a matrix memory with input and forget gates per head and token
-  ``latent_attention_k<K>_v<V>``  attention over compressed rows for prompts on the matrix cores, compiled for rows up to
-                        32 K and latents up to 16 V
+  ``latent_attention_k<K>_v<V>``  attention over compressed rows on the matrix cores, compiled for rows up to 32 K and
+                        latents up to 16 V
   ``attention_diff_k<K>_v<V>_q<Q>``  differential attention for prompts on the matrix cores, compiled for key sizes up to
                         32 K, value sizes up to 16 V and Q tiles of 16 queries a wave
 """
@@ -60,8 +61,8 @@ CORE_SOURCES = ["elementwise.hip", "linear.hip", "rope_store.hip", "attention_si
 ATTENTION_SOURCES = ["attention_mfma.hip"]
 DIFF_ATTENTION_SOURCES = ["attention_diff_mfma.hip"]
 LATENT_ATTENTION_SOURCES = ["latent_attention_mfma.hip"]
-MIXER_SOURCES = ["stream.hip", "mamba.hip", "attention_diff.hip", "residual_scaled.hip", "delta_rule.hip",
-                 "latent_attention.hip"]
+MIXER_SOURCES = ["stream.hip", "mamba.hip", "attention_diff.hip", "residual_scaled.hip", "delta_rule.hip"]
+LATENT_SOURCES = ["latent_attention.hip"]
 FEEDFORWARD_SOURCES = ["moe.hip", "moe_few.hip", "moe_grouped.hip", "activation.hip"]
 STREAMS_SOURCES = ["streams.hip"]
 MLSTM_SOURCES = ["mlstm.hip"]
@@ -209,6 +210,8 @@ def _spec(name: str):
         return CORE_SOURCES, ()
     if name == "mixers":
         return MIXER_SOURCES, ()
+    if name == "latent":
+        return LATENT_SOURCES, ()
     if name == "recurrent":
         return RECURRENT_SOURCES, ()
     if name == "sink_attention":

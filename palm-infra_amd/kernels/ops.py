@@ -780,19 +780,6 @@ _MIXER_SIGNATURES = {
     "palm_delta_rule": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int,
                         c_void_p, c_void_p, c_void_p, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                         c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p],
-    "palm_latent_prep": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p,
-                         c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int],
-    "palm_latent_query": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                          c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
-    "palm_latent_query_mfma": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
-                               c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
-    "palm_latent_turn": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
-                         c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
-    "palm_latent_gather": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
-                           c_void_p, c_void_p],
-    "palm_latent_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                              c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p],
-    "palm_latent_output": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
 }
 _mixers = None
 
@@ -809,6 +796,21 @@ def mixers():
     return _mixers
 
 
+_LATENT_SIGNATURES = {
+    "palm_latent_prep": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p,
+                         c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int],
+    "palm_latent_query": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                          c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
+    "palm_latent_query_mfma": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
+                               c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
+    "palm_latent_turn": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p,
+                         c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
+    "palm_latent_gather": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                           c_void_p, c_void_p],
+    "palm_latent_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                              c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p],
+    "palm_latent_output": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+}
 _RECURRENT_SIGNATURES = {
     "palm_retention": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p,
                        c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int,
@@ -882,6 +884,10 @@ def _small(name: str, signatures: dict):
             fn.argtypes, fn.restype = argtypes, c_int
         _small_libraries[name] = lib
     return lib
+
+
+def latent_lib():
+    return _small("latent", _LATENT_SIGNATURES)
 
 
 def recurrent():
@@ -1373,7 +1379,7 @@ def latent_prep(down: torch.Tensor, q_rank: int, kv_off: int, kv_rank: int, rot_
     _need(q_norm_w.shape == (q_rank,) and q_norm_w.dtype == F32, f"{what}: the query norm's weight is float32 [{q_rank}]")
     _latent_rotation(what, cos, sin, n, rot_dim)
     cq = torch.empty((n, q_rank), dtype=down.dtype, device=down.device)
-    library.call(mixers(), "palm_latent_prep", _stream(), _p(down), _code(down, what), down.shape[1], q_rank, kv_off, kv_rank, rot_dim,
+    library.call(latent_lib(), "palm_latent_prep", _stream(), _p(down), _code(down, what), down.shape[1], q_rank, kv_off, kv_rank, rot_dim,
                  _p(q_norm_w), _p(kv_norm_w), float(eps), _p(cos), _p(sin), _p(ctx.positions), _p(ctx.tok_slot), _p(block_table),
                  block_table.shape[1], _p(rows_cache), int(write_cache), _p(cq), n, _p(rows_t), _p(table_t), ROTARY_PAIRINGS[pairing])
     return cq
@@ -1439,10 +1445,10 @@ def latent_query(q: torch.Tensor, uk: torch.Tensor, cos, sin, heads: int, dim: i
     if uk_t is not None and q.dtype == BF16 and rot_dim % 8 == 0 and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0:
         _dev(what, uk_t)
         _need(uk_t.shape == (heads, kv_rank, dim) and uk_t.dtype == BF16, f"{what}: transposed key matrices {tuple(uk_t.shape)} {uk_t.dtype}")
-        library.call(mixers(), "palm_latent_query_mfma", _stream(), _p(q), q.stride(0), _p(uk_t), _p(cos), _p(sin), n, heads, dim, rot_dim, kv_rank,
+        library.call(latent_lib(), "palm_latent_query_mfma", _stream(), _p(q), q.stride(0), _p(uk_t), _p(cos), _p(sin), n, heads, dim, rot_dim, kv_rank,
                      ROTARY_PAIRINGS[pairing], _p(qa), *keep)
         return qa
-    library.call(mixers(), "palm_latent_query", _stream(), _p(q), _code(q, what), q.stride(0), _p(uk), _code(uk, what + " key matrix"), _p(cos), _p(sin),
+    library.call(latent_lib(), "palm_latent_query", _stream(), _p(q), _code(q, what), q.stride(0), _p(uk), _code(uk, what + " key matrix"), _p(cos), _p(sin),
                  n, heads, dim, rot_dim, kv_rank, ROTARY_PAIRINGS[pairing], _p(qa), *keep)
     return qa
 
@@ -1529,11 +1535,11 @@ def latent_attention_expanded(q: torch.Tensor, uk: torch.Tensor, uv: torch.Tenso
     page0, seq_of, page_of, n_pages = ctx.memo[key]
     positions = n_pages * PAGE_TOKENS
     turned = torch.empty((n, heads, dim + rot_dim), dtype=BF16, device=q.device)
-    library.call(mixers(), "palm_latent_turn", _stream(), _p(q), _CODES[BF16], q.stride(0), _p(cos), _p(sin), n, heads, dim, rot_dim, kv_rank,
+    library.call(latent_lib(), "palm_latent_turn", _stream(), _p(q), _CODES[BF16], q.stride(0), _p(cos), _p(sin), n, heads, dim, rot_dim, kv_rank,
                  ROTARY_PAIRINGS[pairing], _p(turned), *_latent_store(what, store, q, kv_rank, rot_dim, ctx, pairing))
     c = torch.empty((positions, kv_rank), dtype=BF16, device=q.device)
     k2 = torch.empty((positions, rot_dim), dtype=BF16, device=q.device)
-    library.call(mixers(), "palm_latent_gather", _stream(), _p(rows_cache), _CODES[BF16], _p(block_table), block_table.shape[1], _p(ctx.seq_slot),
+    library.call(latent_lib(), "palm_latent_gather", _stream(), _p(rows_cache), _CODES[BF16], _p(block_table), block_table.shape[1], _p(ctx.seq_slot),
                  _p(ctx.seq_start), _p(ctx.seq_new), _p(seq_of), _p(page_of), n_pages, kv_rank, rot_dim, _p(c), _p(k2))
     keys = linear_library(c, uk)                 # [positions, heads * dim]
     values = linear_library(uv, c)               # [heads * vdim, positions]: positions innermost, as the kernel reads values
@@ -1597,7 +1603,7 @@ def latent_attention(qa: torch.Tensor, rows_cache: torch.Tensor, block_table: to
                      _p(block_table), _p(table_t), block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new),
                      ctx.n_seqs, int(ctx.max_new), heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(sink), _p(out), None, None, 0, 0, None)
         return out
-    library.call(mixers(), "palm_latent_attention", _stream(), _p(qa), _p(rows_cache), _code(rows_cache, what), _p(block_table),
+    library.call(latent_lib(), "palm_latent_attention", _stream(), _p(qa), _p(rows_cache), _code(rows_cache, what), _p(block_table),
                  block_table.shape[1], _p(ctx.seq_slot), _p(ctx.seq_start), _p(ctx.seq_new), _p(ctx.cu_new), ctx.n_seqs, int(ctx.max_new),
                  heads, kv_rank, rot_dim, float(scale), int(window or 0), _p(sink), _p(out))
     return out
@@ -1700,7 +1706,7 @@ def latent_output(o_lat: torch.Tensor, uv: torch.Tensor, gate: torch.Tensor | No
     _need(gate is None or (gate.is_cuda and gate.shape == (n, heads) and gate.dtype == out_dtype and (n == 0 or gate.stride(1) == 1)),
           f"{what}: the gate is {out_dtype} [{n}, {heads}] with contiguous rows")
     out = torch.empty((n, heads * vdim), dtype=out_dtype, device=o_lat.device)
-    library.call(mixers(), "palm_latent_output", _stream(), _p(o_lat), _p(uv), _code(uv, what + " value matrix"), _p(gate),
+    library.call(latent_lib(), "palm_latent_output", _stream(), _p(o_lat), _p(uv), _code(uv, what + " value matrix"), _p(gate),
                  gate.stride(0) if gate is not None else 0, _code(out, what), n, heads, kv_rank, vdim, _p(out))
     return out
 
